@@ -1,6 +1,7 @@
 from .engine_config import EngineConfig, build_engine_config, canonical_dtype
 from .givizen import GivizenConfig
 from .nokipel import NokipelConfig
+from .nopunex import NopunexConfig
 from .polosun import PolosunConfig
 from .qwen2 import Qwen2Config
 from .senuvik import SenuvikConfig
@@ -20,9 +21,10 @@ register_architecture("Polosun", PolosunConfig)
 register_architecture("Givizen", GivizenConfig)
 register_architecture("Nokipel", NokipelConfig)
 register_architecture("Senuvik", SenuvikConfig)
+register_architecture("Nopunex", NopunexConfig)
 
 __all__ = [
     "ARCHITECTURES", "Architecture", "ConfigError", "EngineConfig", "GivizenConfig", "LayerCall", "LayerSpec",
-    "ModelSpec", "NokipelConfig", "PartSpec", "PolosunConfig", "Qwen2Config", "SenuvikConfig", "architecture_of", "build_engine_config",
+    "ModelSpec", "NokipelConfig", "NopunexConfig", "PartSpec", "PolosunConfig", "Qwen2Config", "SenuvikConfig", "architecture_of", "build_engine_config",
     "canonical_dtype", "config_from_dict", "load_config", "register_architecture",
 ]

@@ -74,12 +74,15 @@ class LayerCall:
                unit before reading it.
     ``adds_embedding`` the embedding's rows (scaled, as they entered the stream) join the
                stream once more right in front of this call.
+    ``entry``  the model's entry step (``ModelSpec.entry``) runs right in front of this
+               call, as the entry of that number; ``None``: it does not.
     """
 
     layer: int
     cache: int
     writes: bool = True
     adds_embedding: bool = False
+    entry: int | None = None
 
 
 @dataclass(frozen=True)
@@ -99,6 +102,11 @@ class ModelSpec:
     layer_prefix: str = "model.layers.{index}."
     embedding_scale: float = 1.0          # the embedding's rows are multiplied by this on their way into the stream
     logit_softcap: float | None = None    # logits <- cap * tanh(logits / cap)
+    logit_scale: float = 1.0              # logits <- scale * logits, in front of the cap
+    # what remakes the stream in front of the calls that have an ``entry`` (a part of the role "entry"), and the prefix of
+    # its tensors' names
+    entry: PartSpec | None = None
+    entry_name: str = "entry"
     extra: dict[str, Any] = field(default_factory=dict, compare=False)
 
     def __post_init__(self) -> None:
@@ -108,6 +116,8 @@ class ModelSpec:
                 raise ValueError(f"run order names layer {call.layer}, model has {len(self.layers)}")
             if call.cache < 0:
                 raise ValueError("cache unit indices are non-negative")
+            if call.entry is not None and (self.entry is None or call.entry < 0):
+                raise ValueError(f"layer {call.layer} is run behind entry {call.entry}, and the model has no such step")
             if call.writes:
                 units.setdefault(call.cache, call.layer)
         for call in self.order:

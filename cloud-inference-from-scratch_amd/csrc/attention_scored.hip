@@ -10,7 +10,12 @@
 //   ... or when j <= i and floor(i / chunk) = floor(j / chunk)   chunk > 0: chunks counted from position 0
 //   p_ij = exp(s_ij) / (sum_j exp(s_ij) + exp(sink[head]))   sinks given: one more term in the denominator, which
 //                                                        has no key and no value, no scale and no bias
-//   o_i  = sum_j p_ij v_j,  o_i <- o_i * sigmoid(gate[i, head])   gate given
+//   o_i  = sum_j p_ij v_j,  o_i <- o_i * sigmoid(gate[i, head])   gate given; or, with a gate per number of the head,
+//                                                        o_i[d] <- o_i[d] * sigmoid(gate[i, head * vdim + d])
+//
+// Differential heads (two maps): queries and keys come in pairs, every map is a softmax of its own over the same values,
+// and  o_i = (a1_i - lambda a2_i) / sqrt(mean((a1_i - lambda a2_i)^2) + eps) * factor  over the head's vdim numbers.  A
+// query or key row then holds its two maps one after the other (D numbers in all).
 //
 // Keys have D numbers per head, values DV (the two may differ).  Cache layout as everywhere in this library:
 // keys [pages, kv_heads, page_size, D], values transposed [pages, kv_heads, DV, page_size].  Scores, the softmax,
@@ -70,7 +75,9 @@ __device__ __forceinline__ float wave_sum_squares(const bf16_t* p, int n, int la
     return wave_sum(sum);
 }
 
-// One wave per (token, head slot): slots 0..H-1 queries, H..H+G-1 keys, H+G..H+2G-1 values.
+// One wave per (token, head slot): slots 0..H-1 queries, H..H+G-1 keys, H+G..H+G+V-1 values.  With `maps` > 1 the query and
+// key heads come in runs of that many (the maps of one head), laid side by side in the rows and in the cache; there are
+// V = kv_heads value heads, and H = maps * q_heads, G = maps * kv_heads.
 template <typename T>
 __global__ void __launch_bounds__(256)
 heads_prepare_kernel(const T* __restrict__ proj, int proj_stride, int q_off, int k_off, int v_off,
@@ -80,9 +87,13 @@ heads_prepare_kernel(const T* __restrict__ proj, int proj_stride, int q_off, int
                      const int* __restrict__ block_table, int table_width, T* __restrict__ q_out,
                      T* __restrict__ k_pool, T* __restrict__ v_pool, int tokens, int q_heads, int kv_heads,
                      int dim, int vdim, int D, int DV, int page_shift, int write_kv,
-                     const float* __restrict__ cos_table, const float* __restrict__ sin_table, int rot, int neighbours) {
+                     const float* __restrict__ cos_table, const float* __restrict__ sin_table, int rot, int neighbours,
+                     int maps) {
     const int lane = threadIdx.x % kWave;
-    const int slots = q_heads + 2 * kv_heads;
+    const int value_heads = kv_heads;
+    q_heads *= maps;
+    kv_heads *= maps;
+    const int slots = q_heads + kv_heads + value_heads;
     const long unit = static_cast<long>(blockIdx.x) * (blockDim.x / kWave) + threadIdx.x / kWave;
     if (unit >= static_cast<long>(tokens) * slots) return;
     const int token = static_cast<int>(unit / slots);
@@ -99,7 +110,7 @@ heads_prepare_kernel(const T* __restrict__ proj, int proj_stride, int q_off, int
     if (slot >= q_heads + kv_heads) {  // a value head: copied, padded, into the transposed pool
         const int head = slot - q_heads - kv_heads;
         const T* src = row + v_off + head * vdim;
-        T* dst = v_pool + ((page * kv_heads + head) * DV << page_shift) + (pos & (page_size - 1));
+        T* dst = v_pool + ((page * value_heads + head) * DV << page_shift) + (pos & (page_size - 1));
         for (int d = lane; d < DV; d += kWave)
             dst[static_cast<size_t>(d) << page_shift] = d < vdim ? src[d] : from_float<T>(0.f);
         return;
@@ -127,7 +138,7 @@ heads_prepare_kernel(const T* __restrict__ proj, int proj_stride, int q_off, int
     if (is_q && temp_every > 0)
         after = 1.0f + temp_coef * logf(static_cast<float>((pos + 1) / temp_every) + 1.0f);
     T* dst = is_q ? q_out + (static_cast<size_t>(token) * q_heads + head) * D
-                  : k_pool + (((page * kv_heads + head) << page_shift) + (pos & (page_size - 1))) * D;
+                  : k_pool + ((((page * value_heads + head / maps) << page_shift) + (pos & (page_size - 1))) * maps + head % maps) * D;
     const int half = rot / 2;
     const float* cos_row = rot > 0 ? cos_table + static_cast<size_t>(pos) * half : nullptr;
     const float* sin_row = rot > 0 ? sin_table + static_cast<size_t>(pos) * half : nullptr;
@@ -157,7 +168,9 @@ heads_prepare_kernel(const T* __restrict__ proj, int proj_stride, int q_off, int
 // One workgroup (4 waves) per (query token, query head); each wave takes 64-key chunks in turn, one key per
 // lane for the scores, then one slice of the value head per lane; the four running (max, sum, accumulator)
 // triples meet in LDS.  Any D, DV that are multiples of 8 up to 256; float32 or bfloat16 storage.
-constexpr int kMaxSlices = 4;
+// With `maps` = 2 a query or key row holds two maps of D numbers each; they are walked one after the other.
+constexpr int kMaxSlices = 4;       // pieces of 64 numbers of a value head that a lane keeps ...
+constexpr int kMaxWideSlices = 16;  // ... and in the form for wide values
 
 template <typename T>
 __device__ __forceinline__ void load8(const T* p, float (&v)[8]);
@@ -187,6 +200,11 @@ struct ScoreShape {
     int window;           // <= 0: all keys
     int chunk;            // > 0: i sees j <= i only inside its own chunk, floor(i / chunk) == floor(j / chunk)
     int keep;             // > 0 (with a window): keys 0 .. keep - 1 are seen from behind the window too
+    int gate_wide;        // the gate has a number for every number of the head (head * vdim + d), not one per head
+    int vdim;             // numbers of a value head that are not padding
+    float lambda;         // two maps: the second one's weight ...
+    float factor;         // ... the factor behind the norm of their difference ...
+    float eps;            // ... and that norm's eps
 };
 
 // The first key that the query at position `pos` sees.
@@ -195,19 +213,21 @@ __device__ __forceinline__ int first_seen(int pos, int window, int chunk) {
     return window > 0 ? max(0, pos + 1 - window) : 0;
 }
 
-template <typename T>
+template <typename T, int SLICES>
 __global__ void __launch_bounds__(256)
 scored_attention_generic_kernel(const T* __restrict__ q, const T* __restrict__ k_pool, const T* __restrict__ v_pool,
                                 const int* __restrict__ block_table, int table_width,
                                 const int* __restrict__ positions, const int* __restrict__ seq_of_token,
                                 const int* __restrict__ seq_slot, const T* __restrict__ gate, int gate_stride,
                                 T* __restrict__ out, int q_heads, int kv_heads, int D, int DV, int page_size,
-                                ScoreShape shape) {
+                                int maps, ScoreShape shape) {
     extern __shared__ float lds[];
     float* q_s = lds;            // [D]
     float* acc_s = lds + D;      // [4][DV]
+    float* done_s = acc_s + 4 * DV;  // [maps][DV]
     __shared__ float m_s[4];
     __shared__ float l_s[4];
+    __shared__ float scratch[16];
 
     const int token = blockIdx.x;
     const int head = blockIdx.y;
@@ -220,86 +240,107 @@ scored_attention_generic_kernel(const T* __restrict__ q, const T* __restrict__ k
     const int* table = block_table + static_cast<size_t>(seq_slot[seq_of_token[token]]) * table_width;
     const float slope = shape.slopes ? shape.slopes[head] : 0.f;
 
-    const T* q_row = q + (static_cast<size_t>(token) * q_heads + head) * D;
-    for (int d = threadIdx.x; d < D; d += blockDim.x) q_s[d] = to_float(q_row[d]);
-    __syncthreads();
-
-    float m = -INFINITY;
-    float l = 0.f;
-    float acc[kMaxSlices] = {0.f, 0.f, 0.f, 0.f};
     // the keys in the order they are walked: the kept first ones that lie in front of the window, then the window's
     const int kept = (shape.window > 0 && shape.keep > 0) ? min(shape.keep, lo) : 0;
     const int walk = kept + len - lo;
-    for (int base = wave * kWave; base < walk; base += 4 * kWave) {
-        const int at = base + lane;
-        const int key = at < kept ? at : at - kept + lo;
-        const bool valid = at < walk;
-        float s = -INFINITY;
-        uint32_t head_block = 0;
-        uint32_t in_page = 0;
-        if (valid) {
-            const int page = table[key / page_size];
-            head_block = static_cast<uint32_t>(page) * kv_heads + kv_head;
-            in_page = key % page_size;
-            const T* k_row = k_pool + (static_cast<size_t>(head_block) * page_size + in_page) * D;
-            float dot = 0.f;
-            for (int d = 0; d < D; d += 8) {
-                float kk[8];
-                load8<T>(k_row + d, kk);
+    for (int map = 0; map < maps; ++map) {
+        __syncthreads();  // (the map before has been read out)
+        const T* q_row = q + ((static_cast<size_t>(token) * q_heads + head) * maps + map) * D;
+        for (int d = threadIdx.x; d < D; d += blockDim.x) q_s[d] = to_float(q_row[d]);
+        __syncthreads();
+
+        float m = -INFINITY;
+        float l = 0.f;
+        float acc[SLICES];
 #pragma unroll
-                for (int j = 0; j < 8; ++j) dot = fmaf(q_s[d + j], kk[j], dot);
+        for (int i = 0; i < SLICES; ++i) acc[i] = 0.f;
+        for (int base = wave * kWave; base < walk; base += 4 * kWave) {
+            const int at = base + lane;
+            const int key = at < kept ? at : at - kept + lo;
+            const bool valid = at < walk;
+            float s = -INFINITY;
+            uint32_t head_block = 0;
+            uint32_t in_page = 0;
+            if (valid) {
+                const int page = table[key / page_size];
+                head_block = static_cast<uint32_t>(page) * kv_heads + kv_head;
+                in_page = key % page_size;
+                const T* k_row = k_pool + ((static_cast<size_t>(head_block) * page_size + in_page) * maps + map) * D;
+                float dot = 0.f;
+                for (int d = 0; d < D; d += 8) {
+                    float kk[8];
+                    load8<T>(k_row + d, kk);
+#pragma unroll
+                    for (int j = 0; j < 8; ++j) dot = fmaf(q_s[d + j], kk[j], dot);
+                }
+                s = dot * shape.scale;
+                if (shape.softcap > 0.f) s = shape.softcap * tanhf(s / shape.softcap);
+                s -= slope * static_cast<float>(pos - key);
             }
-            s = dot * shape.scale;
-            if (shape.softcap > 0.f) s = shape.softcap * tanhf(s / shape.softcap);
-            s -= slope * static_cast<float>(pos - key);
-        }
-        const float m_new = fmaxf(m, wave_max(s));  // finite: lane 0 of every chunk is valid
-        const float alpha = expf(m - m_new);
-        const float p = valid ? expf(s - m_new) : 0.f;
-        l = l * alpha + wave_sum(p);
+            const float m_new = fmaxf(m, wave_max(s));  // finite: lane 0 of every chunk is valid
+            const float alpha = expf(m - m_new);
+            const float p = valid ? expf(s - m_new) : 0.f;
+            l = l * alpha + wave_sum(p);
 #pragma unroll
-        for (int i = 0; i < kMaxSlices; ++i) acc[i] *= alpha;
-        const int count = min(kWave, walk - base);
-        for (int j = 0; j < count; ++j) {
-            const float pj = __shfl(p, j, kWave);
-            const uint32_t block_j = __shfl(head_block, j, kWave);
-            const uint32_t in_page_j = __shfl(in_page, j, kWave);
-            const T* v_column = v_pool + static_cast<size_t>(block_j) * page_size * DV + in_page_j;
+            for (int i = 0; i < SLICES; ++i) acc[i] *= alpha;
+            const int count = min(kWave, walk - base);
+            for (int j = 0; j < count; ++j) {
+                const float pj = __shfl(p, j, kWave);
+                const uint32_t block_j = __shfl(head_block, j, kWave);
+                const uint32_t in_page_j = __shfl(in_page, j, kWave);
+                const T* v_column = v_pool + static_cast<size_t>(block_j) * page_size * DV + in_page_j;
 #pragma unroll
-            for (int i = 0; i < kMaxSlices; ++i) {
-                const int d = lane + kWave * i;
-                if (d < DV) acc[i] = fmaf(pj, to_float(v_column[static_cast<size_t>(d) * page_size]), acc[i]);
+                for (int i = 0; i < SLICES; ++i) {
+                    const int d = lane + kWave * i;
+                    if (d < DV) acc[i] = fmaf(pj, to_float(v_column[static_cast<size_t>(d) * page_size]), acc[i]);
+                }
             }
+            m = m_new;
         }
-        m = m_new;
-    }
-    if (lane == 0) {
-        m_s[wave] = m;
-        l_s[wave] = l;
-    }
+        if (lane == 0) {
+            m_s[wave] = m;
+            l_s[wave] = l;
+        }
 #pragma unroll
-    for (int i = 0; i < kMaxSlices; ++i) {
-        const int d = lane + kWave * i;
-        if (d < DV) acc_s[wave * DV + d] = acc[i];
+        for (int i = 0; i < SLICES; ++i) {
+            const int d = lane + kWave * i;
+            if (d < DV) acc_s[wave * DV + d] = acc[i];
+        }
+        __syncthreads();
+        float m_all = m_s[0];
+        for (int w = 1; w < 4; ++w) m_all = fmaxf(m_all, m_s[w]);
+        const float sink = shape.sinks ? shape.sinks[head] : -INFINITY;
+        m_all = fmaxf(m_all, sink);
+        float den = shape.sinks ? expf(sink - m_all) : 0.f;
+        float e[4];
+        for (int w = 0; w < 4; ++w) {
+            e[w] = expf(m_s[w] - m_all);  // a wave that saw no key has m = -inf: weight 0
+            den += l_s[w] * e[w];
+        }
+        for (int d = threadIdx.x; d < DV; d += blockDim.x) {
+            float num = 0.f;
+            for (int w = 0; w < 4; ++w) num += acc_s[w * DV + d] * e[w];
+            done_s[map * DV + d] = num / den;
+        }
     }
-    __syncthreads();
-    float m_all = m_s[0];
-    for (int w = 1; w < 4; ++w) m_all = fmaxf(m_all, m_s[w]);
-    const float sink = shape.sinks ? shape.sinks[head] : -INFINITY;
-    m_all = fmaxf(m_all, sink);
-    float den = shape.sinks ? expf(sink - m_all) : 0.f;
-    float e[4];
-    for (int w = 0; w < 4; ++w) {
-        e[w] = expf(m_s[w] - m_all);  // a wave that saw no key has m = -inf: weight 0
-        den += l_s[w] * e[w];
+    // (a thread reads the numbers of `done_s` that it wrote itself)
+    float by = 1.f;
+    if (maps > 1) {
+        float sum = 0.f;
+        for (int d = threadIdx.x; d < shape.vdim; d += blockDim.x) {
+            const float x = done_s[d] - shape.lambda * done_s[DV + d];
+            done_s[d] = x;
+            sum += x * x;
+        }
+        by = shape.factor / sqrtf(block_sum(sum, scratch) / static_cast<float>(shape.vdim) + shape.eps);
     }
-    float open = 1.f;
-    if (gate) open = 1.0f / (1.0f + expf(-to_float(gate[static_cast<size_t>(token) * gate_stride + head])));
+    const T* gates = gate ? gate + static_cast<size_t>(token) * gate_stride : nullptr;
     T* out_row = out + (static_cast<size_t>(token) * q_heads + head) * DV;
     for (int d = threadIdx.x; d < DV; d += blockDim.x) {
-        float num = 0.f;
-        for (int w = 0; w < 4; ++w) num += acc_s[w * DV + d] * e[w];
-        out_row[d] = from_float<T>(num / den * open);
+        float x = d < shape.vdim ? done_s[d] * by : 0.f;
+        if (gates && d < shape.vdim)
+            x *= 1.0f / (1.0f + expf(-to_float(gates[shape.gate_wide ? head * shape.vdim + d : head])));
+        out_row[d] = from_float<T>(x);
     }
 }
 
@@ -352,11 +393,41 @@ __device__ __forceinline__ float fast_tanh(float y) {
     return 1.f - 2.f * __builtin_amdgcn_rcpf(e + 1.f);
 }
 
-template <int D, int DV, int RT>
-__global__ void __launch_bounds__(64 * kScoredWaves, RT <= 2 ? 2 : 1) scored_attention_mfma_kernel(ScoredArgs a) {
-    constexpr int NK = D / 32;
+// A head's read-out (number d in x[d / 64] of lane d % 64), normed where it is a difference of two maps, gated, stored.
+template <int MAPS, int DV, int N>
+__device__ __forceinline__ void write_head(const ScoredArgs& a, const float (&x)[N], size_t token, int head, int lane) {
+    float factor = 1.f;
+    if (MAPS == 2) {
+        float sum = 0.f;
+#pragma unroll
+        for (int i = 0; i < N; ++i) sum += x[i] * x[i];  // (padding is zero)
+        factor = a.shape.factor / sqrtf(wave_sum(sum) / static_cast<float>(a.shape.vdim) + a.shape.eps);
+    }
+    const bf16_t* gates = a.gate ? a.gate + token * a.gate_stride : nullptr;
+    if (gates && !a.shape.gate_wide) factor *= 1.0f / (1.0f + __expf(-to_float(gates[head])));
+    bf16_t* dst = a.out + (token * a.q_heads + head) * DV;
+#pragma unroll
+    for (int i = 0; i < N; ++i) {
+        const int d = lane + i * kWave;
+        if (d >= DV) continue;
+        float y = x[i] * factor;
+        if (gates && a.shape.gate_wide && d < a.shape.vdim)
+            y *= 1.0f / (1.0f + __expf(-to_float(gates[head * a.shape.vdim + d])));
+        dst[d] = from_float<bf16_t>(y);
+    }
+}
+
+// MAPS = 2: rows of the first map fill the first RT / 2 tiles of 16, the same rows of the second map the others; the two
+// maps of a query or key row lie side by side, D / 2 numbers each.
+template <int D, int DV, int RT, int MAPS>
+__global__ void __launch_bounds__(64 * kScoredWaves, RT * (D / 4 + DV) <= 2 * (32 + 128) ? 2 : 1)
+scored_attention_mfma_kernel(ScoredArgs a) {
+    constexpr int MD = D / MAPS;      // numbers of a map
+    constexpr int NK = MD / 32;
     constexpr int ND = DV / 16;
     constexpr int ROWS = 16 * RT;
+    constexpr int RTM = RT / MAPS;    // tiles of a map
+    constexpr int MROWS = 16 * RTM;   // rows of a map
     constexpr int STEP = kKeysPerBlock * kScoredWaves;
     __shared__ float m_s[kScoredWaves][ROWS];
     __shared__ float l_s[kScoredWaves][ROWS];
@@ -421,13 +492,14 @@ __global__ void __launch_bounds__(64 * kScoredWaves, RT <= 2 ? 2 : 1) scored_att
     float row_slope[RT];  // its head's slope, in base-2 units
 #pragma unroll
     for (int rt = 0; rt < RT; ++rt) {
-        const int row = rt * 16 + r;
+        const int row = (rt % RTM) * 16 + r;
         const bool valid = row < n_rows;
         const int tok = valid ? row / group : 0;
         const int head = kv_head * group + (valid ? row - tok * group : 0);
         row_pos[rt] = valid ? start + q0 + tok : -1;
         row_slope[rt] = a.shape.slopes ? a.shape.slopes[head] * kLog2e : 0.f;
-        const bf16_t* q_row = a.q + (static_cast<size_t>(first_row_token + tok) * a.q_heads + head) * D + g * (D / 4);
+        const bf16_t* q_row = a.q + (static_cast<size_t>(first_row_token + tok) * a.q_heads + head) * D + (rt / RTM) * MD +
+                              g * (MD / 4);
 #pragma unroll
         for (int j = 0; j < NK; ++j)
             qf[rt][j] = valid ? *reinterpret_cast<const uint4*>(q_row + j * 8) : uint4{0, 0, 0, 0};
@@ -457,16 +529,17 @@ __global__ void __launch_bounds__(64 * kScoredWaves, RT <= 2 ? 2 : 1) scored_att
             const int page = table[key >> a.page_shift];
             const bf16_t* k_row = a.k_pool +
                 (((static_cast<size_t>(page) * a.kv_heads + kv_head) << a.page_shift) + (key & page_mask)) * D +
-                g * (D / 4);
-            uint4 kf[NK];
+                g * (MD / 4);
+            uint4 kf[MAPS * NK];
 #pragma unroll
-            for (int j = 0; j < NK; ++j) kf[j] = *reinterpret_cast<const uint4*>(k_row + j * 8);
+            for (int j = 0; j < MAPS * NK; ++j)
+                kf[j] = *reinterpret_cast<const uint4*>(k_row + (j / NK) * MD + (j % NK) * 8);
 #pragma unroll
             for (int rt = 0; rt < RT; ++rt) {
                 floatx4 acc = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
                 for (int j = 0; j < NK; ++j)
-                    acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8, kf[j]),
+                    acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8, kf[(rt / RTM) * NK + j]),
                                                                   __builtin_bit_cast(bf16x8, qf[rt][j]), acc, 0, 0, 0);
                 s[rt][kt] = acc;
             }
@@ -587,7 +660,8 @@ __global__ void __launch_bounds__(64 * kScoredWaves, RT <= 2 ? 2 : 1) scored_att
         const size_t unit = (static_cast<size_t>(tile) * a.kv_heads + kv_head) * a.n_splits + split;
         float* po = a.part_o + unit * ROWS * DV;
         float* pml = a.part_ml + unit * ROWS * 2;
-        for (int row = wave; row < n_rows; row += kScoredWaves) {
+        for (int at = wave; at < n_rows * MAPS; at += kScoredWaves) {
+            const int row = MAPS == 1 ? at : at < n_rows ? at : MROWS + at - n_rows;
             float m_all = m_s[0][row];
 #pragma unroll
             for (int w = 1; w < kScoredWaves; ++w) m_all = fmaxf(m_all, m_s[w][row]);
@@ -608,27 +682,34 @@ __global__ void __launch_bounds__(64 * kScoredWaves, RT <= 2 ? 2 : 1) scored_att
     for (int row = wave; row < n_rows; row += kScoredWaves) {
         const int tok = row / group;
         const int head = kv_head * group + (row - tok * group);
-        float m_all = m_s[0][row];
+        float inverse[MAPS];  // 1 / the denominator of each map
 #pragma unroll
-        for (int w = 1; w < kScoredWaves; ++w) m_all = fmaxf(m_all, m_s[w][row]);
-        float den = 0.f;
-        if (a.shape.sinks) {
-            const float sink = a.shape.sinks[head] * kLog2e;
-            m_all = fmaxf(m_all, sink);
-            den = __builtin_amdgcn_exp2f(sink - m_all);
-        }
+        for (int map = 0; map < MAPS; ++map) {
+            const int at = map * MROWS + row;
+            float m_all = m_s[0][at];
 #pragma unroll
-        for (int w = 0; w < kScoredWaves; ++w) {
-            const float mine = m_s[w][row];
-            den += (mine == -INFINITY) ? 0.f : l_s[w][row] * __builtin_amdgcn_exp2f(mine - m_all);
+            for (int w = 1; w < kScoredWaves; ++w) m_all = fmaxf(m_all, m_s[w][at]);
+            float den = 0.f;
+            if (a.shape.sinks) {
+                const float sink = a.shape.sinks[head] * kLog2e;
+                m_all = fmaxf(m_all, sink);
+                den = __builtin_amdgcn_exp2f(sink - m_all);
+            }
+#pragma unroll
+            for (int w = 0; w < kScoredWaves; ++w) {
+                const float mine = m_s[w][at];
+                den += (mine == -INFINITY) ? 0.f : l_s[w][at] * __builtin_amdgcn_exp2f(mine - m_all);
+            }
+            inverse[map] = 1.0f / den;
         }
-        float factor = 1.0f / den;
-        if (a.gate) {
-            const float z = to_float(a.gate[static_cast<size_t>(first_row_token + tok) * a.gate_stride + head]);
-            factor *= 1.0f / (1.0f + __expf(-z));
+        float x[(DV + kWave - 1) / kWave];
+#pragma unroll
+        for (int i = 0; i < (DV + kWave - 1) / kWave; ++i) {
+            const int d = lane + i * kWave;
+            x[i] = d < DV ? o_s[row][d] * inverse[0] : 0.f;
+            if (MAPS == 2 && d < DV) x[i] -= a.shape.lambda * (o_s[MROWS + row][d] * inverse[MAPS - 1]);
         }
-        bf16_t* dst = a.out + (static_cast<size_t>(first_row_token + tok) * a.q_heads + head) * DV;
-        for (int d = lane; d < DV; d += kWave) dst[d] = from_float<bf16_t>(o_s[row][d] * factor);
+        write_head<MAPS, DV>(a, x, static_cast<size_t>(first_row_token + tok), head, lane);
     }
 }
 
@@ -637,7 +718,9 @@ __global__ void __launch_bounds__(64 * kScoredWaves, RT <= 2 ? 2 : 1) scored_att
 // sums are then fetched without waiting on one another.
 constexpr int kMergeShares = 64;  // shares whose factors one pass keeps in a lane each
 
-__global__ void __launch_bounds__(256) scored_attention_merge_kernel(ScoredArgs a, int rows_per_tile, int DV) {
+template <int DV, int MAPS>
+__global__ void __launch_bounds__(256) scored_attention_merge_kernel(ScoredArgs a, int rows_per_tile) {
+    constexpr int N = (DV + kWave - 1) / kWave;
     const int lane = threadIdx.x & (kWave - 1);
     const int wave = threadIdx.x / kWave;
     const int tile = blockIdx.x;
@@ -653,59 +736,66 @@ __global__ void __launch_bounds__(256) scored_attention_merge_kernel(ScoredArgs 
     const size_t unit0 = (static_cast<size_t>(tile) * a.kv_heads + kv_head) * a.n_splits;
     const int tok = row / group;
     const int head = kv_head * group + (row - tok * group);
-    float m_all = -INFINITY;
-    for (int sp = lane; sp < a.n_splits; sp += kWave)
-        m_all = fmaxf(m_all, a.part_ml[((unit0 + sp) * rows_per_tile + row) * 2]);
-    m_all = wave_max(m_all);
-    float sink_term = 0.f;  // the sink's share of the denominator, counted once
-    if (a.shape.sinks) {
-        const float sink = a.shape.sinks[head] * kLog2e;
-        m_all = fmaxf(m_all, sink);
-        sink_term = __builtin_amdgcn_exp2f(sink - m_all);
-    }
-    float den = 0.f;        // this lane's shares of it
-    float acc[4] = {0.f, 0.f, 0.f, 0.f};  // DV <= 256: four numbers a lane
-    for (int base = 0; base < a.n_splits; base += kMergeShares) {
-        float mine = 0.f;  // the factor of share base + lane; 0 for a share without keys
-        if (base + lane < a.n_splits) {
-            const float* ml = a.part_ml + ((unit0 + base + lane) * rows_per_tile + row) * 2;
-            mine = (ml[0] == -INFINITY) ? 0.f : __builtin_amdgcn_exp2f(ml[0] - m_all);
-            den += ml[1] * mine;
-        }
-        const int count = min(kMergeShares, a.n_splits - base);
-        for (int sp = 0; sp < count; ++sp) {
-            const float f = __shfl(mine, sp, kWave);
-            const float* po = a.part_o + ((unit0 + base + sp) * rows_per_tile + row) * DV;
+    float x[N];
 #pragma unroll
-            for (int i = 0; i < 4; ++i)
-                if (lane + i * kWave < DV) acc[i] = fmaf(f == 0.f ? 0.f : po[lane + i * kWave], f, acc[i]);
+    for (int map = 0; map < MAPS; ++map) {
+        const int at = map * (rows_per_tile / MAPS) + row;
+        float m_all = -INFINITY;
+        for (int sp = lane; sp < a.n_splits; sp += kWave)
+            m_all = fmaxf(m_all, a.part_ml[((unit0 + sp) * rows_per_tile + at) * 2]);
+        m_all = wave_max(m_all);
+        float sink_term = 0.f;  // the sink's share of the denominator, counted once
+        if (a.shape.sinks) {
+            const float sink = a.shape.sinks[head] * kLog2e;
+            m_all = fmaxf(m_all, sink);
+            sink_term = __builtin_amdgcn_exp2f(sink - m_all);
         }
-    }
-    float factor = 1.0f / (wave_sum(den) + sink_term);
-    if (a.gate) {
-        const float z = to_float(a.gate[static_cast<size_t>(first_row_token + tok) * a.gate_stride + head]);
-        factor *= 1.0f / (1.0f + __expf(-z));
-    }
-    bf16_t* dst = a.out + (static_cast<size_t>(first_row_token + tok) * a.q_heads + head) * DV;
+        float den = 0.f;        // this lane's shares of it
+        float acc[N];
 #pragma unroll
-    for (int i = 0; i < 4; ++i)
-        if (lane + i * kWave < DV) dst[lane + i * kWave] = from_float<bf16_t>(acc[i] * factor);
+        for (int i = 0; i < N; ++i) acc[i] = 0.f;
+        for (int base = 0; base < a.n_splits; base += kMergeShares) {
+            float mine = 0.f;  // the factor of share base + lane; 0 for a share without keys
+            if (base + lane < a.n_splits) {
+                const float* ml = a.part_ml + ((unit0 + base + lane) * rows_per_tile + at) * 2;
+                mine = (ml[0] == -INFINITY) ? 0.f : __builtin_amdgcn_exp2f(ml[0] - m_all);
+                den += ml[1] * mine;
+            }
+            const int count = min(kMergeShares, a.n_splits - base);
+            for (int sp = 0; sp < count; ++sp) {
+                const float f = __shfl(mine, sp, kWave);
+                const float* po = a.part_o + ((unit0 + base + sp) * rows_per_tile + at) * DV;
+#pragma unroll
+                for (int i = 0; i < N; ++i)
+                    if (lane + i * kWave < DV) acc[i] = fmaf(f == 0.f ? 0.f : po[lane + i * kWave], f, acc[i]);
+            }
+        }
+        const float inverse = 1.0f / (wave_sum(den) + sink_term);
+#pragma unroll
+        for (int i = 0; i < N; ++i)
+            x[i] = map == 0 ? acc[i] * inverse : x[i] - a.shape.lambda * (acc[i] * inverse);
+    }
+    write_head<MAPS, DV>(a, x, static_cast<size_t>(first_row_token + tok), head, lane);
 }
 
-template <int D, int DV>
+// MOST: the most tiles of 16 rows a workgroup of these sizes takes
+template <int D, int DV, int MAPS = 1, int MOST = 4>
 int launch_scored(hipStream_t s, const ScoredArgs& a, int row_tiles) {
     dim3 grid(a.n_tiles, a.kv_heads, a.n_splits);
-    if (row_tiles == 1)
-        scored_attention_mfma_kernel<D, DV, 1><<<grid, 64 * kScoredWaves, 0, s>>>(a);
-    else if (row_tiles == 2)
-        scored_attention_mfma_kernel<D, DV, 2><<<grid, 64 * kScoredWaves, 0, s>>>(a);
-    else if (row_tiles == 4)
-        scored_attention_mfma_kernel<D, DV, 4><<<grid, 64 * kScoredWaves, 0, s>>>(a);
-    else
-        return CIE_BAD_ARGUMENT;
+    if (row_tiles > MOST || row_tiles < MAPS) return CIE_BAD_ARGUMENT;
+    if constexpr (MAPS == 1) {
+        if (row_tiles == 1) scored_attention_mfma_kernel<D, DV, 1, 1><<<grid, 64 * kScoredWaves, 0, s>>>(a);
+    }
+    if constexpr (MOST >= 2) {
+        if (row_tiles == 2) scored_attention_mfma_kernel<D, DV, 2, MAPS><<<grid, 64 * kScoredWaves, 0, s>>>(a);
+    }
+    if constexpr (MOST >= 4) {
+        if (row_tiles == 4) scored_attention_mfma_kernel<D, DV, 4, MAPS><<<grid, 64 * kScoredWaves, 0, s>>>(a);
+    }
+    if (row_tiles != 1 && row_tiles != 2 && row_tiles != 4) return CIE_BAD_ARGUMENT;
     if (hipGetLastError() != hipSuccess) return CIE_LAUNCH_FAILED;
     if (a.n_splits > 1)
-        scored_attention_merge_kernel<<<dim3(a.n_tiles, a.kv_heads, 4 * row_tiles), 256, 0, s>>>(a, 16 * row_tiles, DV);
+        scored_attention_merge_kernel<DV, MAPS><<<dim3(a.n_tiles, a.kv_heads, 4 * row_tiles / MAPS), 256, 0, s>>>(a, 16 * row_tiles);
     return cie_after_launch();
 }
 
@@ -717,8 +807,9 @@ CIE_API int cie_heads_prepare(void* stream, int dtype, const void* proj, int pro
                               const int* seq_slot, const int* block_table, int table_width, void* q_out,
                               void* k_pool, void* v_pool, int tokens, int q_heads, int kv_heads, int dim, int vdim,
                               int D, int DV, int page_size, int write_kv, const float* cos_table,
-                              const float* sin_table, int rot, int neighbours) {
+                              const float* sin_table, int rot, int neighbours, int maps) {
     if (rot < 0 || rot % 2 || rot > dim || (rot > 0 && (!cos_table || !sin_table))) return CIE_BAD_ARGUMENT;
+    if (maps < 1 || maps > 2 || (maps > 1 && norm_mode == 3)) return CIE_BAD_ARGUMENT;
     if (tokens < 0 || q_heads <= 0 || kv_heads <= 0 || dim <= 0 || vdim <= 0 || D < dim || DV < vdim ||
         page_size <= 0 || (page_size & (page_size - 1)) || table_width <= 0 || norm_mode < 0 || norm_mode > 3 ||
         (norm_mode >= 2 && (!q_weight || (write_kv && !k_weight))) || (norm_mode != 0 && !(eps > 0.f)) || temp_every < 0 ||
@@ -727,7 +818,7 @@ CIE_API int cie_heads_prepare(void* stream, int dtype, const void* proj, int pro
     if (tokens == 0) return CIE_OK;
     int page_shift = 0;
     while ((1 << page_shift) < page_size) ++page_shift;
-    const long units = static_cast<long>(tokens) * (q_heads + 2 * kv_heads);
+    const long units = static_cast<long>(tokens) * (maps * (q_heads + kv_heads) + kv_heads);
     const long blocks = (units + 3) / 4;
     if (blocks > 0x7fffffffL) return CIE_BAD_ARGUMENT;
     hipStream_t s = static_cast<hipStream_t>(stream);
@@ -736,13 +827,13 @@ CIE_API int cie_heads_prepare(void* stream, int dtype, const void* proj, int pro
             static_cast<const float*>(proj), proj_stride, q_off, k_off, v_off, q_weight, k_weight, norm_mode, eps,
             temp_coef, temp_every, positions, seq_of_token, seq_slot, block_table, table_width,
             static_cast<float*>(q_out), static_cast<float*>(k_pool), static_cast<float*>(v_pool), tokens, q_heads,
-            kv_heads, dim, vdim, D, DV, page_shift, write_kv, cos_table, sin_table, rot, neighbours);
+            kv_heads, dim, vdim, D, DV, page_shift, write_kv, cos_table, sin_table, rot, neighbours, maps);
     else if (dtype == CIE_BF16)
         heads_prepare_kernel<bf16_t><<<static_cast<unsigned>(blocks), 256, 0, s>>>(
             static_cast<const bf16_t*>(proj), proj_stride, q_off, k_off, v_off, q_weight, k_weight, norm_mode, eps,
             temp_coef, temp_every, positions, seq_of_token, seq_slot, block_table, table_width,
             static_cast<bf16_t*>(q_out), static_cast<bf16_t*>(k_pool), static_cast<bf16_t*>(v_pool), tokens, q_heads,
-            kv_heads, dim, vdim, D, DV, page_shift, write_kv, cos_table, sin_table, rot, neighbours);
+            kv_heads, dim, vdim, D, DV, page_shift, write_kv, cos_table, sin_table, rot, neighbours, maps);
     else
         return CIE_BAD_ARGUMENT;
     return cie_after_launch();
@@ -754,34 +845,37 @@ CIE_API int cie_scored_attention_generic(void* stream, int dtype, const void* q,
                                          const void* gate, int gate_stride, void* out, int tokens, int q_heads,
                                          int kv_heads, int D, int DV, int page_size, int window, float scale,
                                          float softcap, const float* slopes, const float* sinks, int chunk,
-                                         int keep) {
+                                         int keep, int gate_wide, int real_vdim, int maps, float lambda, float factor,
+                                         float eps) {
     if (tokens < 0 || q_heads <= 0 || kv_heads <= 0 || q_heads % kv_heads || D <= 0 || D % 8 || DV <= 0 || DV % 8 ||
-        D > kWave * kMaxSlices || DV > kWave * kMaxSlices || page_size <= 0 || table_width <= 0 || q_heads > 65535 ||
-        (gate && gate_stride < q_heads))
+        DV > kWave * kMaxWideSlices || page_size <= 0 || table_width <= 0 || q_heads > 65535 || real_vdim <= 0 ||
+        real_vdim > DV || maps < 1 || maps > 2 || (maps == 2 && !(eps > 0.f)) ||
+        (gate && gate_stride < (gate_wide ? q_heads * real_vdim : q_heads)))
         return CIE_BAD_ARGUMENT;
     if (tokens == 0) return CIE_OK;
     hipStream_t s = static_cast<hipStream_t>(stream);
     dim3 grid(tokens, q_heads);
-    const size_t lds = (static_cast<size_t>(D) + 4 * DV) * sizeof(float);
+    const size_t lds = (static_cast<size_t>(D) + (4 + maps) * DV) * sizeof(float);
+    if (lds > 60 * 1024) return CIE_BAD_ARGUMENT;
     if (chunk < 0 || (chunk > 0 && window > 0) || keep < 0 || (keep > 0 && window <= 0)) return CIE_BAD_ARGUMENT;
-    const ScoreShape shape{scale, softcap, slopes, sinks, window, chunk, keep};
-    if (dtype == CIE_F32)
-        scored_attention_generic_kernel<float><<<grid, 256, lds, s>>>(
-            static_cast<const float*>(q), static_cast<const float*>(k_pool), static_cast<const float*>(v_pool),
-            block_table, table_width, positions, seq_of_token, seq_slot, static_cast<const float*>(gate), gate_stride,
-            static_cast<float*>(out), q_heads, kv_heads, D, DV, page_size, shape);
-    else if (dtype == CIE_BF16)
-        scored_attention_generic_kernel<bf16_t><<<grid, 256, lds, s>>>(
-            static_cast<const bf16_t*>(q), static_cast<const bf16_t*>(k_pool), static_cast<const bf16_t*>(v_pool),
-            block_table, table_width, positions, seq_of_token, seq_slot, static_cast<const bf16_t*>(gate), gate_stride,
-            static_cast<bf16_t*>(out), q_heads, kv_heads, D, DV, page_size, shape);
-    else
-        return CIE_BAD_ARGUMENT;
+    const ScoreShape shape{scale, softcap, slopes, sinks, window, chunk, keep, gate_wide, real_vdim, lambda, factor, eps};
+#define CIE_GENERIC(T, SLICES)                                                                                          \
+    scored_attention_generic_kernel<T, SLICES><<<grid, 256, lds, s>>>(                                                  \
+        static_cast<const T*>(q), static_cast<const T*>(k_pool), static_cast<const T*>(v_pool), block_table, table_width, \
+        positions, seq_of_token, seq_slot, static_cast<const T*>(gate), gate_stride, static_cast<T*>(out), q_heads, kv_heads, \
+        D, DV, page_size, maps, shape)
+    const bool wide = DV > kWave * kMaxSlices;
+    if (dtype == CIE_F32 && !wide) CIE_GENERIC(float, kMaxSlices);
+    else if (dtype == CIE_F32) CIE_GENERIC(float, kMaxWideSlices);
+    else if (dtype == CIE_BF16 && !wide) CIE_GENERIC(bf16_t, kMaxSlices);
+    else if (dtype == CIE_BF16) CIE_GENERIC(bf16_t, kMaxWideSlices);
+    else return CIE_BAD_ARGUMENT;
+#undef CIE_GENERIC
     return cie_after_launch();
 }
 
-// bfloat16 on the matrix cores: (D, DV) one of (64, 64), (128, 128), (64, 128), (128, 64); pages of at least 4 keys;
-// a token's heads of one key head fill at most `row_tiles` tiles of 16 rows.
+// bfloat16 on the matrix cores: (D, DV) as the last lines list them; pages of at least 4 keys; a token's heads of one key
+// head fill at most `row_tiles` tiles of 16 rows (of each of the `maps`).
 CIE_API int cie_scored_attention_mfma(void* stream, const void* q, const void* k_pool, const void* v_pool,
                                       const int* block_table, int table_width, const int* tile_seq,
                                       const int* tile_q0, int n_tiles, const int* seq_slot, const int* seq_start,
@@ -789,15 +883,17 @@ CIE_API int cie_scored_attention_mfma(void* stream, const void* q, const void* k
                                       int gate_stride, void* out, int q_heads, int kv_heads, int D, int DV,
                                       int page_size, int tokens_per_tile, int row_tiles, int window, float scale,
                                       float softcap, const float* slopes, const float* sinks, int n_splits,
-                                      int keys_per_split, float* part_o, float* part_ml, int chunk, int keep) {
+                                      int keys_per_split, float* part_o, float* part_ml, int chunk, int keep,
+                                      int gate_wide, int real_vdim, int maps, float lambda, float factor, float eps) {
     if (chunk < 0 || (chunk > 0 && window > 0) || keep < 0 || (keep > 0 && window <= 0)) return CIE_BAD_ARGUMENT;
     if (n_tiles < 0 || q_heads <= 0 || kv_heads <= 0 || q_heads % kv_heads || page_size < 4 ||
         (page_size & (page_size - 1)) || table_width <= 0 || tokens_per_tile < 1 || kv_heads > 65535 ||
-        (tile_seq == nullptr) != (tile_q0 == nullptr) || (gate && gate_stride < q_heads))
+        (tile_seq == nullptr) != (tile_q0 == nullptr) || maps < 1 || maps > 2 || (maps == 2 && (!(eps > 0.f) || sinks)) ||
+        real_vdim <= 0 || real_vdim > DV || (gate && gate_stride < (gate_wide ? q_heads * real_vdim : q_heads)))
         return CIE_BAD_ARGUMENT;
-    if (tokens_per_tile * (q_heads / kv_heads) > 16 * row_tiles) return CIE_BAD_ARGUMENT;
+    if (tokens_per_tile * (q_heads / kv_heads) * maps > 16 * row_tiles) return CIE_BAD_ARGUMENT;
     if (n_splits < 1 || n_splits > 65535 ||
-        (n_splits > 1 && (keys_per_split < 128 || keys_per_split % 128 || !part_o || !part_ml || DV > 256)))
+        (n_splits > 1 && (keys_per_split < 128 || keys_per_split % 128 || !part_o || !part_ml)))
         return CIE_BAD_ARGUMENT;
     if (n_tiles == 0) return CIE_OK;
     ScoredArgs a;
@@ -825,11 +921,28 @@ CIE_API int cie_scored_attention_mfma(void* stream, const void* q, const void* k
     while ((1 << a.page_shift) < page_size) ++a.page_shift;
     a.tokens_per_tile = tokens_per_tile;
     a.n_tiles = n_tiles;
-    a.shape = ScoreShape{scale, softcap, slopes, sinks, window, chunk, keep};
+    a.shape = ScoreShape{scale, softcap, slopes, sinks, window, chunk, keep, gate_wide, real_vdim, lambda, factor, eps};
     hipStream_t s = static_cast<hipStream_t>(stream);
+    if (maps == 2) {
+        if (D == 64 && DV == 64) return launch_scored<64, 64, 2>(s, a, row_tiles);
+        if (D == 64 && DV == 128) return launch_scored<64, 128, 2>(s, a, row_tiles);
+        if (D == 128 && DV == 64) return launch_scored<128, 64, 2>(s, a, row_tiles);
+        if (D == 128 && DV == 128) return launch_scored<128, 128, 2>(s, a, row_tiles);
+        if (D == 128 && DV == 256) return launch_scored<128, 256, 2, 2>(s, a, row_tiles);
+        if (D == 256 && DV == 128) return launch_scored<256, 128, 2, 2>(s, a, row_tiles);
+        if (D == 256 && DV == 256) return launch_scored<256, 256, 2, 2>(s, a, row_tiles);
+        return CIE_BAD_ARGUMENT;
+    }
     if (D == 64 && DV == 64) return launch_scored<64, 64>(s, a, row_tiles);
     if (D == 128 && DV == 128) return launch_scored<128, 128>(s, a, row_tiles);
     if (D == 64 && DV == 128) return launch_scored<64, 128>(s, a, row_tiles);
     if (D == 128 && DV == 64) return launch_scored<128, 64>(s, a, row_tiles);
+    if (D == 96 && DV == 64) return launch_scored<96, 64>(s, a, row_tiles);
+    if (D == 128 && DV == 96) return launch_scored<128, 96>(s, a, row_tiles);
+    if (D == 160 && DV == 128) return launch_scored<160, 128, 1, 2>(s, a, row_tiles);
+    if (D == 192 && DV == 160) return launch_scored<192, 160, 1, 2>(s, a, row_tiles);
+    if (D == 256 && DV == 192) return launch_scored<256, 192, 1, 2>(s, a, row_tiles);
+    if (D == 320 && DV == 256) return launch_scored<320, 256, 1, 2>(s, a, row_tiles);
+    if (D == 576 && DV == 512) return launch_scored<576, 512, 1, 1>(s, a, row_tiles);
     return CIE_BAD_ARGUMENT;
 }

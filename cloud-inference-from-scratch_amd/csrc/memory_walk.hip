@@ -628,8 +628,8 @@ time_decay_kernel(const float* __restrict__ low, const T* __restrict__ w2t, cons
 template <typename T>
 __global__ void __launch_bounds__(1024)
 gated_group_norm_kernel(const float* __restrict__ y, const T* __restrict__ gate, long ldg,
-                        const float* __restrict__ weight, T* __restrict__ out, int width, int groups, float eps,
-                        int gate_first) {
+                        const float* __restrict__ weight, int weight_width, T* __restrict__ out, int width, int groups,
+                        float eps, int gate_first) {
     extern __shared__ float staged[];  // [width], then [groups]
     float* inverse = staged + width;
     const size_t token = blockIdx.x;
@@ -657,7 +657,7 @@ gated_group_norm_kernel(const float* __restrict__ y, const T* __restrict__ gate,
     T* dst = out + token * width;
     for (int c = threadIdx.x; c < width; c += blockDim.x) {
         float x = staged[c] * inverse[c / per];
-        if (weight) x *= weight[c];
+        if (weight) x *= weight[weight_width == width ? c : c % per];  // (a number per column, or one group's for all)
         if (g_row && !gate_first) x *= silu_f(to_float(g_row[c]));
         dst[c] = from_float<T>(x);
     }
@@ -813,10 +813,10 @@ CIE_API int cie_time_decay(void* stream, int dtype, const float* low, const void
 }
 
 CIE_API int cie_gated_group_norm(void* stream, int dtype, const float* y, const void* gate, long ldg,
-                                 const float* weight, void* out, int tokens, int width, int groups, float eps,
-                                 int gate_first) {
+                                 const float* weight, int weight_width, void* out, int tokens, int width, int groups,
+                                 float eps, int gate_first) {
     if (tokens < 0 || width <= 0 || groups <= 0 || width % groups || !(eps > 0.f) || !y || !out ||
-        (gate && ldg < width) || (static_cast<size_t>(width) + groups) * sizeof(float) > 64 * 1024)
+        (gate && ldg < width) || (weight && weight_width != width && weight_width != width / groups) || (static_cast<size_t>(width) + groups) * sizeof(float) > 64 * 1024)
         return CIE_BAD_ARGUMENT;
     if (tokens == 0) return CIE_OK;
     hipStream_t s = static_cast<hipStream_t>(stream);
@@ -824,10 +824,10 @@ CIE_API int cie_gated_group_norm(void* stream, int dtype, const float* y, const 
     const size_t lds = (static_cast<size_t>(width) + groups) * sizeof(float);
     if (dtype == CIE_F32)
         gated_group_norm_kernel<float><<<tokens, threads, lds, s>>>(y, static_cast<const float*>(gate), ldg, weight,
-                                                                 static_cast<float*>(out), width, groups, eps, gate_first);
+                                                                 weight_width, static_cast<float*>(out), width, groups, eps, gate_first);
     else if (dtype == CIE_BF16)
         gated_group_norm_kernel<bf16_t><<<tokens, threads, lds, s>>>(y, static_cast<const bf16_t*>(gate), ldg, weight,
-                                                                  static_cast<bf16_t*>(out), width, groups, eps, gate_first);
+                                                                  weight_width, static_cast<bf16_t*>(out), width, groups, eps, gate_first);
     else
         return CIE_BAD_ARGUMENT;
     return cie_after_launch();

@@ -81,6 +81,19 @@ _i = int
 _f = float
 
 
+def _row_view(name: str, t: torch.Tensor, shape: tuple, dtypes: tuple) -> None:
+    """A GPU matrix whose rows are in one piece each and may lie apart."""
+    if not (t.is_cuda and t.dim() == 2 and t.stride(1) == 1 and t.dtype in dtypes and tuple(t.shape) == tuple(shape)
+            and (t.shape[0] <= 1 or t.stride(0) >= t.shape[1])):
+        raise ValueError(f"{name} must be a {list(shape)} GPU view with unit inner stride in one of {dtypes}, is "
+                         f"{tuple(t.shape)} {t.dtype} with strides {t.stride()}")
+
+
+def _ld(t: torch.Tensor) -> int:
+    """The distance of a view's rows (a single row has none of its own)."""
+    return t.stride(0) if t.shape[0] > 1 else max(t.stride(0), t.shape[1])
+
+
 def _check_pools(k_pool: torch.Tensor, v_pool: torch.Tensor, dtype: torch.dtype, kv_heads: int,
                  head_dim: int) -> int:
     """Keys [pages, Hkv, page_size, D], values transposed [pages, Hkv, D, page_size]; returns page_size."""
@@ -101,7 +114,8 @@ def embed(table: torch.Tensor, ids: torch.Tensor, out: Optional[torch.Tensor] = 
     """``out[t] = float32(table[ids[t]]) * scale``; ids int32 [T] (already checked against the vocabulary).
     With ``feed`` (int32 [T]) and ``pool`` (int32): row t takes ``pool[feed[t]]`` as its id where
     ``feed[t] >= 0`` (tokens another kernel left on the device; ``feed[t]`` must index ``pool``).
-    ``rows`` ([T, hidden] in the table's dtype) also takes the same values, rounded to that dtype."""
+    ``rows`` ([T, hidden] in the table's dtype; a view whose rows lie apart is fine) also takes the same values, rounded
+    to that dtype."""
     _gpu("table", table, dims=2)
     _gpu("ids", ids, torch.int32, 1)
     vocab, hidden = table.shape
@@ -117,12 +131,11 @@ def embed(table: torch.Tensor, ids: torch.Tensor, out: Optional[torch.Tensor] = 
     if not (out.shape == (tokens, hidden)):
         raise ValueError(f"out must be {(tokens, hidden)}, is {tuple(out.shape)}")
     if rows is not None:
-        _gpu("rows", rows, table.dtype, 2)
-        if not (rows.shape == (tokens, hidden)):
-            raise ValueError(f"rows must be {(tokens, hidden)}, is {tuple(rows.shape)}")
+        _row_view("rows", rows, (tokens, hidden), (table.dtype,))
     _run("cie_embed", load_library().cie_embed(_stream(), _i(_code(table.dtype)), _ptr(table), _ptr(ids), _ptr(feed),
                                                _ptr(pool if feed is not None else None), _ptr(out), _ptr(rows),
-                                               _i(tokens), _i(hidden), _i(vocab), _f(scale)))
+                                               _ld(rows) if rows is not None else 0, _i(tokens), _i(hidden), _i(vocab),
+                                               _f(scale)))
     return out
 
 
@@ -927,6 +940,79 @@ def latent_rows(proj: torch.Tensor, weight: torch.Tensor, heads: int, plain: int
     return rows
 
 
+def latent_down(proj: torch.Tensor, q_off: int, q_rank: int, c_off: int, q_weight: Optional[torch.Tensor],
+                c_weight: torch.Tensor, latent: int, turned: int, rotary: Optional[tuple], positions: torch.Tensor,
+                seq_of_token: torch.Tensor, seq_slot: torch.Tensor, block_table: torch.Tensor, k_pool: torch.Tensor,
+                v_pool: torch.Tensor, eps: float, write_kv: bool = True) -> Optional[torch.Tensor]:
+    """Behind the down projections of a layer whose keys are compressed (``csrc/latent.hip``): the query latent
+    (``q_rank`` numbers from column ``q_off`` of ``proj``; 0: none) under its RMS norm comes back as [T, q_rank]; the key
+    latent (``latent`` numbers from ``c_off``) under its own and the shared key part behind it (``turned`` numbers, turned
+    by the position) go to the token's place in the cache: keys ``[turned | latent | zeros]``, values ``[latent | zeros]``.
+    ``rotary = (cos, sin, rot, neighbours)`` or ``None``; norm weights float32."""
+    if not (proj.is_cuda and proj.dim() == 2 and proj.stride(1) == 1 and proj.dtype in _CODES):
+        raise ValueError("proj must be a float32 or bfloat16 GPU matrix with unit inner stride")
+    tokens = proj.shape[0]
+    if min(q_off, q_rank, c_off) < 0 or proj.shape[1] < max(q_off + q_rank, c_off + latent + turned):
+        raise ValueError(f"proj {tuple(proj.shape)} does not hold latents of {q_rank} and {latent}+{turned} at {q_off}, {c_off}")
+    for name, w, size in (("q_weight", q_weight if q_rank else None, q_rank), ("c_weight", c_weight, latent)):
+        if w is not None:
+            _gpu(name, w, torch.float32, 1)
+            if w.shape[0] != size:
+                raise ValueError(f"{name} must be [{size}], is {tuple(w.shape)}")
+    if q_rank and q_weight is None:
+        raise ValueError("the query latent's norm has a weight")
+    width, value_width = k_pool.shape[3], v_pool.shape[2]
+    page_size = _check_kv_pools(k_pool, v_pool, proj.dtype, 1, width, value_width)
+    if width < latent + turned or value_width < latent:
+        raise ValueError(f"cache entries of {width} and {value_width} do not hold a latent of {latent} and {turned} turned numbers")
+    cos, sin, rot, neighbours = _check_rotary(rotary, turned)
+    _gpu("block_table", block_table, torch.int32, 2)
+    for name, meta in (("positions", positions), ("seq_of_token", seq_of_token)):
+        _gpu(name, meta, torch.int32, 1)
+        if meta.shape[0] < tokens:
+            raise ValueError(f"{name} has {meta.shape[0]} entries for {tokens} tokens")
+    _gpu("seq_slot", seq_slot, torch.int32, 1)
+    q_latent = torch.empty((tokens, q_rank), dtype=proj.dtype, device=proj.device) if q_rank else None
+    _run("cie_latent_down", load_library().cie_latent_down(
+        _stream(), _i(_code(proj.dtype)), _ptr(proj), _ld(proj), _i(q_off), _i(q_rank), _i(c_off), _ptr(q_weight), _ptr(c_weight),
+        _ptr(q_latent), _ptr(cos), _ptr(sin), _i(rot), _i(1 if neighbours else 0), _ptr(positions), _ptr(seq_of_token),
+        _ptr(seq_slot), _ptr(block_table), _i(block_table.shape[1]), _ptr(k_pool), _ptr(v_pool), _i(tokens), _i(latent),
+        _i(turned), _i(width), _i(value_width), _i(page_size), _f(eps), _i(1 if write_kv else 0)))
+    return q_latent
+
+
+def _check_rotary(rotary: Optional[tuple], most: int) -> tuple:
+    if rotary is None:
+        return None, None, 0, False
+    cos, sin, rot, neighbours = rotary
+    if rot < 2 or rot % 2 or rot > most:
+        raise ValueError(f"{rot} turning numbers of {most}: even, at least 2, at most all of them")
+    for name, table in (("cos", cos), ("sin", sin)):
+        _gpu(name, table, torch.float32, 2)
+        if table.shape[1] != rot // 2:
+            raise ValueError(f"{name} {tuple(table.shape)} does not hold {rot // 2} pairs per position")
+    return cos, sin, rot, neighbours
+
+
+def latent_queries(q: torch.Tensor, heads: int, plain: int, turned: int, latent: int, width: int, rotary: Optional[tuple],
+                   positions: torch.Tensor) -> torch.Tensor:
+    """Query rows [T, heads * width] for entries ``[turned | latent | zeros]`` from ``q`` [T, heads * (plain + turned)]:
+    each head's turned part, turned by the position, and the zeros; the room between them is left for the folded part."""
+    _row_view("q", q, (q.shape[0], heads * (plain + turned)), tuple(_CODES))
+    tokens = q.shape[0]
+    if width < turned + latent:
+        raise ValueError(f"rows of {width} do not hold {turned} + {latent} numbers")
+    cos, sin, rot, neighbours = _check_rotary(rotary, turned)
+    _gpu("positions", positions, torch.int32, 1)
+    if positions.shape[0] < tokens:
+        raise ValueError("one position per token")
+    rows = torch.empty((tokens, heads * width), dtype=q.dtype, device=q.device)
+    _run("cie_latent_queries", load_library().cie_latent_queries(
+        _stream(), _i(_code(q.dtype)), _ptr(q), _ld(q), _ptr(cos), _ptr(sin), _i(rot), _i(1 if neighbours else 0),
+        _ptr(positions), _ptr(rows), _i(tokens), _i(heads), _i(plain), _i(turned), _i(latent), _i(width)))
+    return rows
+
+
 RETENTION_ROWS = (4, 8, 16, 32)  # rows of a head's memory that one thread keeps in registers
 RETENTION_SLICE = 64             # value columns of a head that one workgroup takes
 RETENTION_LDS_FLOATS = 15 * 1024
@@ -1311,7 +1397,7 @@ def time_decay(low: torch.Tensor, w2t: torch.Tensor, w0: torch.Tensor, h: torch.
 def gated_group_norm(y: torch.Tensor, gate: Optional[torch.Tensor], weight: Optional[torch.Tensor], groups: int,
                      eps: float, out_dtype: torch.dtype, gate_first: bool) -> torch.Tensor:
     """The RMS norm of float32 rows ``y`` [T, W] in ``groups`` equal consecutive parts (each over its own root mean
-    square), times ``weight`` (float32 [W]), with ``silu(gate)`` multiplied in front of the norm (``gate_first``) or
+    square), times ``weight`` (float32 [W], or one group's numbers for all groups alike), with ``silu(gate)`` multiplied in front of the norm (``gate_first``) or
     behind it.  ``gate`` [T, W] in ``out_dtype`` (a view with unit inner stride)."""
     _gpu("y", y, torch.float32, 2)
     tokens, width = y.shape
@@ -1323,14 +1409,16 @@ def gated_group_norm(y: torch.Tensor, gate: Optional[torch.Tensor], weight: Opti
                 and tuple(gate.shape) == (tokens, width)):
             raise ValueError(f"gate must be a [{tokens}, {width}] view of {out_dtype} with unit inner stride")
         ldg = gate.stride(0) if tokens > 1 else max(gate.stride(0), width)
+    weight_width = 0
     if weight is not None:
         _gpu("weight", weight, torch.float32, 1)
-        if weight.shape[0] != width:
-            raise ValueError(f"weight must be [{width}]")
+        weight_width = weight.shape[0]
+        if weight_width not in (width, width // groups):
+            raise ValueError(f"weight must be [{width}], or [{width // groups}] for every group alike")
     out = torch.empty((tokens, width), dtype=out_dtype, device=y.device)
     _run("cie_gated_group_norm", load_library().cie_gated_group_norm(
-        _stream(), _i(_code(out_dtype)), _ptr(y), _ptr(gate), ldg, _ptr(weight), _ptr(out), _i(tokens), _i(width),
-        _i(groups), _f(eps), _i(1 if gate_first else 0)))
+        _stream(), _i(_code(out_dtype)), _ptr(y), _ptr(gate), ldg, _ptr(weight), _i(weight_width), _ptr(out), _i(tokens),
+        _i(width), _i(groups), _f(eps), _i(1 if gate_first else 0)))
     return out
 
 
@@ -1449,6 +1537,198 @@ def group_norm_add(residual: torch.Tensor, branch: Optional[torch.Tensor], weigh
     return out
 
 
+# ---------------------------------------------------------------------------
+DELTA_ROWS = (4, 8, 16, 32)       # rows of a column that one of its 16 lanes keeps in registers
+DELTA_COLUMNS = (1, 2, 4, 8)      # columns a thread takes
+DELTA_STATE_NUMBERS = 128         # numbers of the memory a thread keeps at most (64 with 32 rows)
+DELTA_LDS_BYTES = 40 * 1024
+DELTA_MAX_TAPS = 64
+DELTA_BLOCKS_FROM = 16            # tokens a sequence (on average) from which the memory is walked in blocks of 32 tokens
+DELTA_BLOCKS_MAX_DIM = 256        # ... for keys of up to this many numbers
+DELTA_BLOCKS_MAX_BYTES = 2 << 30  # ... while the blocks' scratch memory is no larger
+
+
+def plan_delta_walk(dim: int, vdim: int) -> tuple[int, int, int, int, int]:
+    """(rows a thread, columns a thread, threads, columns a workgroup, tokens staged at once) of the token-by-token form
+    for memories of ``dim`` x ``vdim``: all columns of a head in one workgroup where its registers hold them (the read-out's
+    norm and gate then ride along), else slices."""
+    if not (1 <= dim <= 512 and vdim >= 1):
+        raise ValueError(f"a memory of {dim} x {vdim}: keys of up to 512 numbers")
+    rows = next(r for r in DELTA_ROWS if 16 * r >= dim)
+    most = 2 if rows == 32 else 8
+    columns = next((c for c in DELTA_COLUMNS if c <= most and 32 * c >= vdim), most)
+    slice_cols = min(vdim, 32 * columns)
+    threads = -(-16 * -(-slice_cols // columns) // 64) * 64
+    chunk = max(1, min(16, DELTA_LDS_BYTES // (4 * (32 * rows + 2 * slice_cols + 3))))
+    return rows, columns, threads, slice_cols, chunk
+
+
+def delta_rule(proj: torch.Tensor, offsets: tuple[int, int, int, int, int, int], taps_w: torch.Tensor, a_log: torch.Tensor,
+               dt_bias: torch.Tensor, q_scale: float, norm_weight: torch.Tensor, eps: float, state: torch.Tensor,
+               past: torch.Tensor, seq_of_token: torch.Tensor, seq_slot: torch.Tensor, q_start_loc: torch.Tensor,
+               sequences: int, heads: int, kv_heads: int, dim: int, vdim: int, blocks: Optional[bool] = None) -> torch.Tensor:
+    """The gated delta rule over a step's tokens (``csrc/delta_rule.hip``).  ``proj`` [T, ...] holds each token's queries
+    and keys (kv_heads x dim), values and gates (heads x vdim), step-size and decay logits (heads) from the columns
+    ``offsets`` on; ``taps_w`` [2 kv_heads dim + heads vdim, taps] in proj's type; ``a_log``, ``dt_bias`` float32 [heads];
+    ``norm_weight`` float32 [vdim].  ``state`` float32 [slots, heads, vdim, dim] and ``past`` float32 [slots, heads,
+    max(taps - 1, 1), 2 dim + vdim] are read and moved on at the sequences' slots.  Steps of ``DELTA_BLOCKS_FROM`` tokens a
+    sequence and more go in blocks of 32 tokens on the matrix cores (``blocks``: force it or forbid it): the same sums in
+    another order.  Returns the normed, gated read-out [T, heads * vdim] in proj's type."""
+    if not (proj.is_cuda and proj.dim() == 2 and proj.stride(1) == 1 and proj.dtype in _CODES):
+        raise ValueError("proj must be a float32 or bfloat16 GPU matrix with unit inner stride")
+    tokens = proj.shape[0]
+    if heads < 1 or kv_heads < 1 or heads % kv_heads:
+        raise ValueError(f"{heads} heads are no multiple of {kv_heads} key heads")
+    sizes = (kv_heads * dim, kv_heads * dim, heads * vdim, heads * vdim, heads, heads)
+    if min(offsets) < 0 or max(o + n for o, n in zip(offsets, sizes)) > proj.shape[1]:
+        raise ValueError(f"proj {tuple(proj.shape)} does not hold the parts at {offsets}")
+    _gpu("taps_w", taps_w, proj.dtype, 2)
+    channels, taps = taps_w.shape
+    if channels != 2 * kv_heads * dim + heads * vdim or not 1 <= taps <= DELTA_MAX_TAPS:
+        raise ValueError(f"taps {tuple(taps_w.shape)} for {2 * kv_heads * dim + heads * vdim} channels (up to {DELTA_MAX_TAPS} taps)")
+    for name, t, size in (("a_log", a_log, heads), ("dt_bias", dt_bias, heads), ("norm_weight", norm_weight, vdim)):
+        _gpu(name, t, torch.float32, 1)
+        if t.shape[0] != size:
+            raise ValueError(f"{name} must be [{size}], is {tuple(t.shape)}")
+    _gpu("state", state, torch.float32, 4)
+    _gpu("past", past, torch.float32, 4)
+    if (tuple(state.shape[1:]) != (heads, vdim, dim) or tuple(past.shape[1:]) != (heads, max(taps - 1, 1), 2 * dim + vdim)
+            or not eps > 0):
+        raise ValueError(f"state {tuple(state.shape)} / past {tuple(past.shape)} do not fit {heads} heads of {dim} x {vdim}")
+    for name, meta, least in (("seq_slot", seq_slot, sequences), ("seq_of_token", seq_of_token, tokens),
+                              ("q_start_loc", q_start_loc, sequences + 1)):
+        _gpu(name, meta, torch.int32, 1)
+        if meta.shape[0] < least:
+            raise ValueError(f"{name} has {meta.shape[0]} entries, {least} are needed")
+    f32 = dict(dtype=torch.float32, device=proj.device)
+    common = (_stream(), _i(_code(proj.dtype)), _ptr(proj), _ld(proj), *(_i(o) for o in offsets), _ptr(taps_w), _i(taps),
+              _ptr(a_log), _ptr(dt_bias), _f(q_scale))
+    lib = load_library()
+    padded, cols16 = -(-dim // 16) * 16, -(-vdim // 16) * 16
+    places = (tokens // 32 + sequences + 1) * heads
+    per_block = 32 * (padded + cols16 + 33)
+    if blocks is None:
+        blocks = tokens >= DELTA_BLOCKS_FROM * max(sequences, 1)
+    if blocks and dim <= DELTA_BLOCKS_MAX_DIM and 4 * places * per_block <= DELTA_BLOCKS_MAX_BYTES:
+        y = torch.empty((tokens, heads * vdim), **f32)
+        rows = torch.empty((tokens, 2 * kv_heads * padded), **f32)
+        values = torch.empty((tokens, heads * vdim), **f32)
+        steps = torch.empty((2, tokens, heads), **f32)
+        scratch = torch.empty(places * per_block, **f32)
+        _run("cie_delta_blocks", lib.cie_delta_blocks(
+            *common, _ptr(state), _ptr(past), _ptr(seq_of_token), _ptr(seq_slot), _ptr(q_start_loc), _ptr(y), _ptr(rows),
+            _ptr(values), _ptr(steps), _ptr(scratch), _i(tokens), _i(sequences), _i(heads), _i(kv_heads), _i(dim), _i(vdim)))
+    else:
+        per_thread, columns, threads, slice_cols, chunk = plan_delta_walk(dim, vdim)
+        whole = slice_cols >= vdim
+        out = torch.empty((tokens, heads * vdim), dtype=proj.dtype, device=proj.device) if whole else None
+        y = None if whole else torch.empty((tokens, heads * vdim), **f32)
+        _run("cie_delta_walk", lib.cie_delta_walk(
+            *common, _ptr(norm_weight), _f(eps), _ptr(state), _ptr(past), _ptr(seq_slot), _ptr(q_start_loc), _ptr(out), _ptr(y),
+            _i(sequences), _i(heads), _i(kv_heads), _i(dim), _i(vdim), _i(per_thread), _i(columns), _i(threads), _i(slice_cols),
+            _i(chunk)))
+        if whole:
+            return out
+    gate = proj[:, offsets[3]: offsets[3] + heads * vdim]
+    return gated_group_norm(y, gate, norm_weight, heads, eps, proj.dtype, gate_first=False)
+
+
+# ---------------------------------------------------------------------------
+def layer_norm_add(residual: torch.Tensor, branch: Optional[torch.Tensor], weight: torch.Tensor, bias: torch.Tensor, eps: float,
+                   out_dtype: torch.dtype, rows: Optional[torch.Tensor] = None,
+                   plus: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """``residual += branch + plus`` (whatever of it is given; float32, in place unless ``rows``), then the layer norm of
+    every row under ``weight`` and ``bias`` (float32 [H]).  ``branch`` [T, H] float32 or ``out_dtype``; ``plus`` float32
+    [T, H], or [H] for every row alike.  With ``rows`` (int32 [n]) only those rows come back, in that order."""
+    _gpu("residual", residual, torch.float32, 2)
+    tokens, hidden = residual.shape
+    for name, t in (("weight", weight), ("bias", bias)):
+        _gpu(name, t, torch.float32, 1)
+        if t.shape[0] != hidden:
+            raise ValueError(f"{name} must be [{hidden}], is {tuple(t.shape)}")
+    if not (hidden <= MAX_NORM_WIDTH and eps > 0):
+        raise ValueError(f"rows of {hidden} numbers with eps {eps} do not fit the norm kernel")
+    if branch is not None:
+        _gpu("branch", branch, dims=2)
+        if not (branch.shape == residual.shape and branch.dtype in (torch.float32, out_dtype)):
+            raise ValueError(f"branch {tuple(branch.shape)} {branch.dtype} does not fit {tuple(residual.shape)} {out_dtype}")
+    plus_stride = 0
+    if plus is not None:
+        _gpu("plus", plus, torch.float32)
+        if plus.shape != residual.shape and tuple(plus.shape) != (hidden,):
+            raise ValueError(f"plus {tuple(plus.shape)} vs residual {tuple(residual.shape)}")
+        plus_stride = hidden if plus.dim() == 2 else 0
+    n_out = tokens
+    if rows is not None:
+        _gpu("rows", rows, torch.int32, 1)
+        n_out = rows.shape[0]
+    out = torch.empty((n_out, hidden), dtype=out_dtype, device=residual.device)
+    _run("cie_layer_norm_add", load_library().cie_layer_norm_add(
+        _stream(), _i(_code(branch.dtype if branch is not None else out_dtype)), _i(_code(out_dtype)), _ptr(residual),
+        _ptr(branch), _ptr(plus), plus_stride, _ptr(weight), _ptr(bias), _ptr(out), _ptr(rows), _i(n_out), _i(hidden), _f(eps)))
+    return out
+
+
+def branch_layer_norm_add(residual: torch.Tensor, branch: Optional[torch.Tensor], weight: torch.Tensor, bias: torch.Tensor,
+                          eps: float, out_dtype: torch.dtype, parts: Optional[torch.Tensor] = None,
+                          branch_gate: Optional[torch.Tensor] = None, part_weight: Optional[torch.Tensor] = None,
+                          branch2: Optional[torch.Tensor] = None, scales: tuple[float, float] = (1.0, 1.0),
+                          next_norm: Optional[tuple] = None, rows_out: Optional[torch.Tensor] = None) -> Optional[torch.Tensor]:
+    """``residual += layer norm of y`` under ``weight`` and ``bias``, with ``y`` as in :func:`branch_norm_add`, row by row,
+    in float32 and in place.  ``next_norm = (weight, bias)``: the layer norm of the new stream under those comes back in
+    ``out_dtype``.  ``rows_out`` ([T, H] in ``out_dtype``; its rows may lie apart) takes the new stream itself."""
+    _gpu("residual", residual, torch.float32, 2)
+    tokens, hidden = residual.shape
+    vectors = [("weight", weight), ("bias", bias)]
+    if next_norm is not None:
+        vectors += [("the next norm's weight", next_norm[0]), ("the next norm's bias", next_norm[1])]
+    for name, t in vectors:
+        _gpu(name, t, torch.float32, 1)
+        if t.shape[0] != hidden:
+            raise ValueError(f"{name} must be [{hidden}], is {tuple(t.shape)}")
+    if not (hidden <= MAX_NORM_WIDTH and eps > 0):
+        raise ValueError(f"rows of {hidden} numbers with eps {eps} do not fit the norm kernel")
+    if branch is None and parts is None and branch2 is None:
+        raise ValueError("nothing to add")
+    kinds = set()
+    for name, t in (("branch", branch), ("branch2", branch2)):
+        if t is not None:
+            _gpu(name, t, dims=2)
+            if not (t.shape == residual.shape and t.dtype in (torch.float32, out_dtype)):
+                raise ValueError(f"{name} {tuple(t.shape)} {t.dtype} does not fit {tuple(residual.shape)} {out_dtype}")
+            kinds.add(t.dtype)
+    if len(kinds) > 1:
+        raise ValueError("the two branches must be of one type")
+    gate_stride = 1
+    if branch_gate is not None:
+        if not (branch_gate.is_cuda and branch_gate.dtype == torch.float32 and branch_gate.dim() == 1):
+            raise ValueError("branch_gate must be a float32 GPU vector")
+        if branch is None or branch_gate.shape[0] != tokens:
+            raise ValueError("a gate comes with a branch, one logit per row")
+        gate_stride = max(branch_gate.stride(0), 1)
+    n_parts = 0
+    if parts is not None:
+        _gpu("parts", parts, torch.float32, 3)
+        if not (parts.shape[0] == tokens and parts.shape[2] == hidden):
+            raise ValueError(f"parts {tuple(parts.shape)} do not fit {tuple(residual.shape)}")
+        n_parts = parts.shape[1]
+    if part_weight is not None:
+        _gpu("part_weight", part_weight, torch.float32)
+        if parts is None or part_weight.numel() != tokens * n_parts:
+            raise ValueError("part weights come with parts, one per part and row")
+    if rows_out is not None:
+        _row_view("rows_out", rows_out, (tokens, hidden), (out_dtype,))
+    normed = torch.empty((tokens, hidden), dtype=out_dtype, device=residual.device) if next_norm is not None else None
+    kind = kinds.pop() if kinds else torch.float32
+    _run("cie_branch_layer_norm_add", load_library().cie_branch_layer_norm_add(
+        _stream(), _i(_code(kind)), _i(_code(out_dtype)), _ptr(residual), _ptr(branch), _ptr(branch_gate), _i(gate_stride),
+        _ptr(branch2), _f(scales[0]), _f(scales[1]), _ptr(parts), _ptr(part_weight), _i(n_parts), _ptr(weight), _ptr(bias),
+        _ptr(rows_out), _ld(rows_out) if rows_out is not None else 0, _i(tokens), _i(hidden), _f(eps),
+        _ptr(next_norm[0] if next_norm is not None else None), _ptr(next_norm[1] if next_norm is not None else None),
+        _ptr(normed)))
+    return normed
+
+
 def clamped_glu(gate_up: torch.Tensor, limit: float, alpha: float, offset: float, cubic: float = 0.0) -> torch.Tensor:
     """``g * sigmoid(alpha * (g + cubic * g^3)) * (u + offset)`` with ``g = min(gate, limit)``,
     ``u = clamp(up, -limit, limit)`` for gate_up [T, 2I] (gate half first).  ``cubic = 0`` is the plain sigmoid
@@ -1474,8 +1754,14 @@ def soft_cap_(x: torch.Tensor, cap: float) -> torch.Tensor:
 
 
 # ---------------------------------------------------------------------------
+MAX_GENERIC_VALUE = 1024   # numbers of a value head in the generic attention
 NORM_MODES = {None: 0, "unit": 1, "weight": 2, "whole": 3}
 SCORED_MFMA_DIMS = ((64, 64), (128, 128), (64, 128), (128, 64))  # (key, value) head sizes of the matrix-core form
+# ... those of heads with two maps: (a map's numbers, value numbers) -> the most tiles of 16 rows a workgroup takes ...
+DIFFERENTIAL_MFMA_DIMS = {(32, 64): 4, (32, 128): 4, (64, 64): 4, (64, 128): 4, (64, 256): 2, (128, 128): 2, (128, 256): 2}
+# ... and those of cache entries whose value is a part of the key: (entry, value) -> the most tiles of 16 rows
+LATENT_MFMA_DIMS = {(64, 64): 4, (96, 64): 4, (128, 96): 4, (128, 128): 4, (160, 128): 2, (192, 160): 2, (256, 192): 2,
+                    (320, 256): 2, (576, 512): 1}
 
 
 def _check_kv_pools(k_pool: torch.Tensor, v_pool: torch.Tensor, dtype: torch.dtype, kv_heads: int, dim: int,
@@ -1493,7 +1779,7 @@ def heads_prepare(proj: torch.Tensor, offsets: tuple[int, int, int], q_heads: in
                   k_weight: Optional[torch.Tensor], eps: float, temperature: Optional[tuple[float, int]],
                   positions: torch.Tensor, seq_of_token: torch.Tensor, seq_slot: torch.Tensor,
                   block_table: torch.Tensor, k_pool: torch.Tensor, v_pool: torch.Tensor, tokens: int,
-                  write_kv: bool = True, rotary: Optional[tuple] = None) -> torch.Tensor:
+                  write_kv: bool = True, rotary: Optional[tuple] = None, maps: int = 1) -> torch.Tensor:
     """From projected rows ``proj`` [T, >= ...] (queries at column ``offsets[0]``, keys at ``offsets[1]``, values at
     ``offsets[2]``, heads of ``dim`` / ``dim`` / ``vdim`` numbers) to queries ``[T, q_heads * kernel_dim]`` and the
     token's cache entries: per-head RMS norm of queries and keys (``norm``: ``None``, ``"unit"`` or ``"weight"`` with
@@ -1502,14 +1788,18 @@ def heads_prepare(proj: torch.Tensor, offsets: tuple[int, int, int], q_heads: in
     every)``), heads zero-padded up to the kernels' sizes.  ``rotary = (cos, sin, rot, neighbours)``: after the norm
     the first ``rot`` numbers of every query and key head turn by the token's position, in pairs of neighbours
     ``(2i, 2i + 1)`` or of the halves ``(i, i + rot / 2)``; cos and sin are float32 ``[positions, rot / 2]`` and must
-    reach every position of the step (the caller sees to that)."""
+    reach every position of the step (the caller sees to that).  ``maps=2``: every query and key head is a pair of maps
+    of ``dim`` numbers each, projected one after the other; the queries come back and the keys go to the cache with a
+    head's maps side by side, ``kernel_dim`` numbers each."""
+    if maps not in (1, 2) or (maps > 1 and norm == "whole"):
+        raise ValueError(f"one or two maps a head (two not under the norm over all heads), got {maps}")
     if not (proj.is_cuda and proj.dim() == 2 and proj.stride(1) == 1):
         raise ValueError("proj must be 2-d on the GPU with unit inner stride")
     dtype = proj.dtype
     q_off, k_off, v_off = offsets
-    need = q_off + q_heads * dim
+    need = q_off + q_heads * maps * dim
     if write_kv:
-        need = max(need, k_off + kv_heads * dim, v_off + kv_heads * vdim)
+        need = max(need, k_off + kv_heads * maps * dim, v_off + kv_heads * vdim)
     if not (proj.shape[0] >= tokens and proj.shape[1] >= need and min(offsets) >= 0):
         raise ValueError(f"proj {tuple(proj.shape)} too small for {tokens} tokens of {need} numbers")
     if norm not in NORM_MODES:
@@ -1527,7 +1817,7 @@ def heads_prepare(proj: torch.Tensor, offsets: tuple[int, int, int], q_heads: in
                 raise ValueError(f"{name} {tuple(w.shape)} does not fit heads of {dim} under the {norm!r} norm")
     if kernel_dim < dim or kernel_vdim < vdim:
         raise ValueError("the kernels' head sizes must hold the projection's")
-    page_size = _check_kv_pools(k_pool, v_pool, dtype, kv_heads, kernel_dim, kernel_vdim)
+    page_size = _check_kv_pools(k_pool, v_pool, dtype, kv_heads, maps * kernel_dim, kernel_vdim)
     _gpu("block_table", block_table, torch.int32, 2)
     for name, meta in (("positions", positions), ("seq_of_token", seq_of_token)):
         _gpu(name, meta, torch.int32, 1)
@@ -1547,13 +1837,13 @@ def heads_prepare(proj: torch.Tensor, offsets: tuple[int, int, int], q_heads: in
             _gpu(name, table, torch.float32, 2)
             if table.shape[1] != rot // 2 or not table.is_contiguous():
                 raise ValueError(f"{name} {tuple(table.shape)} does not hold {rot // 2} pairs per position")
-    q_out = torch.empty((tokens, q_heads * kernel_dim), dtype=dtype, device=proj.device)
+    q_out = torch.empty((tokens, q_heads * maps * kernel_dim), dtype=dtype, device=proj.device)
     _run("cie_heads_prepare", load_library().cie_heads_prepare(
         _stream(), _i(_code(dtype)), _ptr(proj), _i(proj.stride(0)), _i(q_off), _i(k_off), _i(v_off), _ptr(q_weight),
         _ptr(k_weight), _i(NORM_MODES[norm]), _f(eps), _f(coef), _i(every), _ptr(positions), _ptr(seq_of_token),
         _ptr(seq_slot), _ptr(block_table), _i(block_table.shape[1]), _ptr(q_out), _ptr(k_pool), _ptr(v_pool),
         _i(tokens), _i(q_heads), _i(kv_heads), _i(dim), _i(vdim), _i(kernel_dim), _i(kernel_vdim), _i(page_size),
-        _i(1 if write_kv else 0), _ptr(cos), _ptr(sin), _i(rot), _i(1 if neighbours else 0)))
+        _i(1 if write_kv else 0), _ptr(cos), _ptr(sin), _i(rot), _i(1 if neighbours else 0), _i(maps)))
     return q_out
 
 
@@ -1571,13 +1861,26 @@ def _check_score_shape(q_heads: int, slopes, sinks, softcap, window=None, chunk=
         raise ValueError(f"the cap on the scores must be positive, got {softcap}")
 
 
-def _check_gate(gate, tokens: int, q_heads: int, dtype: torch.dtype) -> int:
+def _check_gate(gate, tokens: int, numbers: int, dtype: torch.dtype) -> int:
     if gate is None:
         return 0
     if not (gate.is_cuda and gate.dim() == 2 and gate.stride(1) == 1 and gate.dtype == dtype
-            and gate.shape[0] >= tokens and gate.shape[1] >= q_heads):
-        raise ValueError(f"gate {tuple(gate.shape)} {gate.dtype} does not hold {tokens} rows of {q_heads} heads")
-    return gate.stride(0)
+            and gate.shape[0] >= tokens and gate.shape[1] >= numbers):
+        raise ValueError(f"gate {tuple(gate.shape)} {gate.dtype} does not hold {tokens} rows of {numbers} gates")
+    return _ld(gate)
+
+
+def _check_maps(differential, vdim: int, real_vdim: Optional[int], sinks) -> tuple[int, int, float, float, float]:
+    """(maps, numbers of a value head that are not padding, lambda, factor, eps)."""
+    real = vdim if real_vdim is None else int(real_vdim)
+    if not 1 <= real <= vdim:
+        raise ValueError(f"{real_vdim} numbers of a value head of {vdim}")
+    if differential is None:
+        return 1, real, 0.0, 1.0, 1.0
+    lam, factor, eps = (float(x) for x in differential)
+    if sinks is not None or not eps > 0:
+        raise ValueError("two maps come without a sink and with a positive eps")
+    return 2, real, lam, factor, eps
 
 
 def scored_attention_generic(q: torch.Tensor, k_pool: torch.Tensor, v_pool: torch.Tensor, block_table: torch.Tensor,
@@ -1585,17 +1888,23 @@ def scored_attention_generic(q: torch.Tensor, k_pool: torch.Tensor, v_pool: torc
                              q_heads: int, kv_heads: int, dim: int, vdim: int, window: Optional[int], scale: float,
                              softcap: Optional[float] = None, slopes: Optional[torch.Tensor] = None,
                              sinks: Optional[torch.Tensor] = None, gate: Optional[torch.Tensor] = None,
-                             chunk: Optional[int] = None, keep_first: int = 0) -> torch.Tensor:
+                             chunk: Optional[int] = None, keep_first: int = 0, gate_wide: bool = False,
+                             real_vdim: Optional[int] = None, differential: Optional[tuple] = None) -> torch.Tensor:
     """Attention of each token over its request's cached keys with shaped scores (see ``csrc/attention_scored.hip``;
     ``chunk``: a token sees the keys of its own chunk of that many positions, counted from position 0, up to itself;
     ``keep_first``: beside its window a token sees the first that many keys of its sequence):
     ``q`` [T, q_heads * dim]; returns [T, q_heads * vdim].  ``gate`` [T, >= q_heads] (a view is fine): head h's output
-    is multiplied by ``sigmoid(gate[t, h])``.  float32 or bfloat16."""
+    is multiplied by ``sigmoid(gate[t, h])``; with ``gate_wide`` the gate has a number for each of a head's
+    ``real_vdim`` numbers (``vdim`` less its padding).  ``differential = (lambda, factor, eps)``: query and key heads are
+    pairs of maps (``q`` [T, q_heads * 2 * dim]), each a softmax of its own over the same values; head h's output is
+    ``factor * (a1 - lambda a2) / rms(a1 - lambda a2)``.  float32 or bfloat16."""
     _gpu("q", q, dims=2)
-    if not (q.shape == (tokens, q_heads * dim) and q_heads % kv_heads == 0 and dim % 8 == 0 and vdim % 8 == 0
-            and dim <= 256 and vdim <= 256):
-        raise ValueError(f"q {tuple(q.shape)} does not fit {tokens} tokens of {q_heads} heads of {dim} (multiples of 8 up to 256)")
-    page_size = _check_kv_pools(k_pool, v_pool, q.dtype, kv_heads, dim, vdim)
+    maps, real, lam, factor, eps = _check_maps(differential, vdim, real_vdim, sinks)
+    if not (q.shape == (tokens, q_heads * maps * dim) and q_heads % kv_heads == 0 and dim % 8 == 0 and vdim % 8 == 0
+            and vdim <= MAX_GENERIC_VALUE and 4 * (dim + (4 + maps) * vdim) <= 60 * 1024):
+        raise ValueError(f"q {tuple(q.shape)} does not fit {tokens} tokens of {q_heads} heads of {dim} and {vdim} (multiples of "
+                         f"8, values up to {MAX_GENERIC_VALUE})")
+    page_size = _check_kv_pools(k_pool, v_pool, q.dtype, kv_heads, maps * dim, vdim)
     _gpu("block_table", block_table, torch.int32, 2)
     for name, meta in (("positions", positions), ("seq_of_token", seq_of_token)):
         _gpu(name, meta, torch.int32, 1)
@@ -1603,13 +1912,14 @@ def scored_attention_generic(q: torch.Tensor, k_pool: torch.Tensor, v_pool: torc
             raise ValueError(f"{name} has {meta.shape[0]} entries for {tokens} tokens")
     _gpu("seq_slot", seq_slot, torch.int32, 1)
     _check_score_shape(q_heads, slopes, sinks, softcap, window, chunk, keep_first)
-    gate_stride = _check_gate(gate, tokens, q_heads, q.dtype)
+    gate_stride = _check_gate(gate, tokens, q_heads * real if gate_wide else q_heads, q.dtype)
     out = torch.empty((tokens, q_heads * vdim), dtype=q.dtype, device=q.device)
     _run("cie_scored_attention_generic", load_library().cie_scored_attention_generic(
         _stream(), _i(_code(q.dtype)), _ptr(q), _ptr(k_pool), _ptr(v_pool), _ptr(block_table), _i(block_table.shape[1]),
         _ptr(positions), _ptr(seq_of_token), _ptr(seq_slot), _ptr(gate), _i(gate_stride), _ptr(out), _i(tokens),
         _i(q_heads), _i(kv_heads), _i(dim), _i(vdim), _i(page_size), _i(window or 0), _f(scale), _f(softcap or 0.0),
-        _ptr(slopes), _ptr(sinks), _i(chunk or 0), _i(keep_first)))
+        _ptr(slopes), _ptr(sinks), _i(chunk or 0), _i(keep_first), _i(1 if gate_wide else 0), _i(real), _i(maps), _f(lam),
+        _f(factor), _f(eps)))
     return out
 
 
@@ -1621,21 +1931,27 @@ def scored_attention_mfma(q: torch.Tensor, k_pool: torch.Tensor, v_pool: torch.T
                           softcap: Optional[float] = None, slopes: Optional[torch.Tensor] = None,
                           sinks: Optional[torch.Tensor] = None, gate: Optional[torch.Tensor] = None,
                           n_splits: int = 1, keys_per_split: int = 0, chunk: Optional[int] = None,
-                          keep_first: int = 0) -> torch.Tensor:
-    """The same on the matrix cores (bfloat16, (dim, vdim) in ``SCORED_MFMA_DIMS``, pages of a power of two >= 4):
+                          keep_first: int = 0, gate_wide: bool = False, real_vdim: Optional[int] = None,
+                          differential: Optional[tuple] = None) -> torch.Tensor:
+    """The same on the matrix cores (bfloat16, (dim, vdim) in ``SCORED_MFMA_DIMS`` or ``LATENT_MFMA_DIMS``, with two maps in
+    ``DIFFERENTIAL_MFMA_DIMS``; pages of a power of two >= 4; two maps' rows fill ``row_tiles`` tiles together):
     tiles of ``tokens_per_tile`` consecutive tokens of one sequence (``tile_seq``, ``tile_q0`` int32 [n_tiles]; both
     ``None``: tile i is sequence i's first), whose rows times the heads per key head fill ``row_tiles`` tiles of 16.
     ``n_splits > 1``: every tile's keys in that many shares of ``keys_per_split`` (a multiple of 128; the shares must
     cover the longest range of keys a tile sees), a workgroup each, joined by a second kernel."""
     _gpu("q", q, torch.bfloat16, 2)
-    if not (q.shape == (tokens, q_heads * dim) and q_heads % kv_heads == 0 and (dim, vdim) in SCORED_MFMA_DIMS):
+    maps, real, lam, factor, eps = _check_maps(differential, vdim, real_vdim, sinks)
+    most = (DIFFERENTIAL_MFMA_DIMS.get((dim, vdim)) if maps == 2
+            else 4 if (dim, vdim) in SCORED_MFMA_DIMS else LATENT_MFMA_DIMS.get((dim, vdim)))
+    if most is None or not (q.shape == (tokens, q_heads * maps * dim) and q_heads % kv_heads == 0):
         raise ValueError(f"q {tuple(q.shape)} / heads of {dim}, {vdim} are not what the matrix-core form takes")
-    page_size = _check_kv_pools(k_pool, v_pool, q.dtype, kv_heads, dim, vdim)
+    page_size = _check_kv_pools(k_pool, v_pool, q.dtype, kv_heads, maps * dim, vdim)
     if page_size < 4 or page_size & (page_size - 1):
         raise ValueError(f"pages must hold a power of two >= 4 keys, hold {page_size}")
     group = q_heads // kv_heads
-    if row_tiles not in (1, 2, 4) or tokens_per_tile < 1 or tokens_per_tile * group > 16 * row_tiles:
-        raise ValueError(f"{tokens_per_tile} tokens of {group} heads do not fit {row_tiles} tiles of 16 rows")
+    if (row_tiles not in (1, 2, 4) or not maps <= row_tiles <= most or tokens_per_tile < 1
+            or tokens_per_tile * group * maps > 16 * row_tiles):
+        raise ValueError(f"{tokens_per_tile} tokens of {group} heads do not fit {row_tiles} tiles of 16 rows (at most {most})")
     _gpu("block_table", block_table, torch.int32, 2)
     if (tile_seq is None) != (tile_q0 is None):
         raise ValueError("tile_seq and tile_q0 come together")
@@ -1653,7 +1969,7 @@ def scored_attention_mfma(q: torch.Tensor, k_pool: torch.Tensor, v_pool: torch.T
     if tile_seq is None and n_tiles > sequences:
         raise ValueError(f"{n_tiles} tiles for {sequences} sequences")
     _check_score_shape(q_heads, slopes, sinks, softcap, window, chunk, keep_first)
-    gate_stride = _check_gate(gate, tokens, q_heads, q.dtype)
+    gate_stride = _check_gate(gate, tokens, q_heads * real if gate_wide else q_heads, q.dtype)
     out = torch.empty((tokens, q_heads * vdim), dtype=q.dtype, device=q.device)
     part_o = part_ml = None
     if n_splits > 1:
@@ -1667,9 +1983,10 @@ def scored_attention_mfma(q: torch.Tensor, k_pool: torch.Tensor, v_pool: torch.T
     _run("cie_scored_attention_mfma", load_library().cie_scored_attention_mfma(
         _stream(), _ptr(q), _ptr(k_pool), _ptr(v_pool), _ptr(block_table), _i(block_table.shape[1]), _ptr(tile_seq),
         _ptr(tile_q0), _i(n_tiles), _ptr(seq_slot), _ptr(seq_start), _ptr(seq_q_len), _ptr(q_start_loc), _ptr(gate),
-        _i(gate_stride), _ptr(out), _i(q_heads), _i(kv_heads), _i(dim), _i(vdim), _i(page_size), _i(tokens_per_tile),
+        _i(gate_stride), _ptr(out), _i(q_heads), _i(kv_heads), _i(maps * dim), _i(vdim), _i(page_size), _i(tokens_per_tile),
         _i(row_tiles), _i(window or 0), _f(scale), _f(softcap or 0.0), _ptr(slopes), _ptr(sinks), _i(n_splits),
-        _i(keys_per_split), _ptr(part_o), _ptr(part_ml), _i(chunk or 0), _i(keep_first)))
+        _i(keys_per_split), _ptr(part_o), _ptr(part_ml), _i(chunk or 0), _i(keep_first), _i(1 if gate_wide else 0), _i(real),
+        _i(maps), _f(lam), _f(factor), _f(eps)))
     return out
 
 

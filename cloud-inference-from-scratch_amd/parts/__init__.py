@@ -1,4 +1,4 @@
-from . import (attention, block, feed_forward, latent_attention, norm, parallel_mixers, position,  # noqa: F401
+from . import (attention, block, delta_rule, entry, feed_forward, latent_attention, norm, parallel_mixers, position,  # noqa: F401
                recurrent, routed_experts, scored_attention)  # (fill the registries)
 from .base import (
     BLOCKS,

@@ -21,6 +21,9 @@ Interfaces (``x`` is ``[tokens, hidden]`` in the engine's activation dtype,
                 unit of this call (``PagedView`` or ``StateView``), ``writes``
                 tells whether this call appends to it.
 ``FeedForward`` ``forward(x) -> y``
+``Entry``       ``joint(tokens) -> [tokens, 2 * hidden]`` and ``forward(joint, number) -> (residual, plus)``: remakes
+                the stream in front of a call of the run order from a row's two halves, the stream and the
+                embedding's rows; ``plus`` (float32) still joins the new stream.
 ``Block``       ``forward(residual, pending, batch, view, writes) -> (residual, pending)``
                 ``pending`` is a branch output not yet added to the residual, so
                 that the add fuses with the next norm.
@@ -40,6 +43,7 @@ POSITIONS: dict[str, Callable[..., Any]] = {}
 MIXERS: dict[str, Callable[..., Any]] = {}
 FEED_FORWARDS: dict[str, Callable[..., Any]] = {}
 BLOCKS: dict[str, Callable[..., Any]] = {}
+ENTRIES: dict[str, Callable[..., Any]] = {}
 
 _REGISTRIES = {
     "norm": NORMS,
@@ -47,11 +51,12 @@ _REGISTRIES = {
     "mixer": MIXERS,
     "feed_forward": FEED_FORWARDS,
     "block": BLOCKS,
+    "entry": ENTRIES,
 }
 
 
 def register_part(role: str, kind: str, factory: Callable[..., Any]) -> None:
-    """``role`` is one of norm, position, mixer, feed_forward, block."""
+    """``role`` is one of norm, position, mixer, feed_forward, block, entry."""
     _REGISTRIES[role][kind] = factory
 
 

@@ -11,7 +11,7 @@ cheaper form or rides along with the product behind it (``parts/linear.py``).
 ``BranchNormBlock``: the sublayers read the stream itself and their outputs are normed before they are added:
 ``h += norm1(mixer(h)); h += norm2(feed_forward(h))``.
 
-``SandwichNormBlock``: a norm in front of every sublayer and one on its output, which is then scaled per channel:
+``SandwichNormBlock``: a norm in front of every sublayer and one on its output, which may then be scaled per channel:
 ``h += s1 * norm1_out(mixer(norm1(h))); h += s2 * norm2_out(feed_forward(norm2(h)))``.
 
 ``ParallelDepthBlock``: both branches read the same stream, and the next layer reads a weighted average of what
@@ -121,6 +121,17 @@ def normalise(norm, residual: torch.Tensor, pending, dtype: torch.dtype, rows=No
     return norm.forward(residual, pending, dtype)
 
 
+def whole_stream(residual: torch.Tensor, pending) -> torch.Tensor:
+    """The float32 stream with what is pending added to it."""
+    if isinstance(pending, WeightedPair):
+        pending = pending.combined()
+    if isinstance(pending, torch.Tensor):
+        return residual + pending.float()
+    if pending is None or isinstance(pending, (Added, RowSumsq, NormedRows)):
+        return residual
+    raise ValueError(f"a branch that is still {type(pending).__name__} cannot be added here")
+
+
 register_part("block", "pre_norm", PreNormBlock)
 
 
@@ -137,7 +148,7 @@ class BranchNormBlock(PreNormBlock):
         super().__init__(spec)
         self.has_feed_forward = spec.feed_forward.kind != "none"
         for norm in (self.norm1, self.norm2):
-            if not hasattr(norm, "add_normed"):
+            if not hasattr(norm, "add_normed") or hasattr(norm, "joins_into"):
                 raise ValueError("this arrangement takes norms that can add a normed branch (rms_norm_one_plus)")
 
     def _parts(self):
@@ -282,12 +293,15 @@ register_part("block", "parallel_depth_average", ParallelDepthBlock)
 
 class SandwichNormBlock(PreNormBlock):
     """``h += s1 * norm1_out(mixer(norm1(h)))``, then ``h += s2 * norm2_out(feed_forward(norm2(h)))``: norms on both
-    sides of a sublayer, and a learned scale per channel (``s1``, ``s2``: the checkpoint tensors ``<layer>ls1`` and
-    ``<layer>ls2``, or whatever the spec's ``names`` call ``scale1`` and ``scale2``) on what joins the stream.  The
-    scale is folded into the output norm's weight once, in float32.  One kernel norms a sublayer's output, adds it
-    and makes the norm that the next sublayer reads (the next layer's first norm too, where that layer is of this
-    kind), so the stream is read and written once per sublayer.  The output norms are of a kind with ``add_normed``
-    (``rms_norm_groups`` with one group).  A layer without feed-forward has neither second norm nor ``s2``."""
+    sides of a sublayer, and (the layer's option ``layer_scale``, on unless it says otherwise) a learned scale per channel
+    (``s1``, ``s2``: the checkpoint tensors ``<layer>ls1`` and ``<layer>ls2``, or whatever the spec's ``names`` call
+    ``scale1`` and ``scale2``) on what joins the stream.  The scale is folded into the output norm once, in float32.  One
+    kernel norms a sublayer's output, adds it and makes the norm that the next sublayer reads (the first norm of the layer
+    that runs next too, where that layer is of this kind), so the stream is read and written once per sublayer.  The output
+    norms are of a kind with ``add_normed`` (``rms_norm_groups`` with one group, ``layer_norm``).  A layer without
+    feed-forward has neither second norm nor ``s2``."""
+
+    takes_follower = True
 
     def __init__(self, spec: LayerSpec) -> None:
         super().__init__(spec)
@@ -297,13 +311,8 @@ class SandwichNormBlock(PreNormBlock):
         self.norm2_out = build_part("norm", spec.norm2_out) if self.has_feed_forward else None
         self.layer_scale = bool(spec.option("layer_scale", True))
         for norm in (self.norm1_out, self.norm2_out):
-            if norm is not None and not hasattr(norm, "add_normed"):
-                raise ValueError("this arrangement takes output norms that can add a normed branch")
-        self.next_block: Any = None
-
-    def link_next(self, block: Any) -> None:
-        """The block that runs after this one (``None``: the last); its first norm rides in this block's last kernel."""
-        self.next_block = block if isinstance(block, SandwichNormBlock) else None
+            if norm is not None and not hasattr(norm, "joins_into"):
+                raise ValueError("this arrangement takes output norms that can add a normed branch and make the norm behind it")
 
     def _parts(self):
         parts = [("norm1", self.norm1), ("mixer", self.mixer), ("norm1_out", self.norm1_out)]
@@ -332,32 +341,38 @@ class SandwichNormBlock(PreNormBlock):
 
     def bind(self, tensors, prefix, dtype, device) -> None:
         super().bind(tensors, prefix, dtype, device)
-        # the scale per channel and the output norm's weight multiply one after the other: their float32 product, once
-        self.out_weight1 = self.norm1_out.weight_f32
-        self.out_weight2 = self.norm2_out.weight_f32 if self.has_feed_forward else None
+        # the scale per channel and the output norm multiply one after the other: their float32 product, once
+        self.scale1 = self.scale2 = None
         if self.layer_scale:
-            self.out_weight1 = (self.out_weight1 * tensors[prefix + self.spec.name_of("scale1")].float()).contiguous()
+            self.scale1 = self.norm1_out.scaled(tensors[prefix + self.spec.name_of("scale1")])
             if self.has_feed_forward:
-                self.out_weight2 = (self.out_weight2 * tensors[prefix + self.spec.name_of("scale2")].float()).contiguous()
+                self.scale2 = self.norm2_out.scaled(tensors[prefix + self.spec.name_of("scale2")])
 
-    def forward(self, residual: torch.Tensor, pending, batch, view, writes: bool = True):
-        if isinstance(pending, NormedRows) and pending.owner is self:
+    def forward(self, residual: torch.Tensor, pending, batch, view, writes: bool = True, plus: Optional[torch.Tensor] = None,
+                follower: Any = None, stream_rows: Optional[torch.Tensor] = None):
+        """``follower``: the block that runs next, whose first norm may ride in this block's last kernel.
+        ``stream_rows`` ([T, H] in the activation type): the last kernel leaves the stream there too."""
+        if isinstance(pending, NormedRows) and pending.owner is self and plus is None:
             x = pending.first
+        elif plus is not None and getattr(self.norm1, "takes_plus", False):
+            x = self.norm1.forward(residual, None if isinstance(pending, NormedRows) else pending, self.dtype, plus=plus)
         else:
+            if plus is not None:
+                raise ValueError("the first norm of this layer cannot add rows to the stream")
             x = normalise(self.norm1, residual, pending, self.dtype)
         mixed = self.mixer.forward(x, batch, view, writes)
-        follower = self.next_block
-        after = follower.norm1.weight_f32 if follower is not None else None
+        last = self.norm2_out if self.has_feed_forward else self.norm1_out
+        then = follower.norm1 if isinstance(follower, SandwichNormBlock) and last.joins_into(follower.norm1) else None
         if self.has_feed_forward:
-            _, x = self.norm1_out.add_normed(residual, mixed, self.dtype, weight=self.out_weight1,
-                                             then=self.norm2.weight_f32)
-            fed = self.feed_forward.forward(x)
-            last = self.norm2_out.add_normed(residual, fed, self.dtype, weight=self.out_weight2, then=after)
+            inner = self.norm1_out.joins_into(self.norm2)
+            x = self.norm1_out.add_normed(residual, mixed, self.dtype, scale=self.scale1, then=self.norm2 if inner else None)
+            if not inner:
+                x = normalise(self.norm2, residual, None, self.dtype)
+            made = self.norm2_out.add_normed(residual, self.feed_forward.forward(x), self.dtype, scale=self.scale2, then=then,
+                                             stream_rows=stream_rows)
         else:
-            last = self.norm1_out.add_normed(residual, mixed, self.dtype, weight=self.out_weight1, then=after)
-        if follower is None:
-            return residual, None
-        return residual, NormedRows(last[1], None, follower)
+            made = self.norm1_out.add_normed(residual, mixed, self.dtype, scale=self.scale1, then=then, stream_rows=stream_rows)
+        return residual, None if then is None else NormedRows(made, None, follower)
 
 
 register_part("block", "sandwich_norm", SandwichNormBlock)

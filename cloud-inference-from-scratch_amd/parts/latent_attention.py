@@ -27,12 +27,8 @@ from ..weights.tensors import TensorSpec
 from .attention import attend
 from .base import Part, build_part, register_part
 from .linear import linear
-
-
-def positions_bound(batch) -> int:
-    """Positions a step's rotation tables have to reach: its longest context, or, for a step that is captured and
-    replayed with other contexts, the bound it was captured for."""
-    return batch.static_plan.max_keys if batch.static_plan is not None else batch.max_context
+from .position import positions_bound
+from .scored_attention import scored_attend
 
 
 class LatentAttention(Part):
@@ -110,3 +106,122 @@ class LatentAttention(Part):
 
 
 register_part("mixer", "latent_attention", LatentAttention)
+
+
+class WindowedLatentAttention(Part):
+    """The same attention with what its scores may be shaped by: queries that come from a latent of their own
+    (``q_rank``: ``q = W_uq norm(W_dq x)``; ``None``: ``q = W_q x``), a window (the token and the ``window - 1`` before
+    it), a sink per head in the softmax's denominator, and no gate on the output.  A token's cache entry is
+    ``[turned key part | normed latent | zeros]`` and its value the normed latent alone, so that the attention kernels
+    that shape their scores (``scored_attend``) see one key head for all query heads, whose value is narrower than its
+    key.  ``q_rank=0`` reads the rank off the checkpoint."""
+
+    graph_safe = True
+
+    def __init__(self, hidden_size: int, num_heads: int, head_dim: int, rot_dim: int, value_dim: int, kv_rank: int,
+                 scale: float, eps: float, position: Optional[PartSpec] = None, q_rank: Optional[int] = None,
+                 window: Optional[int] = None, sink: bool = False) -> None:
+        for name, value in (("hidden_size", hidden_size), ("num_heads", num_heads), ("head_dim", head_dim),
+                            ("value_dim", value_dim), ("kv_rank", kv_rank)):
+            if isinstance(value, bool) or not isinstance(value, int) or value < 1:
+                raise ValueError(f"{name} must be a positive integer, got {value!r}")
+        if rot_dim < 0 or not eps > 0 or (q_rank is not None and q_rank < 0):
+            raise ValueError(f"a turned part of {rot_dim} numbers, a query latent of {q_rank}, eps {eps}: not negative, eps positive")
+        if window is not None and window < 1:
+            raise ValueError("window must be positive")
+        self.hidden_size, self.num_heads, self.head_dim, self.rot_dim = hidden_size, num_heads, head_dim, rot_dim
+        self.value_dim, self.kv_rank, self.scale, self.eps = value_dim, kv_rank, float(scale), float(eps)
+        self.q_rank, self.window, self.sink = q_rank, window, bool(sink)
+        self.position = build_part("position", position) if position is not None else None
+        if self.position is not None and self.position.rotates and self.position.rotary_dim > rot_dim:
+            raise ValueError(f"{self.position.rotary_dim} turning numbers in a turned part of {rot_dim}")
+        entry = rot_dim + kv_rank
+        fitting = [pair for pair in ops.LATENT_MFMA_DIMS if pair[0] >= entry and pair[1] >= kv_rank]
+        self.mfma_dims = min(fitting) if fitting else None
+        round8 = lambda n: -(-n // 8) * 8
+        self.entry_dim, self.latent_dim = self.mfma_dims or (round8(entry), round8(kv_rank))
+        if self.latent_dim > ops.MAX_GENERIC_VALUE:
+            raise ValueError(f"a latent of {kv_rank} numbers is more than the attention kernels' {ops.MAX_GENERIC_VALUE}")
+
+    def cache_need(self) -> PagedKV:
+        return PagedKV(1, self.entry_dim, self.window,
+                       value_dim=self.latent_dim if self.latent_dim != self.entry_dim else None)
+
+    def expected_tensors(self, prefix: str) -> dict[str, TensorSpec]:
+        h, p, r, v, c, hidden = self.num_heads, self.head_dim, self.rot_dim, self.value_dim, self.kv_rank, self.hidden_size
+        if self.q_rank is None:
+            out = {prefix + "q": TensorSpec((h * (p + r), hidden))}
+        else:
+            rank, drawn = self.q_rank or None, self.q_rank or max(8, hidden // 4 // 8 * 8)
+            out = {prefix + "dq": TensorSpec((rank, hidden), drawn=(drawn, hidden)),
+                   prefix + "dq.norm": TensorSpec((rank,), init="norm", keeps_float32=True, drawn=(drawn,)),
+                   prefix + "uq": TensorSpec((h * (p + r), rank), drawn=(h * (p + r), drawn))}
+        out.update({
+            prefix + "dkv": TensorSpec((c + r, hidden)),
+            prefix + "dkv.norm": TensorSpec((c,), init="norm", keeps_float32=True),
+            prefix + "uk": TensorSpec((h * p, c)),
+            prefix + "uv": TensorSpec((h * v, c)),
+            prefix + "o": TensorSpec((hidden, h * v)),
+        })
+        if self.sink:
+            out[prefix + "sink"] = TensorSpec((h,), keeps_float32=True)
+        return out
+
+    def bind(self, tensors, prefix, dtype, device) -> None:
+        super().bind(tensors, prefix, dtype, device)
+        h, p, r, v, c = self.num_heads, self.head_dim, self.rot_dim, self.value_dim, self.kv_rank
+        pad = lambda t: t if t.shape[0] % 8 == 0 else torch.cat([t, t.new_zeros((8 - t.shape[0] % 8, t.shape[1]))], dim=0)
+        self.dq_weight = self.w_uq = None
+        self.q_latent = 0
+        if self.q_rank is None:
+            first = tensors[prefix + "q"]
+        else:
+            first = tensors[prefix + "dq"]
+            self.q_latent = first.shape[0]
+            self.dq_weight = tensors[prefix + "dq.norm"].float().contiguous()
+            self.w_uq = tensors[prefix + "uq"].contiguous()
+            if self.w_uq.shape[1] != self.q_latent or self.dq_weight.shape[0] != self.q_latent:
+                raise ValueError(f"{prefix}dq, dq.norm and uq disagree on the query latent's size")
+        # (the parts of a row of the product's result start at multiples of 16 bytes)
+        first = pad(first)
+        self.c_offset = first.shape[0]
+        self.w_in = torch.cat([first, pad(tensors[prefix + "dkv"])], dim=0).contiguous()
+        self.dkv_weight = tensors[prefix + "dkv.norm"].float().contiguous()
+        # fold: [heads, C, P] so that (q_plain of head h) @ fold[h].T lies in the latent space
+        self.w_fold = tensors[prefix + "uk"].reshape(h, p, c).transpose(1, 2).contiguous()
+        # unfold: [heads, V, latent_dim] reads a head's weighted sum of latents
+        unfold = torch.zeros((h, v, self.latent_dim), dtype=dtype, device=device)
+        unfold[:, :, :c] = tensors[prefix + "uv"].reshape(h, v, c)
+        self.w_unfold = unfold.contiguous()
+        self.w_o = tensors[prefix + "o"].contiguous()
+        self.sinks = tensors[prefix + "sink"].float().contiguous() if self.sink else None
+
+    def warm_up(self, rows: int) -> None:
+        blank = lambda width: torch.zeros((rows, width), dtype=self.w_in.dtype, device=self.w_in.device)
+        linear(blank(self.hidden_size), self.w_in)
+        if self.w_uq is not None:
+            linear(blank(self.q_latent), self.w_uq)
+        linear(blank(self.num_heads * self.value_dim), self.w_o)
+
+    def forward(self, x: torch.Tensor, batch, view, writes: bool = True) -> torch.Tensor:
+        h, p, r, c = self.num_heads, self.head_dim, self.rot_dim, self.kv_rank
+        rotary = None
+        if self.position is not None and self.position.rotates:
+            if batch.max_context > self.position.max_position:
+                raise ValueError(f"position {batch.max_context - 1} is beyond the rotary table of {self.position.max_position}")
+            cos, sin = self.position.tables(x.device, positions_bound(batch))
+            rotary = (cos, sin, self.position.rotary_dim, getattr(self.position, "pairing", "halves") == "neighbours")
+        proj = linear(x, self.w_in)
+        q_latent = ops.latent_down(proj, 0, self.q_latent, self.c_offset, self.dq_weight, self.dkv_weight, c, r, rotary,
+                                   batch.positions, batch.seq_of_token, batch.seq_slot, view.block_table, view.k_pool,
+                                   view.v_pool, self.eps, write_kv=writes)
+        q = proj[:, : h * (p + r)] if q_latent is None else linear(q_latent, self.w_uq)
+        rows = ops.latent_queries(q, h, p, r, c, self.entry_dim, rotary, batch.positions)
+        ops.block_linear(q, self.w_fold, a_block=p + r, out=rows, out_offset=r, c_block=self.entry_dim)
+        shape = dict(window=self.window, scale=self.scale, sinks=self.sinks)
+        context = scored_attend(rows, batch, view, h, 1, self.entry_dim, self.latent_dim,
+                                ops.LATENT_MFMA_DIMS[self.mfma_dims] if self.mfma_dims else 0, shape)
+        return linear(ops.block_linear(context, self.w_unfold), self.w_o)
+
+
+register_part("mixer", "windowed_latent_attention", WindowedLatentAttention)

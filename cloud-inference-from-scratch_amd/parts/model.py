@@ -15,7 +15,7 @@ from ..kernels import ops
 from ..weights.loader import torch_dtype
 from ..weights.tensors import TensorSpec
 from .base import BLOCKS, build_part
-from .block import normalise
+from .block import normalise, whole_stream
 from .linear import StreamRows, linear
 
 
@@ -33,6 +33,8 @@ def _expected(spec: ModelSpec, blocks: list[Any], final_norm: Any) -> dict[str, 
     out.update(final_norm.expected_tensors(spec.final_norm_name + "."))
     if not spec.tie_word_embeddings:
         out[spec.head_name] = TensorSpec((spec.vocab_size, spec.hidden_size))
+    if spec.entry is not None:
+        out.update(build_part("entry", spec.entry).expected_tensors(spec.entry_name + "."))
     for index, block in enumerate(blocks):
         out.update(block.expected_tensors(spec.layer_prefix.format(index=index)))
     return out
@@ -57,7 +59,17 @@ class DecoderModel:
         self.keeps_embedding = any(call.adds_embedding for call in spec.order)
         if self.keeps_embedding and self.keeps_history:
             raise ValueError("a run order adds the embedding's rows again to layers that average over the depth: not built")
+        self.entry = build_part("entry", spec.entry) if spec.entry is not None else None
+        for call in spec.order:
+            if call.entry is not None and call.entry >= self.entry.times:
+                raise ValueError(f"layer {call.layer} is run behind entry {call.entry}, and there are {self.entry.times}")
+        if self.entry is not None and self.keeps_history:
+            raise ValueError("an entry step remakes a stream that is averaged over the depth: not built")
         calls = [self.blocks[call.layer] for call in spec.order]
+        # what runs behind each call, for blocks that make its first norm themselves; nothing where the stream is remade
+        # or added to in between
+        self.followers = [block if not (call.entry is not None or call.adds_embedding) else None
+                          for block, call in zip(calls[1:], spec.order[1:])] + [None]
         if len(set(map(id, calls))) == len(calls):  # (a layer that runs twice has no single successor)
             for block, follower in zip(calls, calls[1:] + [None]):
                 link = getattr(block, "link_next", None)
@@ -97,7 +109,8 @@ class DecoderModel:
     @property
     def graph_safe(self) -> bool:
         """Whether a decode step of this model may be captured in a graph."""
-        return all(getattr(block, "graph_safe", False) for block in self.blocks) and self.final_norm.graph_safe
+        return (all(getattr(block, "graph_safe", False) for block in self.blocks) and self.final_norm.graph_safe
+                and (self.entry is None or self.entry.graph_safe))
 
     def load(self, source: Any, dtype: str, device: str | torch.device) -> "DecoderModel":
         """Bind weights from a source (``SafetensorsSource`` or ``RandomSource``)."""
@@ -116,6 +129,12 @@ class DecoderModel:
         self.embedding = tensors[self.spec.embedding_name].contiguous()
         self.head = self.embedding if self.spec.tie_word_embeddings else tensors[self.spec.head_name].contiguous()
         self.final_norm.bind(tensors, self.spec.final_norm_name + ".", self.dtype, device)
+        # a factor on the logits goes into the final norm, in float32, where that norm takes it
+        self.folded_scale = hasattr(self.final_norm, "fold_scale")
+        if self.folded_scale and self.spec.logit_scale != 1.0:
+            self.final_norm.fold_scale(self.spec.logit_scale)
+        if self.entry is not None:
+            self.entry.bind(tensors, self.spec.entry_name + ".", self.dtype, device)
         for index, block in enumerate(self.blocks):
             block.bind(tensors, self.spec.layer_prefix.format(index=index), self.dtype, device)
         return self
@@ -126,6 +145,9 @@ class DecoderModel:
         before the first request.  Layers of one specification share their shapes: one of each runs."""
         if self.dtype != torch.bfloat16 or self.device.type != "cuda":
             return
+        if self.entry is not None:
+            for rows in row_counts:
+                self.entry.warm_up(rows)
         seen = set()
         for block in self.blocks:
             key = repr(block.spec)
@@ -144,26 +166,44 @@ class DecoderModel:
             history = torch.empty((len(self.spec.order) + 1, batch.token_ids.shape[0], self.embedding.shape[1]),
                                   dtype=torch.float32, device=self.embedding.device)
         first = self.blocks[self.spec.order[0].layer] if self.spec.order else None
-        rows = None
-        if getattr(first, "reads_stream", False) and self.embedding.dtype != torch.float32:
+        rows = joint = None
+        if self.entry is not None:
+            # (a row's halves: the stream, which the block in front of an entry leaves there, and the embedding's row)
+            joint = self.entry.joint(batch.token_ids.shape[0])
+            rows = joint[:, self.embedding.shape[1]:]
+        elif getattr(first, "reads_stream", False) and self.embedding.dtype != torch.float32:
             # a first layer whose products read the stream itself: the embedding kernel also leaves it in their type
             rows = torch.empty((batch.token_ids.shape[0], self.embedding.shape[1]), dtype=self.embedding.dtype,
                                device=self.embedding.device)
         residual = ops.embed(self.embedding, batch.token_ids, feed=batch.token_feed, pool=batch.token_pool,
                              out=history[0] if history is not None else None, scale=self.spec.embedding_scale,
                              rows=rows)
-        pending = StreamRows(rows) if rows is not None else None
+        pending = StreamRows(rows) if rows is not None and joint is None else None
         embedded = residual.clone() if self.keeps_embedding else None
-        for call in self.spec.order:
+        left = False  # whether the stream lies in the joint rows already
+        for index, call in enumerate(self.spec.order):
             block = self.blocks[call.layer]
             extra = {"history": history} if getattr(block, "keeps_history", False) else {}
             if call.adds_embedding:
                 extra["plus"] = embedded
+            if call.entry is not None:
+                stream = joint[:, : residual.shape[1]]
+                if not left:
+                    stream.copy_(whole_stream(residual, pending))
+                residual, extra["plus"] = self.entry.forward(joint, call.entry)
+                pending = None
+            left = False
+            if getattr(block, "takes_follower", False):
+                extra["follower"] = self.followers[index]
+                if index + 1 < len(self.spec.order) and self.spec.order[index + 1].entry is not None:
+                    extra["stream_rows"], left = joint[:, : residual.shape[1]], True
             residual, pending = block.forward(residual, pending, batch, cache.view(call.cache), call.writes, **extra)
         if batch.logit_rows.shape[0] == 0:  # a step of prompt portions that end before their prompts do
             return torch.empty((0, self.head.shape[0]), dtype=torch.float32, device=residual.device)
         selected = normalise(self.final_norm, residual, pending, self.dtype, rows=batch.logit_rows)
         logits = linear(selected, self.head, None, out_dtype=torch.float32)
+        if self.spec.logit_scale != 1.0 and not self.folded_scale:
+            logits.mul_(self.spec.logit_scale)
         if self.spec.logit_softcap is not None:
             ops.soft_cap_(logits, self.spec.logit_softcap)
         return logits

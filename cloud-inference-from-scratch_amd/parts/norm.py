@@ -1,4 +1,4 @@
-"""RMSNorm, fused with the residual add that precedes it.
+"""RMSNorm (and layer norm), fused with the residual add that precedes it.
 
 Formula of the reference's ``rms_norm`` (src/cloud_engine/attention.py:52-57):
 ``x * rsqrt(mean(x^2) + eps) * weight`` with float32 statistics.  The reference
@@ -8,7 +8,7 @@ the multiply is float32 too and the result is rounded once.
 
 from __future__ import annotations
 
-from typing import Optional
+from typing import Any, Optional
 
 import torch
 
@@ -153,27 +153,104 @@ class GroupedRMSNorm(Part):
                                   plus=plus, **extra)
 
 
-def _add_normed(self, residual: torch.Tensor, branch, out_dtype: torch.dtype, want_rows: bool = False,
-                weight: Optional[torch.Tensor] = None, then: Optional[torch.Tensor] = None):
-    """``residual += norm(branch) * weight`` in float32 and in place, for a norm of one group.  ``branch``: a
+def _addends(branch) -> tuple[Optional[torch.Tensor], dict]:
+    """A branch in the form the adding kernels take: its main tensor, and whatever else is summed with it."""
+    if isinstance(branch, SummedBranch):
+        return branch.main, dict(parts=branch.parts, part_weight=branch.weights, branch_gate=branch.main_gate)
+    if isinstance(branch, WeightedPair):
+        return branch.first, dict(branch2=branch.second, scales=branch.scales)
+    return branch, {}
+
+
+def _add_normed(self, residual: torch.Tensor, branch, out_dtype: torch.dtype, scale: Optional[torch.Tensor] = None,
+                then: Any = None, stream_rows: Optional[torch.Tensor] = None) -> Optional[torch.Tensor]:
+    """``residual += scale * norm(branch)`` in float32 and in place, for a norm of one group.  ``branch``: a
     tensor, a ``SummedBranch`` (rows still to be summed, with their weights and the gate on its main tensor) or a
-    ``WeightedPair``.  ``weight`` (float32 [H]) stands in for the norm's own where the caller has folded a scale per
-    channel into it.  ``then`` (float32 [H]): the RMS norm of the new stream under that weight comes back too.
-    Returns what ``ops.branch_norm_add`` returns."""
+    ``WeightedPair``.  ``scale`` (float32 [H]) is what :meth:`scaled` made.  ``then``: a norm of the same kind, under which
+    the new stream's rows come back.  ``stream_rows`` ([T, H] in ``out_dtype``) takes the new stream itself."""
     if self.groups != 1:
         raise ValueError("a norm on a sublayer's output takes its statistics over the whole row")
-    extra = {}
-    if isinstance(branch, SummedBranch):
-        extra = dict(parts=branch.parts, part_weight=branch.weights, branch_gate=branch.main_gate)
-        branch = branch.main
-    elif isinstance(branch, WeightedPair):
-        extra = dict(branch2=branch.second, scales=branch.scales)
-        branch = branch.first
-    return ops.branch_norm_add(residual, branch, self.weight if weight is None else weight, self.eps, out_dtype,
-                               want_rows=want_rows, next_weight=then, **extra)
+    branch, extra = _addends(branch)
+    made = ops.branch_norm_add(residual, branch, self.weight if scale is None else scale, self.eps, out_dtype,
+                               want_rows=stream_rows is not None, next_weight=None if then is None else then.weight_f32, **extra)
+    rows, normed = made if then is not None else (made, None)
+    if stream_rows is not None:
+        stream_rows.copy_(rows)
+    return normed
+
+
+def _joins_into(self, then: Any) -> bool:
+    """Whether ``add_normed`` can make the rows of the norm ``then`` in the same kernel."""
+    return isinstance(then, GroupedRMSNorm) and then.groups == 1 and then.eps == self.eps and then.size == self.size
+
+
+def _scaled(self, scale: torch.Tensor) -> torch.Tensor:
+    """What ``add_normed`` takes as ``scale``: a scale per channel on the norm's output, with the weight multiplied in."""
+    return (self.weight_f32 * scale.float()).contiguous()
 
 
 GroupedRMSNorm.add_normed = _add_normed
+GroupedRMSNorm.joins_into = _joins_into
+GroupedRMSNorm.scaled = _scaled
+
+
+class LayerNorm(Part):
+    """``(x - mean) / sqrt(variance + eps) * weight + bias`` with the variance the mean of the squared deviations.  The
+    weight's tensor is named like the norm itself, the bias's ``<name>.b``.  In front of a sublayer the kernel that norms
+    also adds what the stream is owed (a branch's tensor, and ``plus``: float32 rows, or one row for all); on a sublayer's
+    output it norms whatever the branch sums to, adds it and makes the layer norm that comes next.  Sums, statistics and
+    scaling are float32.  ``fold_scale`` multiplies weight and bias (a factor on what the norm feeds into a product)."""
+
+    graph_safe = True
+    takes_plus = True
+
+    def __init__(self, size: int, eps: float) -> None:
+        if size <= 0 or not eps > 0:
+            raise ValueError(f"a norm needs a positive size and eps, got {size}, {eps}")
+        if size > ops.MAX_NORM_WIDTH:
+            raise ValueError(f"the norm kernels take rows of up to {ops.MAX_NORM_WIDTH} numbers, not {size}")
+        self.size, self.eps = size, float(eps)
+        self.weight_f32: Optional[torch.Tensor] = None
+        self.bias_f32: Optional[torch.Tensor] = None
+
+    def expected_tensors(self, prefix: str) -> dict[str, TensorSpec]:
+        name = prefix.rstrip(".")
+        return {name: TensorSpec((self.size,), init="norm", keeps_float32=True),
+                name + ".b": TensorSpec((self.size,), keeps_float32=True)}
+
+    def bind(self, tensors, prefix, dtype, device) -> None:
+        super().bind(tensors, prefix, dtype, device)
+        name = prefix.rstrip(".")
+        self.weight_f32 = tensors[name].float().contiguous()
+        self.bias_f32 = tensors[name + ".b"].float().contiguous()
+
+    def fold_scale(self, factor: float) -> None:
+        self.weight_f32 = (self.weight_f32 * factor).contiguous()
+        self.bias_f32 = (self.bias_f32 * factor).contiguous()
+
+    def forward(self, residual: torch.Tensor, branch, out_dtype: torch.dtype, rows: Optional[torch.Tensor] = None,
+                plus: Optional[torch.Tensor] = None) -> torch.Tensor:
+        if isinstance(branch, (Added, RowSumsq)):
+            branch = None
+        if isinstance(branch, SummedBranch):
+            raise ValueError("this norm adds one tensor to the stream: a branch that is still a sum is not its to add")
+        return ops.layer_norm_add(residual, branch, self.weight_f32, self.bias_f32, self.eps, out_dtype, rows=rows, plus=plus)
+
+    def joins_into(self, then: Any) -> bool:
+        return isinstance(then, LayerNorm) and then.eps == self.eps and then.size == self.size
+
+    def scaled(self, scale: torch.Tensor) -> tuple[torch.Tensor, torch.Tensor]:
+        return (self.weight_f32 * scale.float()).contiguous(), (self.bias_f32 * scale.float()).contiguous()
+
+    def add_normed(self, residual: torch.Tensor, branch, out_dtype: torch.dtype, scale: Optional[tuple] = None,
+                   then: Any = None, stream_rows: Optional[torch.Tensor] = None) -> Optional[torch.Tensor]:
+        branch, extra = _addends(branch)
+        weight, bias = (self.weight_f32, self.bias_f32) if scale is None else scale
+        return ops.branch_layer_norm_add(residual, branch, weight, bias, self.eps, out_dtype, rows_out=stream_rows,
+                                         next_norm=None if then is None else (then.weight_f32, then.bias_f32), **extra)
+
+
+register_part("norm", "layer_norm", LayerNorm)
 
 register_part("norm", "rms_norm", RMSNorm)
 register_part("norm", "rms_norm_groups", GroupedRMSNorm)

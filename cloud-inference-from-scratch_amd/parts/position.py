@@ -32,6 +32,12 @@ from .base import Part, register_part
 _TABLES: dict[tuple, tuple[torch.Tensor, torch.Tensor]] = {}
 
 
+def positions_bound(batch) -> int:
+    """Positions a step's rotation tables have to reach: its longest context, or, for a step that is captured and
+    replayed with other contexts, the bound it was captured for."""
+    return batch.static_plan.max_keys if batch.static_plan is not None else batch.max_context
+
+
 class RotaryHalf(Part):
     graph_safe = True
     rotates = True

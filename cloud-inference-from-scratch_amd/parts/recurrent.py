@@ -41,8 +41,8 @@ from ..config.specs import PartSpec
 from ..kernels import ops
 from ..weights.tensors import TensorSpec
 from .base import Part, build_part, register_part
-from .latent_attention import positions_bound
 from .linear import linear
+from .position import positions_bound
 
 
 class Retention(Part):

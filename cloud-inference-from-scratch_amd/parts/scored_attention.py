@@ -16,20 +16,25 @@ the position in other ways.  Every step is a parameter of the part and may be le
   as ``rotary_pairs``, applied after the heads' norm);
 * a sink (``sink``: one learned number per head whose exponential stands in the softmax's denominator, and
   nowhere else);
-* a gate on every head's output (``head_gate``: ``sigmoid(W_g x)_h``, read from the layer's own input);
+* a gate on every head's output (``head_gate``: ``sigmoid(W_g x)_h``, read from the layer's own input), or on every
+  number of the heads' outputs (``output_gate``: ``sigmoid(W_g x)`` has heads x vdim numbers);
+* two maps a head (``differential = d``): queries and keys are projected as pairs of ``head_dim`` numbers, each map is a
+  softmax of its own over the same values, and with ``lambda = exp(lq1 . lk1) - exp(lq2 . lk2) + d`` (learned vectors of
+  ``head_dim`` numbers) a head's output is ``a1 - lambda a2``, divided by its root mean square, times ``1 - d``;
 * key and value heads of different sizes;
 * no keys and values of its own (``own_kv=False``): the layer has no tensors for them and reads the cache unit that
   another layer of the same head sizes writes, with its own queries, mask and everything else.
 
 One product makes queries, keys, values and gate logits; one kernel norms and scales the heads, lays the queries
 out and writes the cache (``ops.heads_prepare``); the attention kernel shapes the scores, and applies sink and
-gate in its epilogue: bfloat16 with head sizes up to 128 on the matrix cores (``ops.scored_attention_mfma``, the
-heads zero-padded to 64 or 128 numbers: no score and no output changes), anything else, and float32, in the
-generic form.  Norm statistics, the logarithm, scores, softmax, value sums and the gate are float32.
+gate in its epilogue (and there joins the two maps of a head): bfloat16 with head sizes up to 128 on the matrix cores
+(``ops.scored_attention_mfma``, the heads zero-padded to 64 or 128 numbers, a map of a pair to 32, 64 or 128: no score
+and no output changes), anything else, and float32, in the generic form.  Norm statistics, the logarithm, scores, softmax, value sums and the gate are float32.
 """
 
 from __future__ import annotations
 
+import math
 import warnings
 from typing import Optional
 
@@ -40,8 +45,8 @@ from ..config.specs import PartSpec
 from ..kernels import ops
 from ..weights.tensors import TensorSpec
 from .base import Part, build_part, register_part
-from .latent_attention import positions_bound
 from .linear import linear
+from .position import positions_bound
 
 _SAID_GENERIC: set = set()
 PROMPT_ROW_TILES = 2  # tiles of 16 (token, head) rows that a workgroup of the matrix-core form takes of a prompt's portion
@@ -59,7 +64,8 @@ class ScoredAttention(Part):
                  q_temperature: Optional[tuple] = None, softcap: Optional[float] = None,
                  slope_base: Optional[float] = None, sink: bool = False, head_gate: bool = False,
                  chunk: Optional[int] = None, qkv_bias: bool = False, position: Optional[PartSpec] = None,
-                 keep_first: int = 0, own_kv: bool = True) -> None:
+                 keep_first: int = 0, own_kv: bool = True, output_gate: bool = False,
+                 differential: Optional[float] = None) -> None:
         for name, value in (("hidden_size", hidden_size), ("num_heads", num_heads), ("num_kv_heads", num_kv_heads),
                             ("head_dim", head_dim), ("value_dim", value_dim)):
             if isinstance(value, bool) or not isinstance(value, int) or value < 1:
@@ -94,31 +100,45 @@ class ScoredAttention(Part):
         self.slope_base, self.sink, self.head_gate = slope_base, bool(sink), bool(head_gate)
         self.chunk, self.qkv_bias = chunk, bool(qkv_bias)
         self.keep_first, self.own_kv = keep_first, bool(own_kv)
+        self.output_gate = bool(output_gate)
+        self.differential = float(differential) if differential is not None else None
+        self.maps = 1 if differential is None else 2
+        if self.output_gate and self.head_gate:
+            raise ValueError("one gate: a number a head or a number for every number of it")
+        if self.maps == 2 and (self.sink or qk_norm is not None or not self.own_kv):
+            raise ValueError("two maps a head come with neither a sink nor a norm on the heads, and with keys of their own")
         self.position = build_part("position", position) if position is not None else None
         if self.position is not None and self.position.rotates and self.position.rotary_dim > head_dim:
             raise ValueError(f"{self.position.rotary_dim} turning numbers in heads of {head_dim}")
         # the head sizes the kernels and the cache see: those of the matrix-core form where it has them
-        sizes = tuple(next((s for s in (64, 128) if s >= n), None) for n in (head_dim, value_dim))
-        self.mfma_dims = sizes if sizes in ops.SCORED_MFMA_DIMS else None
+        if self.maps == 2:
+            fitting = [pair for pair in ops.DIFFERENTIAL_MFMA_DIMS if pair[0] >= head_dim and pair[1] >= value_dim]
+            self.mfma_dims = min(fitting, key=lambda pair: (pair[0], pair[1])) if fitting else None
+            self.most_row_tiles = ops.DIFFERENTIAL_MFMA_DIMS[self.mfma_dims] if fitting else 0
+        else:
+            sizes = tuple(next((s for s in (64, 128) if s >= n), None) for n in (head_dim, value_dim))
+            self.mfma_dims = sizes if sizes in ops.SCORED_MFMA_DIMS else None
+            self.most_row_tiles = 4
         self.kernel_dim, self.kernel_vdim = self.mfma_dims or (_round8(head_dim), _round8(value_dim))
 
     def cache_need(self) -> PagedKV:
         # (a chunk's keys all lie inside a window of the chunk's length: pages behind it go back to the pool)
-        return PagedKV(self.num_kv_heads, self.kernel_dim, self.window if self.chunk is None else self.chunk,
-                       value_dim=self.kernel_vdim if self.kernel_vdim != self.kernel_dim else None,
+        width = self.maps * self.kernel_dim
+        return PagedKV(self.num_kv_heads, width, self.window if self.chunk is None else self.chunk,
+                       value_dim=self.kernel_vdim if self.kernel_vdim != width else None,
                        keep_first=self.keep_first)
 
     def expected_tensors(self, prefix: str) -> dict[str, TensorSpec]:
         h, g, d, v, width = self.num_heads, self.num_kv_heads, self.head_dim, self.value_dim, self.hidden_size
-        out = {prefix + "q": TensorSpec((h * d, width))}
+        out = {prefix + "q": TensorSpec((h * self.maps * d, width))}
         if self.own_kv:
-            out[prefix + "k"] = TensorSpec((g * d, width))
+            out[prefix + "k"] = TensorSpec((g * self.maps * d, width))
             out[prefix + "v"] = TensorSpec((g * v, width))
         out[prefix + "o"] = TensorSpec((width, h * v))
         if self.qkv_bias:
-            out[prefix + "q.b"] = TensorSpec((h * d,))
+            out[prefix + "q.b"] = TensorSpec((h * self.maps * d,))
             if self.own_kv:
-                out[prefix + "k.b"] = TensorSpec((g * d,))
+                out[prefix + "k.b"] = TensorSpec((g * self.maps * d,))
                 out[prefix + "v.b"] = TensorSpec((g * v,))
         if self.qk_norm in ("weight", "whole"):
             whole = self.qk_norm == "whole"
@@ -127,8 +147,11 @@ class ScoredAttention(Part):
                 out[prefix + "k.norm"] = TensorSpec((g * d if whole else d,), init="norm", keeps_float32=True)
         if self.sink:
             out[prefix + "sink"] = TensorSpec((h,), keeps_float32=True)
-        if self.head_gate:
-            out[prefix + "g"] = TensorSpec((h, width))
+        if self.head_gate or self.output_gate:
+            out[prefix + "g"] = TensorSpec((h if self.head_gate else h * v, width))
+        if self.maps == 2:
+            for name in ("lq1", "lk1", "lq2", "lk2"):
+                out[prefix + name] = TensorSpec((d,), keeps_float32=True)
         return out
 
     def bind(self, tensors, prefix, dtype, device) -> None:
@@ -137,9 +160,10 @@ class ScoredAttention(Part):
         blocks = [tensors[prefix + "q"]]
         if self.own_kv:
             blocks += [tensors[prefix + "k"], tensors[prefix + "v"]]
+        d *= self.maps
         self.offsets = (0, h * d, h * d + g * d) if self.own_kv else (0, 0, 0)
         self.gate_offset = None
-        if self.head_gate:
+        if self.head_gate or self.output_gate:
             # gate logits ride in the same product, on columns that start at a multiple of 8 (and the row is
             # padded to one), so that the rows of the result stay 16-byte aligned
             pad = lambda rows: blocks[0].new_zeros((rows, self.hidden_size))
@@ -148,8 +172,9 @@ class ScoredAttention(Part):
                 blocks.append(pad(8 - used % 8))
             self.gate_offset = _round8(used)
             blocks.append(tensors[prefix + "g"])
-            if h % 8:
-                blocks.append(pad(8 - h % 8))
+            gates = blocks[-1].shape[0]
+            if gates % 8:
+                blocks.append(pad(8 - gates % 8))
         self.w_in = torch.cat(blocks, dim=0).contiguous()
         self.b_in = None
         if self.qkv_bias:
@@ -161,6 +186,10 @@ class ScoredAttention(Part):
             self.q_weight = tensors[prefix + "q.norm"].float().contiguous()
             if self.own_kv:
                 self.k_weight = tensors[prefix + "k.norm"].float().contiguous()
+        self.pair = None  # what joins the two maps of a head: lambda, the factor behind the norm, its eps
+        if self.maps == 2:
+            dot = lambda n: float((tensors[f"{prefix}lq{n}"].float() * tensors[f"{prefix}lk{n}"].float()).sum())
+            self.pair = (math.exp(dot(1)) - math.exp(dot(2)) + self.differential, 1.0 - self.differential, self.eps)
         self.sinks = tensors[prefix + "sink"].float().contiguous() if self.sink else None
         self.slopes = None
         if self.slope_base is not None:
@@ -191,60 +220,74 @@ class ScoredAttention(Part):
         q = ops.heads_prepare(proj, self.offsets, self.num_heads, self.num_kv_heads, self.head_dim, self.value_dim,
                               self.kernel_dim, self.kernel_vdim, self.qk_norm, self.q_weight, self.k_weight, self.eps,
                               self.q_temperature, batch.positions, batch.seq_of_token, batch.seq_slot,
-                              view.block_table, view.k_pool, view.v_pool, batch.tokens, write_kv=writes, rotary=rotary)
-        gate = proj[:, self.gate_offset:] if self.head_gate else None
+                              view.block_table, view.k_pool, view.v_pool, batch.tokens, write_kv=writes, rotary=rotary,
+                              maps=self.maps)
+        gate = proj[:, self.gate_offset:] if self.gate_offset is not None else None
         context = self.attend(q, gate, batch, view)
         return linear(context, self.w_o)
 
     def attend(self, q: torch.Tensor, gate, batch, view) -> torch.Tensor:
         shape = dict(window=self.window, scale=self.scale, softcap=self.softcap, slopes=self.slopes,
-                     sinks=self.sinks, gate=gate, chunk=self.chunk, keep_first=self.keep_first)
-        h, g = self.num_heads, self.num_kv_heads
-        group = h // g
-        page_size = view.page_size
-        if q.dtype == torch.bfloat16 and self.mfma_dims and group <= 64 and page_size >= 4 and not page_size & (page_size - 1):
-            # rows of a tile: a token's heads of one key head, and as many tokens as fill the tile
-            least = 1 if group <= 16 else 2 if group <= 32 else 4
-            # the most keys a token sees in this step (a captured step: in any of its replays)
-            bound = batch.static_plan.max_keys if batch.static_plan is not None else batch.max_context
-            reach = self.window if self.chunk is None else self.chunk  # the most keys a token sees, if bounded
-            if reach is not None and self.keep_first:
-                reach += -(-self.keep_first // 32) * 32 + 32  # (the kept first keys are walked in whole blocks of 32)
-            bound = bound if reach is None else min(bound, reach)
+                     sinks=self.sinks, gate=gate, chunk=self.chunk, keep_first=self.keep_first, gate_wide=self.output_gate,
+                     real_vdim=self.value_dim, differential=self.pair)
+        return scored_attend(q, batch, view, self.num_heads, self.num_kv_heads, self.kernel_dim, self.kernel_vdim,
+                             self.most_row_tiles if self.mfma_dims else 0, shape)
 
-            def shares(tiles: int, span: int) -> dict:
-                """Few tiles over many keys: the keys in shares of at least 128, about two workgroups a compute unit."""
-                reach = bound + span + 32                        # a tile's range starts at a multiple of 32
-                wanted = min(2 * ops.compute_units() // max(tiles * g, 1), reach // 128)
-                if wanted < 2:
-                    return {}
-                per = -(-(-(-reach // wanted)) // 128) * 128
-                return dict(n_splits=-(-reach // per), keys_per_split=per)
 
-            if batch.static_plan is not None and batch.static_plan.decode_rows in (None, batch.sequences):
-                # a captured step of single tokens: tile i is sequence i, nothing comes from the host
-                return ops.scored_attention_mfma(q, view.k_pool, view.v_pool, view.block_table, None, None,
-                                                 batch.sequences, batch.seq_slot, batch.seq_start, batch.seq_q_len,
-                                                 batch.q_start_loc, batch.tokens, h, g, self.kernel_dim,
-                                                 self.kernel_vdim, 1, least, **shape, **shares(batch.sequences, 1))
-            row_tiles = max(least, PROMPT_ROW_TILES if batch.max_q_len * group > 16 else 1)
-            while row_tiles > least and -(-batch.tokens * group // (16 * row_tiles)) * g < ops.compute_units():
-                row_tiles //= 2  # (fewer rows a tile where the tiles would not fill the compute units)
-            per_tile = (16 * row_tiles) // group
-            tile_seq, tile_q0, n_tiles = batch.tiles(per_tile, decode=None)
-            return ops.scored_attention_mfma(q, view.k_pool, view.v_pool, view.block_table, tile_seq, tile_q0, n_tiles,
-                                             batch.seq_slot, batch.seq_start, batch.seq_q_len, batch.q_start_loc,
-                                             batch.tokens, h, g, self.kernel_dim, self.kernel_vdim, per_tile,
-                                             row_tiles, **shape, **shares(n_tiles, per_tile))
-        if q.dtype == torch.bfloat16 and (self.kernel_dim, self.kernel_vdim, group, page_size) not in _SAID_GENERIC:
-            _SAID_GENERIC.add((self.kernel_dim, self.kernel_vdim, group, page_size))
-            warnings.warn(f"bfloat16 attention with heads of {self.head_dim} and {self.value_dim} numbers, {group} query "
-                          f"heads per key head and pages of {page_size} takes the generic kernel (the matrix-core form "
-                          f"takes heads of up to 128 numbers, up to 64 heads per key head and pages of a power of two >= 4)",
-                          RuntimeWarning, stacklevel=2)
-        return ops.scored_attention_generic(q, view.k_pool, view.v_pool, view.block_table, batch.positions,
-                                            batch.seq_of_token, batch.seq_slot, batch.tokens, h, g, self.kernel_dim,
-                                            self.kernel_vdim, **shape)
+def scored_attend(q: torch.Tensor, batch, view, h: int, g: int, dim: int, vdim: int, most_row_tiles: int,
+                  shape: dict) -> torch.Tensor:
+    """Pick the attention kernel for this step's rows: ``h`` query heads on ``g`` key heads of ``dim`` and ``vdim``
+    numbers as the kernels see them.  ``most_row_tiles``: the most tiles of 16 rows a workgroup of the matrix-core form
+    takes at these sizes (0: it does not take them).  ``shape``: what both kernels are told about the scores."""
+    window, chunk, keep_first = shape["window"], shape.get("chunk"), shape.get("keep_first", 0)
+    maps = 1 if shape.get("differential") is None else 2
+    group = h // g
+    page_size = view.page_size
+    # rows of a tile: a token's heads of one key head (of each map), and as many tokens as fill the tile
+    least = maps * (1 if group <= 16 else 2 if group <= 32 else 4)
+    if (q.dtype == torch.bfloat16 and group <= 64 and least <= most_row_tiles and page_size >= 4
+            and not page_size & (page_size - 1)):
+        # the most keys a token sees in this step (a captured step: in any of its replays)
+        bound = batch.static_plan.max_keys if batch.static_plan is not None else batch.max_context
+        reach = window if chunk is None else chunk  # the most keys a token sees, if bounded
+        if reach is not None and keep_first:
+            reach += -(-keep_first // 32) * 32 + 32  # (the kept first keys are walked in whole blocks of 32)
+        bound = bound if reach is None else min(bound, reach)
+
+        def shares(tiles: int, span: int) -> dict:
+            """Few tiles over many keys: the keys in shares of at least 128, about two workgroups a compute unit."""
+            reach = bound + span + 32                        # a tile's range starts at a multiple of 32
+            wanted = min(2 * ops.compute_units() // max(tiles * g, 1), reach // 128)
+            if wanted < 2:
+                return {}
+            per = -(-(-(-reach // wanted)) // 128) * 128
+            return dict(n_splits=-(-reach // per), keys_per_split=per)
+
+        if batch.static_plan is not None and batch.static_plan.decode_rows in (None, batch.sequences):
+            # a captured step of single tokens: tile i is sequence i, nothing comes from the host
+            return ops.scored_attention_mfma(q, view.k_pool, view.v_pool, view.block_table, None, None,
+                                             batch.sequences, batch.seq_slot, batch.seq_start, batch.seq_q_len,
+                                             batch.q_start_loc, batch.tokens, h, g, dim, vdim, 1, least, **shape,
+                                             **shares(batch.sequences, 1))
+        wanted = PROMPT_ROW_TILES * maps
+        row_tiles = min(most_row_tiles, max(least, wanted if batch.max_q_len * group > 16 else maps))
+        while row_tiles > least and -(-batch.tokens * group * maps // (16 * row_tiles)) * g < ops.compute_units():
+            row_tiles //= 2  # (fewer rows a tile where the tiles would not fill the compute units)
+        per_tile = (16 * row_tiles) // (group * maps)
+        tile_seq, tile_q0, n_tiles = batch.tiles(per_tile, decode=None)
+        return ops.scored_attention_mfma(q, view.k_pool, view.v_pool, view.block_table, tile_seq, tile_q0, n_tiles,
+                                         batch.seq_slot, batch.seq_start, batch.seq_q_len, batch.q_start_loc,
+                                         batch.tokens, h, g, dim, vdim, per_tile, row_tiles, **shape,
+                                         **shares(n_tiles, per_tile))
+    if q.dtype == torch.bfloat16 and (dim, vdim, group, page_size) not in _SAID_GENERIC:
+        _SAID_GENERIC.add((dim, vdim, group, page_size))
+        warnings.warn(f"bfloat16 attention with heads of {dim} and {vdim} numbers, {group} query heads per key head and pages "
+                      f"of {page_size} takes the generic kernel (the matrix-core form takes heads of up to 128 numbers, pairs "
+                      f"of maps of up to 128 with values of up to 256, latents as ops.LATENT_MFMA_DIMS lists them, a token's "
+                      f"heads on up to 64 rows and pages of a power of two >= 4)",
+                      RuntimeWarning, stacklevel=2)
+    return ops.scored_attention_generic(q, view.k_pool, view.v_pool, view.block_table, batch.positions,
+                                        batch.seq_of_token, batch.seq_slot, batch.tokens, h, g, dim, vdim, **shape)
 
 
 register_part("mixer", "scored_attention", ScoredAttention)
