@@ -5,7 +5,7 @@
     python bench.py [--gpus 1] [--steps K] [--warmup W] [--batch 8] [--context 4096]
                     [--shape 0.5b|3b|7b|14b|32b|72b] [--layers N] [--long-contexts 32768]
                     [--mixed-portions 16,64,248] [--other-shapes 7b,14b]
-    python bench.py --design polosun|givizen|nokipel|senuvik [--design-shapes 3b,7b] [--design-layers 12]
+    python bench.py --design polosun|givizen|nokipel|senuvik|nopunex [--design-shapes 3b,7b] [--design-layers 12]
 
 A "step" is one decode step of the whole engine (scheduler iteration: plan,
 step function, sampling, token hand-over).  Protocol after the reference's
@@ -50,7 +50,12 @@ mixing, and window attention on another layer's keys in turn; a dense
 feed-forward and routed experts) beside the Nokipel model of equal width, head
 sizes, expert sizes, vocabulary and layer count, the closest of the engine's
 models: memories of fixed size beside attention, dense and routed
-feed-forwards.
+feed-forwards.  ``--design nopunex`` measures the Nopunex design (the gated
+delta rule, latent attention under a window and differential attention in
+chunks in turn, each with a dense feed-forward) beside the Polosun model of
+equal width, memory and latent sizes, feed-forward, vocabulary and layer count,
+the closest of the engine's models: a memory of outer products, latent
+attention, dense feed-forwards.
 """
 
 from __future__ import annotations
@@ -518,11 +523,75 @@ def senuvik_costs(config, batch: int, context: float, tokens: int, elem: int) ->
     return moved, flops
 
 
+NOPUNEX_REACH = 1024
+
+
+def nopunex_raw(shape: dict, layers: int) -> dict:
+    """A Nopunex configuration with the width, feed-forward size and vocabulary of a Qwen2.5 shape and layers of realistic
+    proportions: the gated delta rule (heads of 128 x 128, two to a key head, as many numbers of memory as Polosun's
+    retention keeps; 4 taps), latent attention (Polosun's heads of 128 + 32 and latent of 96, queries from a latent of a
+    quarter of the width, a window of 1,024 tokens, stretched frequencies), differential attention (the shape's heads, two
+    maps of half a head each over its values, chunks of 1,024 tokens) in turn, each with a dense feed-forward.  All layers
+    form one pass, which begins with the joining product."""
+    width = shape["hidden_size"]
+    heads, kv_heads = shape["num_attention_heads"], shape["num_key_value_heads"]
+    dim = width // heads
+    mlp = {"kind": "dense", "ff": shape["intermediate_size"]}
+    kinds = [
+        {"type": "delta", "mlp": mlp,
+         "mixer": {"heads": width // 128, "kv_heads": width // 256, "dim": 128, "vdim": 128, "conv": 4}},
+        {"type": "latent_attention", "mlp": mlp,
+         "mixer": {"heads": width // 128, "dim": 128, "rot_dim": 32, "vdim": 128, "q_rank": width // 4, "kv_rank": 96,
+                   "scale": 160 ** -0.5, "mask": {"size": NOPUNEX_REACH},
+                   "rot": {"base": 1000000.0, "dims": 32,
+                           "scaling": {"factor": 4.0, "fast": 32.0, "original": 8192, "slow": 1.0}}}},
+        {"type": "attention", "mlp": mlp,
+         "mixer": {"heads": heads, "kv_heads": kv_heads, "dim": dim // 2, "vdim": dim, "scale": (dim // 2) ** -0.5, "diff": 0.5,
+                   "mask": {"size": NOPUNEX_REACH}, "rot": {"base": 1000000.0, "dims": dim // 2}}},
+    ]
+    return {"architecture": "Nopunex", "vocab": shape["vocab_size"], "width": width, "norm": {"eps": 1e-6}, "logit_scale": 1.0,
+            "loop": {"start": 0, "stop": layers, "times": 1}, "layers": [kinds[i % 3] for i in range(layers)]}
+
+
+def nopunex_costs(config, batch: int, context: float, tokens: int, elem: int) -> tuple[float, float]:
+    """(bytes one decode step has to move, flops of a prefill of ``tokens`` tokens) for a Nopunex configuration whose
+    layers pass once: every weight once (the embedding is only looked up), each request's latents and keys and values
+    inside the window or the token's chunk, each memory read and written in float32; products at two flops per weight and
+    token (the latent's expansions are folded into queries and outputs: as many flops as their weights), attention over
+    the keys each token sees, for a latent in the latent's own space, the memories' updates and both of their reads."""
+    from cie_amd.parts.model import expected_tensors
+
+    expected = expected_tensors(config.model_spec())
+    weights = sum(int(__import__("math").prod(spec.shape)) for name, spec in expected.items()
+                  if name != "embed" and not spec.optional)
+    head = config.vocab_size * config.hidden_size
+    moved, other = float(weights * elem), 0.0
+    for layer in config.raw["layers"]:
+        m = layer["mixer"]
+        if layer["type"] == "delta":
+            moved += batch * 2 * m["heads"] * m["dim"] * m["vdim"] * 4
+            other += 3 * 2.0 * tokens * m["heads"] * m["dim"] * m["vdim"]
+        elif layer["type"] == "latent_attention":
+            size = m["mask"]["size"]
+            entry = m["kv_rank"] + m["rot_dim"]
+            moved += batch * min(context, size) * (entry + m["kv_rank"]) * elem
+            reach = min(tokens, size)
+            pairs = reach * (reach + 1) / 2 + (tokens - reach) * reach
+            other += 2.0 * pairs * m["heads"] * (entry + m["kv_rank"])
+        else:
+            size = m["mask"]["size"]
+            moved += batch * (context % size + 1) * m["kv_heads"] * (2 * m["dim"] + m["vdim"]) * elem
+            whole, rest = tokens // size, tokens % size
+            pairs = whole * size * (size + 1) / 2 + rest * (rest + 1) / 2
+            other += 2.0 * pairs * m["heads"] * 2 * (m["dim"] + m["vdim"])
+    return moved, 2.0 * tokens * (weights - head) + 2.0 * head + other
+
+
 def compare_designs(args) -> int:
-    """``--design polosun``, ``--design givizen``, ``--design nokipel`` or ``--design senuvik``: see the module's text."""
+    """``--design polosun``, ``givizen``, ``nokipel``, ``senuvik`` or ``nopunex``: see the module's text."""
     import torch
 
-    from cie_amd.config import GivizenConfig, NokipelConfig, PolosunConfig, Qwen2Config, SenuvikConfig
+    from cie_amd.config import GivizenConfig, NokipelConfig, NopunexConfig, PolosunConfig, Qwen2Config, SenuvikConfig
     from cie_amd.workloads import SHAPES
 
     elem = 2 if args.dtype == "bf16" else 4
@@ -536,6 +605,9 @@ def compare_designs(args) -> int:
         elif args.design == "senuvik":
             designs = {"senuvik": SenuvikConfig.from_hf_config(senuvik_raw(shape, layers)),
                        "nokipel": NokipelConfig.from_hf_config(nokipel_raw(shape, layers))}
+        elif args.design == "nopunex":
+            designs = {"nopunex": NopunexConfig.from_hf_config(nopunex_raw(shape, layers)),
+                       "polosun": PolosunConfig.from_hf_config(polosun_raw(shape, layers))}
         else:
             designs = {
                 args.design: (PolosunConfig.from_hf_config(polosun_raw(shape, layers)) if args.design == "polosun"
@@ -553,6 +625,8 @@ def compare_designs(args) -> int:
                     return nokipel_costs(config, batch, context, args.prefill_tokens, elem)
                 if design == "senuvik":
                     return senuvik_costs(config, batch, context, args.prefill_tokens, elem)
+                if design == "nopunex":
+                    return nopunex_costs(config, batch, context, args.prefill_tokens, elem)
                 return (decode_bytes(config, layers, batch, context, elem), prefill_flops(config, layers, args.prefill_tokens))
 
             record = {}
@@ -585,8 +659,12 @@ def compare_designs(args) -> int:
     senuvik_layers = (f"window attention ({SENUVIK_WINDOW} tokens beside {SENUVIK_KEPT} kept first ones) + dense, state space + "
                       f"experts, causal attention beside time mixing + experts, window attention on the first layer's keys "
                       f"+ experts in turn; {GIVIZEN_EXPERTS} experts, {GIVIZEN_TOP} per token, and a gated shared expert")
+    nopunex_layers = (f"gated delta rule, latent attention (window {NOPUNEX_REACH}), differential attention (chunks of "
+                      f"{NOPUNEX_REACH}) in turn, each with a dense feed-forward, in one pass behind a joining product; beside "
+                      f"it Polosun: retention, latent_attention, rglru in turn, each with a dense feed-forward")
     beside = ("the Givizen model of equal width, head and expert sizes" if args.design == "nokipel"
               else "the Nokipel model of equal width, head and expert sizes" if args.design == "senuvik"
+              else "the Polosun model of equal width, memory and latent sizes, feed-forward" if args.design == "nopunex"
               else "the Qwen2.5 decoder of equal width, feed-forward")
     print(json.dumps({
         "metric": f"{args.design.capitalize()} beside {beside}, vocabulary and {layers} layers",
@@ -595,6 +673,7 @@ def compare_designs(args) -> int:
         "config": {"layers": layers, "context": args.context, "prefill_tokens": args.prefill_tokens, "page_size": PAGE,
                    "design_layers": ("retention, latent_attention, rglru in turn, each with a dense feed-forward"
                                      if args.design == "polosun" else givizen_layers if args.design == "givizen" else
+                                     nopunex_layers if args.design == "nopunex" else
                                      senuvik_layers + "; beside it Nokipel: " + nokipel_layers if args.design == "senuvik" else
                                      nokipel_layers + "; beside it Givizen: " + givizen_layers)},
         "shapes": out,
@@ -623,9 +702,9 @@ def main(argv=None) -> int:
                              "(default 16,64,248; '' for none, as with --no-points)")
     parser.add_argument("--other-shapes", default="7b,14b",
                         help="further shapes whose decode at the main batch and context and whose prefill go into the points ('' for none)")
-    parser.add_argument("--design", default=None, choices=["polosun", "givizen", "nokipel", "senuvik"],
+    parser.add_argument("--design", default=None, choices=["polosun", "givizen", "nokipel", "senuvik", "nopunex"],
                         help="instead of the default record: this design beside the Qwen2.5 decoder of equal size "
-                             "(nokipel: beside the Givizen model of equal size; senuvik: beside the Nokipel model)")
+                             "(nokipel: beside the Givizen model of equal size; senuvik: beside the Nokipel model; nopunex: beside the Polosun model)")
     parser.add_argument("--design-shapes", default="3b,7b", help="the Qwen2.5 shapes whose sizes the comparison takes")
     parser.add_argument("--design-layers", type=int, default=12, help="layers of both models in the comparison")
     args = parser.parse_args(argv)

@@ -943,6 +943,5 @@ CIE_API int cie_scored_attention_mfma(void* stream, const void* q, const void* k
     if (D == 192 && DV == 160) return launch_scored<192, 160, 1, 2>(s, a, row_tiles);
     if (D == 256 && DV == 192) return launch_scored<256, 192, 1, 2>(s, a, row_tiles);
     if (D == 320 && DV == 256) return launch_scored<320, 256, 1, 2>(s, a, row_tiles);
-    if (D == 576 && DV == 512) return launch_scored<576, 512, 1, 1>(s, a, row_tiles);
     return CIE_BAD_ARGUMENT;
 }

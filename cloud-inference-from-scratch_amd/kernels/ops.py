@@ -1761,7 +1761,7 @@ SCORED_MFMA_DIMS = ((64, 64), (128, 128), (64, 128), (128, 64))  # (key, value) 
 DIFFERENTIAL_MFMA_DIMS = {(32, 64): 4, (32, 128): 4, (64, 64): 4, (64, 128): 4, (64, 256): 2, (128, 128): 2, (128, 256): 2}
 # ... and those of cache entries whose value is a part of the key: (entry, value) -> the most tiles of 16 rows
 LATENT_MFMA_DIMS = {(64, 64): 4, (96, 64): 4, (128, 96): 4, (128, 128): 4, (160, 128): 2, (192, 160): 2, (256, 192): 2,
-                    (320, 256): 2, (576, 512): 1}
+                    (320, 256): 2}
 
 
 def _check_kv_pools(k_pool: torch.Tensor, v_pool: torch.Tensor, dtype: torch.dtype, kv_heads: int, dim: int,
