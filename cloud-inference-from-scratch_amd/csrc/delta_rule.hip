@@ -320,9 +320,11 @@ __global__ void __launch_bounds__(256) delta_keep_kernel(DeltaArgs<T> a) {
 //     S' = exp(L_31) S + sum_j exp(L_31 - L_j) k_j u_j^T
 // (every exponent is at most zero; tokens past a block's end have beta = 0 and so u = 0, and repeat the last L).
 // `delta_prepare_kernel`: every token at once makes its q, k (rows padded with zeros to `padded` numbers), v, beta, log g.
-// `delta_block_kernel`: every block at once makes T diag(beta) V, -T diag(beta exp(L)) K and the 32 x 32 weights of the
-// read-out's second term.  `delta_scan_kernel`: a workgroup per (sequence, head, 16 columns) goes over the blocks in
-// order with its 16 columns of S in registers.  Block b of sequence s has place first_token(s) / 32 + s + b.
+// `delta_block_kernel`: every block at once makes T diag(beta) V, -T diag(beta exp(L)) K, the 32 x 32 weights of the
+// read-out's second term and the powers of the decays.  `delta_scan_kernel`: a workgroup per (sequence, head, 16 columns)
+// goes over the blocks in order with its 16 columns of S in registers; it is a chain of steps, so what it reads lies as
+// its lanes take it (a float4 a lane, 64 lanes in a row: an "operand tile").
+// Block b of sequence s has place first_token(s) / 32 + s + b.
 // Operand layout of the product: lane (l16 = lane % 16, g = lane / 16) gives A[l16][g] and B[g][l16] and gets rows
 // 4 g .. 4 g + 3 of column l16; which four numbers of a sum one product takes does not matter as long as both operands
 // agree, so four products take the numbers 4 g .. 4 g + 3 of a run of 16: a result tile is then an operand as it is.
@@ -335,59 +337,123 @@ struct BlockArgs {
     float* values;  // [tokens, heads * vdim]
     float* beta;    // [tokens, heads]
     float* logs;    // [tokens, heads]
-    float* w;       // [places, heads, 32, padded]: -T diag(beta exp(L)) K
-    float* u;       // [places, heads, 32, cols16]: T diag(beta) V
-    float* p;       // [places, heads, 32, 32]
-    float* fade;    // [places, heads, 32]: L
+    // operand tiles, of 16 tokens (half of a block) and 16 channels or columns each; lane (l16, g) has of
+    float4* w;      // [places, heads, tiles, 2, 64]: -T diag(beta exp(L)) K: token l16, channels 4 g ..
+    float4* q;      // [places, kv_heads, tiles, 2, 64]: token l16, channels 4 g ..
+    float4* k;      // [places, kv_heads, tiles, 2, 64]: tokens 4 g .., channel l16
+    float4* u;      // [places, heads, cols16 / 16, 2, 64]: T diag(beta) V: tokens 4 g .., column l16
+    float4* p;      // [places, heads, 2, 2, 64]: the read-out's weights: row l16 of the first half index, 4 g .. of the second
+    float* fade;    // [places, heads, 2, 32]: exp(L_i), exp(L_31 - L_i)
     float* state;   // [slots, heads, vdim, dim]
     const int* seq_slot;
     const int* q_start_loc;
     float* y;       // [tokens, heads * vdim]
     int heads, kv_heads, dim, vdim, padded, cols16;
+    int tiles;      // of 16 channels: a multiple of 4, the ones past `padded` hold zeros
 };
 
-// One wave per (token, query, key or value head).
-template <typename T>
+// One wave per (run of kRun neighbouring tokens, query or key head or piece of a value head): a lane has NC channels, 64
+// apart, with their taps and last inputs in registers, so that a token's input is read once and not once a tap.  With more
+// than kWindow taps every tap reads its input.
+constexpr int kRun = 16;
+constexpr int kWindow = 4;
+
+template <typename T, int NC>
 __global__ void __launch_bounds__(256)
-delta_prepare_kernel(DeltaArgs<T> a, BlockArgs b, const int* __restrict__ seq_of_token, int tokens) {
+delta_prepare_kernel(DeltaArgs<T> a, BlockArgs b, const int* __restrict__ seq_of_token, int tokens, int pieces) {
     const int lane = threadIdx.x % kWave;
-    const int slots = 2 * a.kv_heads + a.heads;
+    const int slots = 2 * a.kv_heads + a.heads * pieces;
     const long unit = static_cast<long>(blockIdx.x) * (blockDim.x / kWave) + threadIdx.x / kWave;
-    if (unit >= static_cast<long>(tokens) * slots) return;
-    const int token = static_cast<int>(unit / slots);
-    const int what = static_cast<int>(unit - static_cast<long>(token) * slots);
-    const int seq = seq_of_token[token];
-    const int first = a.q_start_loc[seq];
+    const int run = static_cast<int>(unit / slots);
+    if (run * kRun >= tokens) return;
+    const int what = static_cast<int>(unit - static_cast<long>(run) * slots);
     const int per = a.heads / a.kv_heads;
-    const int head = what < 2 * a.kv_heads ? (what % a.kv_heads) * per : what - 2 * a.kv_heads;
-    const float* past = a.past + (static_cast<size_t>(a.seq_slot[seq]) * a.heads + head) * max(a.taps - 1, 1) * (2 * a.dim + a.vdim);
-    if (what >= 2 * a.kv_heads) {
-        for (int c = lane; c < a.vdim; c += kWave)
-            b.values[static_cast<size_t>(token) * a.heads * a.vdim + static_cast<size_t>(head) * a.vdim + c] =
-                convolved(a, head, 2 * a.dim + c, first, token - first, past);
-        if (lane == 0) {
-            float beta, log_decay;
-            steps_of(a, head, token, beta, log_decay);
-            b.beta[static_cast<size_t>(token) * a.heads + head] = beta;
-            b.logs[static_cast<size_t>(token) * a.heads + head] = log_decay;
-        }
-        return;
-    }
+    const bool is_value = what >= 2 * a.kv_heads;
     const bool is_q = what < a.kv_heads;
-    float x[8];  // dim <= 512
-    float sum = 0.f;
+    const int piece = is_value ? (what - 2 * a.kv_heads) % pieces : 0;
+    const int head = is_value ? (what - 2 * a.kv_heads) / pieces : (what % a.kv_heads) * per;
+    const int size = is_value ? a.vdim : a.dim;
+    const int from_channel = is_value ? 2 * a.dim : is_q ? 0 : a.dim;
+    const int width = 2 * a.dim + a.vdim;
+    const bool windowed = a.taps <= kWindow;
+    int col[NC], at[NC];         // the lane's columns of the projection, and their numbers in the head
+    bool real[NC];
+    float tap[NC][kWindow], window[NC][kWindow - 1];
 #pragma unroll
-    for (int i = 0; i < 8; ++i) {
-        const int n = lane + i * kWave;
-        x[i] = n < a.dim ? convolved(a, head, (is_q ? 0 : a.dim) + n, first, token - first, past) : 0.f;
-        sum += x[i] * x[i];
+    for (int i = 0; i < NC; ++i) {
+        at[i] = piece * NC * kWave + lane + i * kWave;
+        real[i] = at[i] < size;
+        int channel;
+        head_channel(a, head, from_channel + (real[i] ? at[i] : 0), col[i], channel);
+        const T* w = a.taps_w + static_cast<size_t>(channel) * a.taps;
+#pragma unroll
+        for (int j = 0; j < kWindow; ++j) {  // (fewer taps than the window: leading zeros)
+            const int from = j - (kWindow - a.taps);
+            tap[i][j] = windowed && from >= 0 ? to_float(w[from]) : 0.f;
+        }
     }
-    const float by = (is_q ? a.q_scale : 1.0f) / sqrtf(wave_sum(sum) + 1e-6f);
-    float* dst = b.rows + (static_cast<size_t>(token) * 2 * a.kv_heads + what) * b.padded;
+    int seq = -1, first = 0;
+    const float* past = nullptr;
+    const int end = min(tokens, (run + 1) * kRun);
+    for (int token = run * kRun; token < end; ++token) {
+        const int now = seq_of_token[token];
+        if (now != seq) {  // (uniform in the wave)
+            seq = now;
+            first = a.q_start_loc[seq];
+            past = a.past + (static_cast<size_t>(a.seq_slot[seq]) * a.heads + head) * max(a.taps - 1, 1) * width + from_channel;
+            if (windowed) {
 #pragma unroll
-    for (int i = 0; i < 8; ++i) {
-        const int n = lane + i * kWave;
-        if (n < b.padded) dst[n] = x[i] * by;
+                for (int i = 0; i < NC; ++i)
+#pragma unroll
+                    for (int j = 0; j < kWindow - 1; ++j) {
+                        const int src = token - first - (kWindow - 1) + j;
+                        const int kept = a.taps - 1 + src;  // its row of the state, if it lies in front of the step
+                        window[i][j] = !real[i] ? 0.f
+                                       : src >= 0 ? to_float(a.proj[static_cast<size_t>(first + src) * a.ldp + col[i]])
+                                       : kept >= 0 ? past[static_cast<size_t>(kept) * width + at[i]] : 0.f;
+                    }
+            }
+        }
+        float x[NC];
+        float sum = 0.f;
+#pragma unroll
+        for (int i = 0; i < NC; ++i) {
+            float acc = 0.f;
+            if (windowed) {
+                const float in = real[i] ? to_float(a.proj[static_cast<size_t>(token) * a.ldp + col[i]]) : 0.f;
+#pragma unroll
+                for (int j = 0; j < kWindow - 1; ++j) acc = fmaf(tap[i][j], window[i][j], acc);
+                acc = fmaf(tap[i][kWindow - 1], in, acc);
+#pragma unroll
+                for (int j = 0; j + 1 < kWindow - 1; ++j) window[i][j] = window[i][j + 1];
+                window[i][kWindow - 2] = in;
+                x[i] = silu_f(acc);
+            } else {
+                x[i] = real[i] ? convolved(a, head, from_channel + at[i], first, token - first, past - from_channel) : 0.f;
+            }
+            sum += x[i] * x[i];
+        }
+        if (is_value) {
+            float* dst = b.values + static_cast<size_t>(token) * a.heads * a.vdim + static_cast<size_t>(head) * a.vdim;
+#pragma unroll
+            for (int i = 0; i < NC; ++i)
+                if (real[i]) dst[at[i]] = x[i];
+        } else {
+            const float by = (is_q ? a.q_scale : 1.0f) / sqrtf(wave_sum(sum) + 1e-6f);
+            float* dst = b.rows + (static_cast<size_t>(token) * 2 * a.kv_heads + what) * b.padded;
+#pragma unroll
+            for (int i = 0; i < NC; ++i)
+                if (at[i] < b.padded) dst[at[i]] = x[i] * by;
+        }
+    }
+    if (is_value && piece == 0 && run * kRun + lane < end) {  // step sizes and decays, a token a lane
+        const size_t token = static_cast<size_t>(run) * kRun + lane;
+        if (lane < kRun) {
+            float beta, log_decay;
+            steps_of(a, head, static_cast<int>(token), beta, log_decay);
+            b.beta[token * a.heads + head] = beta;
+            b.logs[token * a.heads + head] = log_decay;
+        }
     }
 }
 
@@ -450,35 +516,42 @@ __global__ void __launch_bounds__(256) delta_block_kernel(BlockArgs a) {
     __syncthreads();
     const int place = first / kBlock + seq + blockIdx.y;
     const size_t unit = static_cast<size_t>(place) * a.heads + head;
-    {   // this wave's tile of k k^T and of q k^T (the tile above the diagonal is zero)
+    const size_t unit_kv = static_cast<size_t>(place) * a.kv_heads + shared;
+    const bool leads = head % (a.heads / a.kv_heads) == 0;  // writes what the heads of a key head share
+    {   // this wave's tile of k k^T and of (q k^T)^T (the tile above the diagonal is zero)
         const int ti = wave >> 1, tj = wave & 1;
         acc4_t kk = {0.f, 0.f, 0.f, 0.f}, qk = {0.f, 0.f, 0.f, 0.f};
         if (tj <= ti) {
             const float* ka = k_s + (16 * ti + l16) * stride + 4 * g;
             const float* kb = k_s + (16 * tj + l16) * stride + 4 * g;
             const float* qa = q_rows + static_cast<size_t>(min(16 * ti + l16, cn - 1)) * ld + 4 * g;
-#pragma unroll 4
+            float4* q_out = leads && tj == 0 ? a.q + unit_kv * a.tiles * 2 * kWave + ti * kWave + lane : nullptr;
             for (int m = 0; m < padded / 16; ++m) {
                 const float4 x = *reinterpret_cast<const float4*>(ka + 16 * m);
                 const float4 y = *reinterpret_cast<const float4*>(kb + 16 * m);
                 const float4 z = *reinterpret_cast<const float4*>(qa + 16 * m);
+                if (q_out) q_out[m * 2 * kWave] = z;
                 kk = __builtin_amdgcn_mfma_f32_16x16x4f32(x.x, y.x, kk, 0, 0, 0);
-                qk = __builtin_amdgcn_mfma_f32_16x16x4f32(z.x, y.x, qk, 0, 0, 0);
+                qk = __builtin_amdgcn_mfma_f32_16x16x4f32(y.x, z.x, qk, 0, 0, 0);
                 kk = __builtin_amdgcn_mfma_f32_16x16x4f32(x.y, y.y, kk, 0, 0, 0);
-                qk = __builtin_amdgcn_mfma_f32_16x16x4f32(z.y, y.y, qk, 0, 0, 0);
+                qk = __builtin_amdgcn_mfma_f32_16x16x4f32(y.y, z.y, qk, 0, 0, 0);
                 kk = __builtin_amdgcn_mfma_f32_16x16x4f32(x.z, y.z, kk, 0, 0, 0);
-                qk = __builtin_amdgcn_mfma_f32_16x16x4f32(z.z, y.z, qk, 0, 0, 0);
+                qk = __builtin_amdgcn_mfma_f32_16x16x4f32(y.z, z.z, qk, 0, 0, 0);
                 kk = __builtin_amdgcn_mfma_f32_16x16x4f32(x.w, y.w, kk, 0, 0, 0);
-                qk = __builtin_amdgcn_mfma_f32_16x16x4f32(z.w, y.w, qk, 0, 0, 0);
+                qk = __builtin_amdgcn_mfma_f32_16x16x4f32(y.w, z.w, qk, 0, 0, 0);
             }
+            if (q_out)
+                for (int m = padded / 16; m < a.tiles; ++m) q_out[m * 2 * kWave] = float4{0.f, 0.f, 0.f, 0.f};
         }
+        acc4_t p;  // (queries along the lanes: as the scan takes it)
 #pragma unroll
         for (int r = 0; r < 4; ++r) {
             const int i = 16 * ti + 4 * g + r, j = 16 * tj + l16;
-            const float by = i >= j ? expf(log_s[i] - log_s[j]) : 0.f;
-            if (i > j) a_s[i * kTri + j] = beta_s[i] * by * kk[r];
-            a.p[unit * kBlock * kBlock + i * kBlock + j] = i >= j ? by * qk[r] : 0.f;
+            if (i > j) a_s[i * kTri + j] = beta_s[i] * expf(log_s[i] - log_s[j]) * kk[r];
+            const int row = 16 * ti + l16, key = 16 * tj + 4 * g + r;
+            p[r] = row >= key ? expf(log_s[row] - log_s[key]) * qk[r] : 0.f;
         }
+        a.p[((unit * 2 + ti) * 2 + tj) * kWave + lane] = __builtin_bit_cast(float4, p);
     }
     __syncthreads();
     if (wave == 0 && lane < 32) {  // the two 16 x 16 inverses on the diagonal, a column per lane
@@ -505,7 +578,8 @@ __global__ void __launch_bounds__(256) delta_block_kernel(BlockArgs a) {
         t21 = __builtin_amdgcn_mfma_f32_16x16x4f32(y.w, z[3], t21, 0, 0, 0);
 #pragma unroll
         for (int r = 0; r < 4; ++r) t_s[(16 + 4 * g + r) * kTri + l16] = -t21[r];
-        if (lane < kBlock) a.fade[unit * kBlock + lane] = log_s[lane];
+        const int i = lane % kBlock;
+        a.fade[unit * 2 * kBlock + lane] = expf(lane < kBlock ? log_s[i] : log_s[kBlock - 1] - log_s[i]);
     }
     __syncthreads();
     float4 t_a[2][2];         // T's rows as operands: [row tile][run of 16 tokens]
@@ -522,46 +596,58 @@ __global__ void __launch_bounds__(256) delta_block_kernel(BlockArgs a) {
         }
     }
     const int k_tiles = padded / 16, v_tiles = a.cols16 / 16;
-    for (int ct = wave; ct < k_tiles + v_tiles; ct += 4) {
-        const bool is_k = ct < k_tiles;
-        const int col = 16 * (is_k ? ct : ct - k_tiles) + l16;
+    for (int ct = wave; ct < a.tiles + v_tiles; ct += 4) {
+        const bool is_k = ct < a.tiles;
+        const int tile = is_k ? ct : ct - a.tiles;
+        const int col = 16 * tile + l16;
+        float4* dst = (is_k ? a.w + (unit * a.tiles + tile) * 2 * kWave : a.u + (unit * v_tiles + tile) * 2 * kWave) + lane;
         float b[2][4];
 #pragma unroll
-        for (int h = 0; h < 2; ++h)
+        for (int h = 0; h < 2; ++h) {
 #pragma unroll
             for (int e = 0; e < 4; ++e) {
                 const int j = 16 * h + 4 * g + e;
                 if (is_k)
-                    b[h][e] = k_s[j * stride + col] * k_by[h][e];
+                    b[h][e] = tile < k_tiles ? k_s[j * stride + col] : 0.f;
                 else
-                    b[h][e] = v_by[h][e] * (col < a.vdim ? a.values[(static_cast<size_t>(first + c0) + min(j, cn - 1)) * a.heads * a.vdim +
-                                                                    static_cast<size_t>(head) * a.vdim + col] : 0.f);
+                    b[h][e] = col < a.vdim ? a.values[(static_cast<size_t>(first + c0) + min(j, cn - 1)) * a.heads * a.vdim +
+                                                      static_cast<size_t>(head) * a.vdim + col] : 0.f;
             }
+            if (is_k && leads)
+                a.k[((unit_kv * a.tiles + tile) * 2 + h) * kWave + lane] = float4{b[h][0], b[h][1], b[h][2], b[h][3]};
+#pragma unroll
+            for (int e = 0; e < 4; ++e) b[h][e] *= is_k ? k_by[h][e] : v_by[h][e];
+        }
         acc4_t r0 = {0.f, 0.f, 0.f, 0.f}, r1 = {0.f, 0.f, 0.f, 0.f};
-#pragma unroll
-        for (int h = 0; h < 2; ++h) {
-            if (h == 0) {  // (the upper tile has nothing right of the diagonal)
-                r0 = __builtin_amdgcn_mfma_f32_16x16x4f32(t_a[0][h].x, b[h][0], r0, 0, 0, 0);
-                r0 = __builtin_amdgcn_mfma_f32_16x16x4f32(t_a[0][h].y, b[h][1], r0, 0, 0, 0);
-                r0 = __builtin_amdgcn_mfma_f32_16x16x4f32(t_a[0][h].z, b[h][2], r0, 0, 0, 0);
-                r0 = __builtin_amdgcn_mfma_f32_16x16x4f32(t_a[0][h].w, b[h][3], r0, 0, 0, 0);
-            }
-            r1 = __builtin_amdgcn_mfma_f32_16x16x4f32(t_a[1][h].x, b[h][0], r1, 0, 0, 0);
-            r1 = __builtin_amdgcn_mfma_f32_16x16x4f32(t_a[1][h].y, b[h][1], r1, 0, 0, 0);
-            r1 = __builtin_amdgcn_mfma_f32_16x16x4f32(t_a[1][h].z, b[h][2], r1, 0, 0, 0);
-            r1 = __builtin_amdgcn_mfma_f32_16x16x4f32(t_a[1][h].w, b[h][3], r1, 0, 0, 0);
-        }
-        const int width = is_k ? padded : a.cols16;
-        float* dst = (is_k ? a.w : a.u) + unit * kBlock * width + col;
-#pragma unroll
-        for (int r = 0; r < 4; ++r) {
-            dst[static_cast<size_t>(4 * g + r) * width] = r0[r];
-            dst[static_cast<size_t>(16 + 4 * g + r) * width] = r1[r];
-        }
+        // (the upper tile has nothing right of the diagonal; the product's sides as the scan takes the result)
+#define CIE_DELTA_TILE(r, t, h, c, e)                                                        \
+    r = is_k ? __builtin_amdgcn_mfma_f32_16x16x4f32(b[h][e], t_a[t][h].c, r, 0, 0, 0)        \
+             : __builtin_amdgcn_mfma_f32_16x16x4f32(t_a[t][h].c, b[h][e], r, 0, 0, 0)
+        CIE_DELTA_TILE(r0, 0, 0, x, 0); CIE_DELTA_TILE(r1, 1, 0, x, 0); CIE_DELTA_TILE(r0, 0, 0, y, 1); CIE_DELTA_TILE(r1, 1, 0, y, 1);
+        CIE_DELTA_TILE(r0, 0, 0, z, 2); CIE_DELTA_TILE(r1, 1, 0, z, 2); CIE_DELTA_TILE(r0, 0, 0, w, 3); CIE_DELTA_TILE(r1, 1, 0, w, 3);
+        CIE_DELTA_TILE(r1, 1, 1, x, 0); CIE_DELTA_TILE(r1, 1, 1, y, 1); CIE_DELTA_TILE(r1, 1, 1, z, 2); CIE_DELTA_TILE(r1, 1, 1, w, 3);
+#undef CIE_DELTA_TILE
+        dst[0] = __builtin_bit_cast(float4, r0);
+        dst[kWave] = __builtin_bit_cast(float4, r1);
     }
 }
 
-// MT row tiles of 16 a wave: padded <= 64 * MT; wave w has the tiles w, w + 4, ...
+// A barrier for what waves exchange through LDS alone: loads from memory that are under way (the next block's operands)
+// stay so, where __syncthreads() would wait for them.
+__device__ __forceinline__ void lds_barrier() {
+    __builtin_amdgcn_fence(__ATOMIC_RELEASE, "workgroup", "local");
+    __builtin_amdgcn_s_barrier();
+    __builtin_amdgcn_fence(__ATOMIC_ACQUIRE, "workgroup", "local");
+}
+
+// What one block brings to a wave of the scan, in registers.
+template <int MT>
+struct ScanStage {
+    float4 w[MT][2], q[MT][2], k[MT][2], p[2], u[2], grown[2], left[2];
+    float whole;
+};
+
+// MT tiles of 16 channels a wave (tiles = 4 * MT): wave w has the tiles w, w + 4, ...
 template <int MT>
 __global__ void __launch_bounds__(256) delta_scan_kernel(BlockArgs a) {
     const int seq = blockIdx.x / a.heads;
@@ -570,12 +656,10 @@ __global__ void __launch_bounds__(256) delta_scan_kernel(BlockArgs a) {
     const int count = a.q_start_loc[seq + 1] - first;
     if (count <= 0) return;
     const int lane = threadIdx.x % kWave;
-    const int wave = threadIdx.x / kWave;
+    const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x / kWave);
     const int l16 = lane % 16;
     const int g = lane / 16;
     const int col = 16 * blockIdx.y + l16;
-    const int padded = a.padded;
-    const int tiles = padded / 16;
     const int shared = head / (a.heads / a.kv_heads);
     __shared__ float4 part_s[2][4][4][kWave];  // [buffer][wave][u tile 0, 1, o tile 0, 1][lane]
     float* column = a.state + ((static_cast<size_t>(a.seq_slot[seq]) * a.heads + head) * a.vdim + min(col, a.vdim - 1)) * a.dim;
@@ -589,78 +673,52 @@ __global__ void __launch_bounds__(256) delta_scan_kernel(BlockArgs a) {
         }
     const int blocks = (count + kBlock - 1) / kBlock;
     const size_t place0 = static_cast<size_t>(first / kBlock + seq);
-    const size_t ld = static_cast<size_t>(2) * a.kv_heads * padded;
-    const float* rows = a.rows + static_cast<size_t>(first) * ld + static_cast<size_t>(shared) * padded;
-    const size_t k_off = static_cast<size_t>(a.kv_heads) * padded;
-    // what a block needs, fetched a block ahead
-    float4 w_n[2][MT], q_n[2][MT];
-    float k_n[MT][2][4];
-    float4 p_n[2], l_n[2];
-    acc4_t u_n[2];
-    float last_n;
-#define CIE_DELTA_FETCH(block)                                                                                        \
-    {                                                                                                                 \
-        const size_t unit = (place0 + (block)) * a.heads + head;                                                      \
-        const int left = count - (block) * kBlock - 1;                                                                \
-        const float* from = rows + static_cast<size_t>((block) * kBlock) * ld;                                        \
-        const float* w_rows = a.w + unit * kBlock * padded;                                                           \
-        _Pragma("unroll") for (int m = 0; m < MT; ++m) {                                                              \
-            const int at = 16 * min(wave + 4 * m, tiles - 1);                                                         \
-            _Pragma("unroll") for (int t = 0; t < 2; ++t) {                                                           \
-                w_n[t][m] = *reinterpret_cast<const float4*>(w_rows + (16 * t + l16) * padded + at + 4 * g);          \
-                q_n[t][m] = *reinterpret_cast<const float4*>(from + static_cast<size_t>(min(16 * t + l16, left)) * ld + at + 4 * g); \
-                _Pragma("unroll") for (int e = 0; e < 4; ++e)                                                         \
-                    k_n[m][t][e] = from[static_cast<size_t>(min(16 * t + 4 * g + e, left)) * ld + k_off + at + l16];  \
-            }                                                                                                         \
-        }                                                                                                             \
-        _Pragma("unroll") for (int t = 0; t < 2; ++t) {                                                               \
-            l_n[t] = *reinterpret_cast<const float4*>(a.fade + unit * kBlock + 16 * t + 4 * g);                       \
-            p_n[t] = *reinterpret_cast<const float4*>(a.p + unit * kBlock * kBlock + (16 * (wave & 1) + l16) * kBlock + 16 * t + 4 * g); \
-            _Pragma("unroll") for (int e = 0; e < 4; ++e)                                                             \
-                u_n[t][e] = a.u[(unit * kBlock + 16 * t + 4 * g + e) * a.cols16 + col];                               \
-        }                                                                                                             \
-        last_n = a.fade[unit * kBlock + kBlock - 1];                                                                  \
-    }
-    CIE_DELTA_FETCH(0)
-    for (int b = 0; b < blocks; ++b) {
-        float4 w[2][MT], q[2][MT], p[2], l[2];
-        float k[MT][2][4];
-        acc4_t u0[2];
-        const float last = last_n;
+    const size_t ldy = static_cast<size_t>(a.heads) * a.vdim;
+    float* y = a.y + static_cast<size_t>(first + 16 * (wave & 1) + 4 * g) * ldy + static_cast<size_t>(head) * a.vdim + col;
+    auto fetch = [&](ScanStage<MT>& to, int block) {
+        const size_t place = place0 + min(block, blocks - 1);  // (past the end: the last one again, and nobody looks at it)
+        const size_t unit = place * a.heads + head;
+        const float4* w = a.w + (unit * (4 * MT) + wave) * 2 * kWave + lane;
+        const size_t kv = ((place * a.kv_heads + shared) * (4 * MT) + wave) * 2 * kWave;
+        const float4* q = a.q + kv + lane;
+        const float4* k = a.k + kv + lane;
+        const float4* u = a.u + (unit * (a.cols16 / 16) + blockIdx.y) * 2 * kWave + lane;
+        const float4* p = a.p + (unit * 2 + (wave & 1)) * 2 * kWave + lane;
+        const float* fade = a.fade + unit * 2 * kBlock;
+#pragma unroll
+        for (int m = 0; m < MT; ++m)
+#pragma unroll
+            for (int t = 0; t < 2; ++t) {
+                to.w[m][t] = w[(8 * m + t) * kWave];
+                to.q[m][t] = q[(8 * m + t) * kWave];
+            }
 #pragma unroll
         for (int t = 0; t < 2; ++t) {
-            p[t] = p_n[t];
-            l[t] = l_n[t];
-            u0[t] = u_n[t];
-#pragma unroll
-            for (int m = 0; m < MT; ++m) {
-                w[t][m] = w_n[t][m];
-                q[t][m] = q_n[t][m];
-#pragma unroll
-                for (int e = 0; e < 4; ++e) k[m][t][e] = k_n[m][t][e];
-            }
+            to.u[t] = u[t * kWave];
+            to.p[t] = p[t * kWave];
+            to.grown[t] = *reinterpret_cast<const float4*>(fade + 16 * t + 4 * g);
+            to.left[t] = *reinterpret_cast<const float4*>(fade + kBlock + 16 * t + 4 * g);
         }
-        const int ahead = min(b + 1, blocks - 1);  // (the last block is fetched twice: no condition around the loads)
-        CIE_DELTA_FETCH(ahead)
+        to.whole = fade[kBlock - 1];
+#pragma unroll
+        for (int m = 0; m < MT; ++m)
+#pragma unroll
+            for (int t = 0; t < 2; ++t) to.k[m][t] = k[(8 * m + t) * kWave];
+    };
+    auto step = [&](const ScanStage<MT>& in, int b) {
         // this wave's rows' share of -W S and of S^T q, for both tiles of tokens
         acc4_t us[2], os[2];
 #pragma unroll
         for (int t = 0; t < 2; ++t) us[t] = os[t] = acc4_t{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
         for (int m = 0; m < MT; ++m) {
-            if (wave + 4 * m < tiles) {
-#pragma unroll
-                for (int t = 0; t < 2; ++t) {
-                    us[t] = __builtin_amdgcn_mfma_f32_16x16x4f32(w[t][m].x, S[m][0], us[t], 0, 0, 0);
-                    os[t] = __builtin_amdgcn_mfma_f32_16x16x4f32(q[t][m].x, S[m][0], os[t], 0, 0, 0);
-                    us[t] = __builtin_amdgcn_mfma_f32_16x16x4f32(w[t][m].y, S[m][1], us[t], 0, 0, 0);
-                    os[t] = __builtin_amdgcn_mfma_f32_16x16x4f32(q[t][m].y, S[m][1], os[t], 0, 0, 0);
-                    us[t] = __builtin_amdgcn_mfma_f32_16x16x4f32(w[t][m].z, S[m][2], us[t], 0, 0, 0);
-                    os[t] = __builtin_amdgcn_mfma_f32_16x16x4f32(q[t][m].z, S[m][2], os[t], 0, 0, 0);
-                    us[t] = __builtin_amdgcn_mfma_f32_16x16x4f32(w[t][m].w, S[m][3], us[t], 0, 0, 0);
-                    os[t] = __builtin_amdgcn_mfma_f32_16x16x4f32(q[t][m].w, S[m][3], os[t], 0, 0, 0);
-                }
-            }
+#define CIE_DELTA_SHARE(c, e)                                                                          \
+    us[0] = __builtin_amdgcn_mfma_f32_16x16x4f32(in.w[m][0].c, S[m][e], us[0], 0, 0, 0);               \
+    us[1] = __builtin_amdgcn_mfma_f32_16x16x4f32(in.w[m][1].c, S[m][e], us[1], 0, 0, 0);               \
+    os[0] = __builtin_amdgcn_mfma_f32_16x16x4f32(in.q[m][0].c, S[m][e], os[0], 0, 0, 0);               \
+    os[1] = __builtin_amdgcn_mfma_f32_16x16x4f32(in.q[m][1].c, S[m][e], os[1], 0, 0, 0)
+            CIE_DELTA_SHARE(x, 0); CIE_DELTA_SHARE(y, 1); CIE_DELTA_SHARE(z, 2); CIE_DELTA_SHARE(w, 3);
+#undef CIE_DELTA_SHARE
         }
         auto& part = part_s[b & 1];
 #pragma unroll
@@ -668,55 +726,65 @@ __global__ void __launch_bounds__(256) delta_scan_kernel(BlockArgs a) {
             part[wave][t][lane] = __builtin_bit_cast(float4, us[t]);
             part[wave][2 + t][lane] = __builtin_bit_cast(float4, os[t]);
         }
-        __syncthreads();
+        lds_barrier();
         acc4_t u[2], faded[2];
 #pragma unroll
         for (int t = 0; t < 2; ++t) {
-            u[t] = u0[t];
+            u[t] = __builtin_bit_cast(acc4_t, in.u[t]);
 #pragma unroll
             for (int s = 0; s < 4; ++s) u[t] += __builtin_bit_cast(acc4_t, part[s][t][lane]);
-            faded[t] = acc4_t{u[t][0] * expf(last - l[t].x), u[t][1] * expf(last - l[t].y), u[t][2] * expf(last - l[t].z),
-                              u[t][3] * expf(last - l[t].w)};
+            faded[t] = u[t] * __builtin_bit_cast(acc4_t, in.left[t]);
         }
-        if (wave < 2) {  // (uniform in a wave) the read-out of tile `wave`
+#pragma unroll
+        for (int m = 0; m < MT; ++m) S[m] *= in.whole;
+#pragma unroll
+        for (int t = 0; t < 2; ++t) {
+#define CIE_DELTA_KEEP(c, e)                                                                           \
+    _Pragma("unroll") for (int m = 0; m < MT; ++m)                                                     \
+        S[m] = __builtin_amdgcn_mfma_f32_16x16x4f32(in.k[m][t].c, faded[t][e], S[m], 0, 0, 0)
+            CIE_DELTA_KEEP(x, 0); CIE_DELTA_KEEP(y, 1); CIE_DELTA_KEEP(z, 2); CIE_DELTA_KEEP(w, 3);
+#undef CIE_DELTA_KEEP
+        }
+        if (wave < 2) {  // the read-out of tile `wave`
             acc4_t o = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
             for (int s = 0; s < 4; ++s) o += __builtin_bit_cast(acc4_t, part[s][2 + wave][lane]);
-            const float4 lo = wave == 0 ? l[0] : l[1];
-            o[0] *= expf(lo.x);
-            o[1] *= expf(lo.y);
-            o[2] *= expf(lo.z);
-            o[3] *= expf(lo.w);
+            o *= __builtin_bit_cast(acc4_t, wave == 0 ? in.grown[0] : in.grown[1]);
 #pragma unroll
             for (int t = 0; t < 2; ++t) {
-                o = __builtin_amdgcn_mfma_f32_16x16x4f32(p[t].x, u[t][0], o, 0, 0, 0);
-                o = __builtin_amdgcn_mfma_f32_16x16x4f32(p[t].y, u[t][1], o, 0, 0, 0);
-                o = __builtin_amdgcn_mfma_f32_16x16x4f32(p[t].z, u[t][2], o, 0, 0, 0);
-                o = __builtin_amdgcn_mfma_f32_16x16x4f32(p[t].w, u[t][3], o, 0, 0, 0);
+                o = __builtin_amdgcn_mfma_f32_16x16x4f32(in.p[t].x, u[t][0], o, 0, 0, 0);
+                o = __builtin_amdgcn_mfma_f32_16x16x4f32(in.p[t].y, u[t][1], o, 0, 0, 0);
+                o = __builtin_amdgcn_mfma_f32_16x16x4f32(in.p[t].z, u[t][2], o, 0, 0, 0);
+                o = __builtin_amdgcn_mfma_f32_16x16x4f32(in.p[t].w, u[t][3], o, 0, 0, 0);
             }
-            if (col < a.vdim) {
+            float* row = y + static_cast<size_t>(b * kBlock) * ldy;
+            if ((b + 1) * kBlock <= count) {
+                if (col < a.vdim) {
 #pragma unroll
-                for (int r = 0; r < 4; ++r) {
-                    const int i = b * kBlock + 16 * wave + 4 * g + r;
-                    if (i < count)
-                        a.y[static_cast<size_t>(first + i) * a.heads * a.vdim + static_cast<size_t>(head) * a.vdim + col] = o[r];
+                    for (int r = 0; r < 4; ++r) row[r * ldy] = o[r];
                 }
+            } else {
+#pragma unroll
+                for (int r = 0; r < 4; ++r)
+                    if (col < a.vdim && b * kBlock + 16 * wave + 4 * g + r < count) row[r * ldy] = o[r];
             }
         }
-        const float whole = expf(last);
-#pragma unroll
-        for (int m = 0; m < MT; ++m) {
-            if (wave + 4 * m < tiles) {
-                acc4_t s = {S[m][0] * whole, S[m][1] * whole, S[m][2] * whole, S[m][3] * whole};
-#pragma unroll
-                for (int t = 0; t < 2; ++t)
-#pragma unroll
-                    for (int e = 0; e < 4; ++e) s = __builtin_amdgcn_mfma_f32_16x16x4f32(k[m][t][e], faded[t][e], s, 0, 0, 0);
-                S[m] = s;
-            }
-        }
+    };
+    // two blocks are under way while one is worked on
+    ScanStage<MT> s0, s1, s2;
+    fetch(s0, 0);
+    fetch(s1, 1);
+    for (int b = 0;; b += 3) {
+        fetch(s2, b + 2);
+        step(s0, b);
+        if (b + 1 >= blocks) break;
+        fetch(s0, b + 3);
+        step(s1, b + 1);
+        if (b + 2 >= blocks) break;
+        fetch(s1, b + 4);
+        step(s2, b + 2);
+        if (b + 3 >= blocks) break;
     }
-#undef CIE_DELTA_FETCH
     if (col >= a.vdim) return;
 #pragma unroll
     for (int m = 0; m < MT; ++m)
@@ -805,8 +873,8 @@ CIE_API int cie_delta_walk(void* stream, int dtype, const void* proj, long ldp, 
 
 // The same in blocks of 32 tokens on the matrix cores; `y` gets the raw read-out.  Scratch, float32: `rows`
 // [tokens, 2 kv_heads padded], `values` [tokens, heads vdim], `steps` [2, tokens, heads], and for
-// (tokens / 32 + sequences + 1) * heads blocks `blocks` with 32 * padded + 32 * cols16 + 32 * 32 + 32 numbers each;
-// padded and cols16 are dim and vdim rounded up to multiples of 16.
+// tokens / 32 + sequences + 1 blocks `blocks` with heads * (32 * wide + 32 * cols16 + 32 * 32 + 64) + kv_heads * 64 * wide
+// numbers each; padded and cols16 are dim and vdim rounded up to multiples of 16, wide is dim rounded up to one of 64.
 CIE_API int cie_delta_blocks(void* stream, int dtype, const void* proj, long ldp, int q_off, int k_off, int v_off, int g_off,
                              int b_off, int a_off, const void* taps_w, int taps, const float* a_log, const float* dt_bias,
                              float q_scale, float* state, float* past, const int* seq_of_token, const int* seq_slot,
@@ -819,21 +887,28 @@ CIE_API int cie_delta_blocks(void* stream, int dtype, const void* proj, long ldp
     const int cols16 = (vdim + 15) / 16 * 16;
     const int most_blocks = (tokens + kBlock - 1) / kBlock;  // (of one sequence)
     const size_t lds = sizeof(float) * (static_cast<size_t>(kBlock) * (padded + 4) + 2 * kBlock * kTri + 16 * 20 + 2 * kBlock);
-    const long prepare = (static_cast<long>(tokens) * (2 * kv_heads + heads) + 3) / 4;
+    const int channels = dim <= kWave ? 1 : dim <= 2 * kWave ? 2 : 4;  // of a head that a lane takes
+    const int pieces = (vdim + channels * kWave - 1) / (channels * kWave);
+    const long prepare = (static_cast<long>((tokens + kRun - 1) / kRun) * (2 * kv_heads + static_cast<long>(heads) * pieces) + 3) / 4;
     if (lds > 64 * 1024 || most_blocks > 65535 || cols16 / 16 > 65535 || static_cast<long>(sequences) * heads > 0x7fffffffL ||
         prepare > 0x7fffffffL)
         return CIE_BAD_ARGUMENT;
     if (sequences == 0 || tokens == 0) return CIE_OK;
-    const size_t units = (static_cast<size_t>(tokens) / kBlock + sequences + 1) * heads;
+    const size_t places = static_cast<size_t>(tokens) / kBlock + sequences + 1;
+    const size_t units = places * heads;
+    const size_t pair = 2 * kWave;  // the two operand tiles of a block
     BlockArgs b;
     b.rows = rows;
     b.values = values;
     b.beta = steps;
     b.logs = steps + static_cast<size_t>(tokens) * heads;
-    b.w = blocks;
-    b.u = b.w + units * kBlock * padded;
-    b.p = b.u + units * kBlock * cols16;
-    b.fade = b.p + units * kBlock * kBlock;
+    b.tiles = (dim + 63) / 64 * 4;
+    b.w = reinterpret_cast<float4*>(blocks);
+    b.q = b.w + units * b.tiles * pair;
+    b.k = b.q + places * kv_heads * b.tiles * pair;
+    b.u = b.k + places * kv_heads * b.tiles * pair;
+    b.p = b.u + units * (cols16 / 16) * pair;
+    b.fade = reinterpret_cast<float*>(b.p + units * 2 * pair);
     b.state = state;
     b.seq_slot = seq_slot;
     b.q_start_loc = q_start_loc;
@@ -848,20 +923,26 @@ CIE_API int cie_delta_blocks(void* stream, int dtype, const void* proj, long ldp
 #define CIE_DELTA_ARGS(T)                                                                                              \
     delta_args<T>(proj, ldp, q_off, k_off, v_off, g_off, b_off, a_off, taps_w, taps, a_log, dt_bias, q_scale, state, past, \
                   seq_slot, q_start_loc, heads, kv_heads, dim, vdim)
-    if (dtype == CIE_F32)
-        delta_prepare_kernel<float><<<static_cast<unsigned>(prepare), 256, 0, s>>>(CIE_DELTA_ARGS(float), b, seq_of_token, tokens);
-    else if (dtype == CIE_BF16)
-        delta_prepare_kernel<bf16_t><<<static_cast<unsigned>(prepare), 256, 0, s>>>(CIE_DELTA_ARGS(bf16_t), b, seq_of_token, tokens);
-    else
-        return CIE_BAD_ARGUMENT;
+#define CIE_DELTA_PREPARE(T, NC) \
+    delta_prepare_kernel<T, NC><<<static_cast<unsigned>(prepare), 256, 0, s>>>(CIE_DELTA_ARGS(T), b, seq_of_token, tokens, pieces)
+    if (dtype == CIE_F32 && channels == 1) CIE_DELTA_PREPARE(float, 1);
+    else if (dtype == CIE_F32 && channels == 2) CIE_DELTA_PREPARE(float, 2);
+    else if (dtype == CIE_F32) CIE_DELTA_PREPARE(float, 4);
+    else if (dtype == CIE_BF16 && channels == 1) CIE_DELTA_PREPARE(bf16_t, 1);
+    else if (dtype == CIE_BF16 && channels == 2) CIE_DELTA_PREPARE(bf16_t, 2);
+    else if (dtype == CIE_BF16) CIE_DELTA_PREPARE(bf16_t, 4);
+    else return CIE_BAD_ARGUMENT;
+#undef CIE_DELTA_PREPARE
     if (hipGetLastError() != hipSuccess) return CIE_LAUNCH_FAILED;
     delta_block_kernel<<<dim3(sequences * heads, most_blocks), 256, lds, s>>>(b);
     if (hipGetLastError() != hipSuccess) return CIE_LAUNCH_FAILED;
     const dim3 scan_grid(sequences * heads, cols16 / 16);
-    if (padded <= 64)
+    if (b.tiles == 4)
         delta_scan_kernel<1><<<scan_grid, 256, 0, s>>>(b);
-    else if (padded <= 128)
+    else if (b.tiles == 8)
         delta_scan_kernel<2><<<scan_grid, 256, 0, s>>>(b);
+    else if (b.tiles == 12)
+        delta_scan_kernel<3><<<scan_grid, 256, 0, s>>>(b);
     else
         delta_scan_kernel<4><<<scan_grid, 256, 0, s>>>(b);
     if (hipGetLastError() != hipSuccess) return CIE_LAUNCH_FAILED;

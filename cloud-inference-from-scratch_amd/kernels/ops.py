@@ -1605,8 +1605,9 @@ def delta_rule(proj: torch.Tensor, offsets: tuple[int, int, int, int, int, int],
               _ptr(a_log), _ptr(dt_bias), _f(q_scale))
     lib = load_library()
     padded, cols16 = -(-dim // 16) * 16, -(-vdim // 16) * 16
-    places = (tokens // 32 + sequences + 1) * heads
-    per_block = 32 * (padded + cols16 + 33)
+    wide = -(-dim // 64) * 64
+    places = tokens // 32 + sequences + 1
+    per_block = heads * 32 * (wide + cols16 + 34) + kv_heads * 64 * wide
     if blocks is None:
         blocks = tokens >= DELTA_BLOCKS_FROM * max(sequences, 1)
     if blocks and dim <= DELTA_BLOCKS_MAX_DIM and 4 * places * per_block <= DELTA_BLOCKS_MAX_BYTES:

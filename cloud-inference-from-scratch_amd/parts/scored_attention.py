@@ -269,8 +269,7 @@ def scored_attend(q: torch.Tensor, batch, view, h: int, g: int, dim: int, vdim: 
                                              batch.sequences, batch.seq_slot, batch.seq_start, batch.seq_q_len,
                                              batch.q_start_loc, batch.tokens, h, g, dim, vdim, 1, least, **shape,
                                              **shares(batch.sequences, 1))
-        wanted = PROMPT_ROW_TILES * maps
-        row_tiles = min(most_row_tiles, max(least, wanted if batch.max_q_len * group > 16 else maps))
+        row_tiles = min(most_row_tiles, max(least, PROMPT_ROW_TILES if batch.max_q_len * group > 16 else maps))
         while row_tiles > least and -(-batch.tokens * group * maps // (16 * row_tiles)) * g < ops.compute_units():
             row_tiles //= 2  # (fewer rows a tile where the tiles would not fill the compute units)
         per_tile = (16 * row_tiles) // (group * maps)
