@@ -93,7 +93,7 @@ class NopunexConfig:
         return float(self.raw["norm"]["eps"])
 
     def loop(self) -> tuple[int, int, int]:
-        """(start, stop, times): layers start .. stop - 1 run ``times`` times in a row.  No loop: (0, 0, 1)."""
+        """(start, stop, times): how often the run of layers from start to in front of stop is gone through.  No loop: (0, 0, 1)."""
         loop = self.raw.get("loop")
         if loop is None:
             return 0, 0, 1

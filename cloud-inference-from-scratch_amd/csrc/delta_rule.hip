@@ -1,12 +1,12 @@
 // The gated delta rule: per head a float32 memory S [dim, vdim] that every token fades, corrects and reads,
 //
-//     S <- g S;   u = beta (v - S^T k);   S <- S + k u^T;   o = S^T q
+//     S' = g S + k u^T  with the correction  u = beta (v - g S^T k),   read as  S'^T q
 //
-// with one decay g = exp(-exp(a_log) softplus(a + dt_bias)) and one step size beta = sigmoid(b) per head and token.
-// Queries, keys and values come through a causal convolution over each channel's last `taps` inputs and silu; queries
-// and keys are then brought to length one per head (x / sqrt(sum x^2 + 1e-6)), the queries scaled; head h uses query
-// and key head h / (heads / kv_heads).  Each head's o is divided by its root mean square, multiplied by a weight that the
-// heads share and by silu of its gate.  What enters is the projections' rows; everything behind them is float32.
+// where g (the decay, the exponential of -exp(a_log) times a softplus of its logit and bias) and beta (the step size, a
+// sigmoid) are one number per head and token.  In front of it stand a causal convolution over each channel's last `taps`
+// inputs with silu, for queries and keys a scaling to length one (1e-6 beside the sum of squares) and for queries a
+// factor; neighbouring heads share a query and key head.  Behind it a head's read-out is RMS-normed under a weight that
+// the heads share and gated by silu.  What enters is the projections' rows; everything behind them is float32.
 //
 // State per request slot: the memory, kept as [heads, vdim, dim] (a column of S lies in one piece), and the
 // convolutions' last taps - 1 inputs, kept per head as [heads, taps - 1, 2 dim + vdim] (a head's query, key and value

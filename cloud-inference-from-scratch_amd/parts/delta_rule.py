@@ -1,11 +1,12 @@
 """The gated delta rule: a memory of fixed size per head that is corrected, not only added to.
 
-With ``q, k`` (kv_heads x dim) and ``v`` (heads x vdim) projected, passed through a causal convolution over each channel's
-last ``taps`` inputs and silu, ``q`` and ``k`` brought to length one per head and ``q`` scaled by ``dim^-1/2``, per head
-``S <- g S``, ``u = beta (v - S^T k)``, ``S <- S + k u^T``, ``o = S^T q`` with ``beta = sigmoid(W_b x)`` and
-``g = exp(-exp(A_log) softplus(W_a x + dt_bias))``; head h uses query and key head ``h // (heads // kv_heads)``.  Each
-head's ``o`` is divided by its root mean square, multiplied by the weight ``norm`` (vdim numbers for all heads) and by
-``silu(W_g x)``, and the heads are projected.  Products run in the engine's type; everything else, and the state (the
+Queries, keys (``kv_heads`` heads of ``dim``, each serving ``heads / kv_heads`` neighbouring heads) and values (``heads``
+of ``vdim``) are projected and pass a causal convolution over each channel's last ``taps`` inputs and silu; queries and
+keys come to length one per head, queries times ``q_scale``.  A head's memory S becomes ``g S + k u^T`` with the
+correction ``u = beta (v - g S^T k)``, so that with a step size of one the memory answers k with v; the query reads the
+new memory.  Step size (a sigmoid of ``b``) and decay (``A_log``, ``dt_bias`` and a softplus of ``a``) are one number per
+head and token.  The read-out is RMS-normed per head under one weight for all heads, gated by silu of ``g`` and
+projected.  Products run in the engine's type; everything else, and the state (the
 memory [heads, vdim, dim] and the convolutions' last inputs per head), is float32.  A request's state lies in its slot and
 moves on with its tokens, so a prompt may be cut anywhere.  Kernels: ``csrc/delta_rule.hip``.
 """

@@ -1,10 +1,10 @@
 """What remakes the stream in front of a call of the run order.
 
-``JoinEmbedding``: ``x <- W [x; x0] + s_n`` with ``x0`` the embedding's rows as they entered the stream and ``s_n`` a
-vector of the entry's number n: the first step of a run of layers that repeats.  The two halves of a row lie side by
-side in one tensor of the activation type: the embedding kernel fills the right half once a step, the kernel that ends
-the layer in front of an entry leaves the stream in the left one, and one product with float32 results makes the new
-stream.  The vector is handed on to the norm behind it, which adds it in its own kernel.
+``JoinEmbedding``: a stream row and the embedding's row as it entered the stream, side by side, go through one product,
+and a vector that belongs to the entry's number n joins the result: the first step of a run of layers that repeats.
+The two halves of a row lie in one tensor of the activation type: the embedding kernel fills the right half once a step,
+the kernel that ends the layer in front of an entry leaves the stream in the left one, and one product with float32
+results makes the new stream.  The vector is handed on to the norm behind it, which adds it in its own kernel.
 """
 
 from __future__ import annotations

@@ -10,7 +10,7 @@ the position in other ways.  Every step is a parameter of the part and may be le
   itself (``slope_base = b``: head h of H loses ``2^(-b (h + 1) / H) * (i - j)``);
 * a window (``window``: the token itself and the ``window - 1`` before it; with ``keep_first`` the first that many
   tokens of the sequence stay visible from behind the window too, at their own positions), or chunks (``chunk``: the token sees the
-  keys of its own chunk of that many positions up to itself; chunks are counted from position 0 of the sequence);
+  keys of its own chunk of that many positions up to itself; the first chunk begins at position 0);
 * biases on the projections of queries, keys and values (``qkv_bias``);
 * a rotation of the first numbers of every query and key head by the position (``position``: a position part such
   as ``rotary_pairs``, applied after the heads' norm);
