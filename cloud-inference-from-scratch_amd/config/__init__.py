@@ -1,5 +1,6 @@
 from .engine_config import EngineConfig, build_engine_config, canonical_dtype
 from .givizen import GivizenConfig
+from .nogapel import NogapelConfig
 from .nokipel import NokipelConfig
 from .nopunex import NopunexConfig
 from .polosun import PolosunConfig
@@ -22,9 +23,10 @@ register_architecture("Givizen", GivizenConfig)
 register_architecture("Nokipel", NokipelConfig)
 register_architecture("Senuvik", SenuvikConfig)
 register_architecture("Nopunex", NopunexConfig)
+register_architecture("Nogapel", NogapelConfig)
 
 __all__ = [
     "ARCHITECTURES", "Architecture", "ConfigError", "EngineConfig", "GivizenConfig", "LayerCall", "LayerSpec",
-    "ModelSpec", "NokipelConfig", "NopunexConfig", "PartSpec", "PolosunConfig", "Qwen2Config", "SenuvikConfig", "architecture_of", "build_engine_config",
+    "ModelSpec", "NogapelConfig", "NokipelConfig", "NopunexConfig", "PartSpec", "PolosunConfig", "Qwen2Config", "SenuvikConfig", "architecture_of", "build_engine_config",
     "canonical_dtype", "config_from_dict", "load_config", "register_architecture",
 ]

@@ -43,7 +43,8 @@ class LayerSpec:
     ``feed_forward``) to the sub-prefix of the checkpoint's tensor names.
     ``options`` are the arrangement's own constants (a factor on the branches, the layer's depth), which
     the block class reads.  ``norm1_out`` and ``norm2_out`` are the norms on the sublayers' outputs of an arrangement
-    that has norms on both sides of a sublayer.
+    that has norms on both sides of a sublayer.  ``side`` is a branch of its own that follows the layer's other ones
+    (a part of the role "side").
     """
 
     mixer: PartSpec
@@ -55,6 +56,7 @@ class LayerSpec:
     options: tuple[tuple[str, Any], ...] = ()
     norm1_out: PartSpec | None = None
     norm2_out: PartSpec | None = None
+    side: PartSpec | None = None
 
     def option(self, name: str, default: Any = None) -> Any:
         return dict(self.options).get(name, default)
@@ -107,6 +109,12 @@ class ModelSpec:
     # its tensors' names
     entry: PartSpec | None = None
     entry_name: str = "entry"
+    # a norm of the embedding's rows, with which the stream begins
+    embedding_norm: PartSpec | None = None
+    embedding_norm_name: str = "embed.norm"
+    # a second table looked up by token, of that many columns, which the layers' ``side`` parts read; 0: none
+    side_table_columns: int = 0
+    side_table_name: str = "side.embed"
     extra: dict[str, Any] = field(default_factory=dict, compare=False)
 
     def __post_init__(self) -> None:

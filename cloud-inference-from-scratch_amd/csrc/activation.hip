@@ -118,3 +118,43 @@ CIE_API int cie_soft_cap(void* stream, float* x, long count, float cap) {
     soft_cap_kernel<<<static_cast<unsigned>((count + 255) / 256), 256, 0, static_cast<hipStream_t>(stream)>>>(x, count, cap);
     return cie_after_launch();
 }
+
+// The square of relu over a matrix whose rows lie ld_in / ld_out numbers apart: out[t, i] = max(in[t, i], 0)^2, V
+// numbers a thread.
+template <typename T, int V>
+__global__ void squared_relu_kernel(const T* __restrict__ in, long ld_in, T* __restrict__ out, long ld_out, int columns) {
+    const int i = (blockIdx.y * blockDim.x + threadIdx.x) * V;
+    if (i >= columns) return;
+    const T* src = in + static_cast<size_t>(blockIdx.x) * ld_in + i;
+    T* dst = out + static_cast<size_t>(blockIdx.x) * ld_out + i;
+    if constexpr (V == 8) {
+        const uint4 raw = *reinterpret_cast<const uint4*>(src);
+        const uint32_t w[4] = {raw.x, raw.y, raw.z, raw.w};
+        uint32_t packed[4];
+#pragma unroll
+        for (int q = 0; q < 4; ++q)
+            packed[q] = pack_bf16(squared_relu(__uint_as_float(w[q] << 16)), squared_relu(__uint_as_float(w[q] & 0xffff0000u)));
+        *reinterpret_cast<uint4*>(dst) = uint4{packed[0], packed[1], packed[2], packed[3]};
+    } else {
+        *dst = from_float<T>(squared_relu(to_float(*src)));
+    }
+}
+
+CIE_API int cie_squared_relu(void* stream, int dtype, const void* in, long ld_in, void* out, long ld_out, int tokens,
+                             int columns) {
+    if (tokens < 0 || columns <= 0 || ld_in < columns || ld_out < columns || (columns + 255) / 256 > 65535) return CIE_BAD_ARGUMENT;
+    if (tokens == 0) return CIE_OK;
+    hipStream_t s = static_cast<hipStream_t>(stream);
+    const bool by_eight = dtype == CIE_BF16 && columns % 8 == 0 && ld_in % 8 == 0 && ld_out % 8 == 0 &&
+                          ((reinterpret_cast<uintptr_t>(in) | reinterpret_cast<uintptr_t>(out)) & 15) == 0;
+    const dim3 grid(tokens, (columns + 255) / 256), grid8(tokens, (columns / 8 + 255) / 256);
+    if (by_eight)
+        squared_relu_kernel<bf16_t, 8><<<grid8, 256, 0, s>>>(static_cast<const bf16_t*>(in), ld_in, static_cast<bf16_t*>(out), ld_out, columns);
+    else if (dtype == CIE_F32)
+        squared_relu_kernel<float, 1><<<grid, 256, 0, s>>>(static_cast<const float*>(in), ld_in, static_cast<float*>(out), ld_out, columns);
+    else if (dtype == CIE_BF16)
+        squared_relu_kernel<bf16_t, 1><<<grid, 256, 0, s>>>(static_cast<const bf16_t*>(in), ld_in, static_cast<bf16_t*>(out), ld_out, columns);
+    else
+        return CIE_BAD_ARGUMENT;
+    return cie_after_launch();
+}

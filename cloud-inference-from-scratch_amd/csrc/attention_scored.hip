@@ -164,6 +164,189 @@ heads_prepare_kernel(const T* __restrict__ proj, int proj_stride, int q_off, int
     }
 }
 
+// The same preparation for heads whose projections first pass a causal convolution over the tokens, channel by channel:
+//   y_t = sum_j taps[c, j] u_(t - n + 1 + j)   (the last tap meets the token itself),
+// with the inputs of the tokens before the step in `past` [slots, max(n - 1, 1), channels] (float32, oldest first; the
+// channels are those of the queries, the keys and the values in that order), and for values that are mixed with those
+// that an earlier layer of the same step made of the same tokens:
+//   v <- (1 - mix) v + mix * v_first,   the mixed v being what is cached.
+// A layer that is the first of those leaves its convolved values in `first_out`.
+template <typename T>
+struct ConvHeads {
+    const T* taps;         // [channels, n]; null: the projection as it is (n = 1)
+    int n;
+    float* past;
+    const int* q_start_loc;
+    int single;            // every sequence of the step brings one token: the kernel also moves `past` on
+    T* first_out;          // [tokens, kv_heads * vdim] or null
+    const T* first_in;     // likewise
+    float mix;
+};
+constexpr int kMaxConvTaps = 16;  // inputs that `past` keeps, at most, and one
+
+// Numbers d and d + 1 of a row; as one load where every row's start allows it.
+__device__ __forceinline__ float2 load_pair(const float* p, int d, int n, bool paired) {
+    if (paired) return *reinterpret_cast<const float2*>(p + d);
+    return float2{p[d], d + 1 < n ? p[d + 1] : 0.f};
+}
+__device__ __forceinline__ float2 load_pair(const bf16_t* p, int d, int n, bool paired) {
+    if (paired) {
+        const uint32_t raw = *reinterpret_cast<const uint32_t*>(p + d);
+        return float2{__uint_as_float(raw << 16), __uint_as_float(raw & 0xffff0000u)};
+    }
+    return float2{to_float(p[d]), d + 1 < n ? to_float(p[d + 1]) : 0.f};
+}
+__device__ __forceinline__ void store_pair(float* p, float2 v) { *reinterpret_cast<float2*>(p) = v; }
+__device__ __forceinline__ void store_pair(bf16_t* p, float2 v) { *reinterpret_cast<uint32_t*>(p) = pack_bf16(v.x, v.y); }
+
+// One wave per (token, head slot) as above; a lane holds neighbours 2l, 2l + 1 (and those 128 further on).  TAPS: the
+// convolution's taps where the kernel knows them (their loads then travel together), 0: c.n of them.
+template <typename T, int TAPS>
+__global__ void __launch_bounds__(256)
+heads_conv_prepare_kernel(const T* __restrict__ proj, int proj_stride, int q_off, int k_off, int v_off, ConvHeads<T> c,
+                          const float* __restrict__ q_weight, const float* __restrict__ k_weight, int norm_mode, float eps,
+                          float temp_coef, int temp_every, const int* __restrict__ positions,
+                          const int* __restrict__ seq_of_token, const int* __restrict__ seq_slot,
+                          const int* __restrict__ block_table, int table_width, T* __restrict__ q_out,
+                          T* __restrict__ k_pool, T* __restrict__ v_pool, int tokens, int q_heads, int kv_heads, int dim,
+                          int vdim, int D, int DV, int page_shift, const float* __restrict__ cos_table,
+                          const float* __restrict__ sin_table, int rot, int neighbours) {
+    __shared__ float staged[4][256];  // a head of each wave, for partners that another lane holds
+    const int lane = threadIdx.x % kWave;
+    const int wave = threadIdx.x / kWave;
+    const int slots = q_heads + 2 * kv_heads;
+    const long unit = static_cast<long>(blockIdx.x) * 4 + wave;
+    if (unit >= static_cast<long>(tokens) * slots) return;
+    const int token = static_cast<int>(unit / slots);
+    const int slot = static_cast<int>(unit - static_cast<long>(token) * slots);
+    const bool is_q = slot < q_heads, is_v = slot >= q_heads + kv_heads;
+    const int head = is_q ? slot : is_v ? slot - q_heads - kv_heads : slot - q_heads;
+    const int n = is_v ? vdim : dim;
+    const int padded = is_v ? DV : D;
+    const int column = (is_q ? q_off : is_v ? v_off : k_off) + head * n;
+    const int channels = (q_heads + kv_heads) * dim + kv_heads * vdim;
+    const int channel = is_v ? (q_heads + kv_heads) * dim + head * vdim : (is_q ? 0 : q_heads * dim) + head * dim;
+    const int pos = positions[token];
+    const int seq = seq_of_token[token];
+    const int slot_row = seq_slot[seq];
+    const int taps = TAPS > 0 ? TAPS : c.n;
+    const int first = c.q_start_loc[seq];
+    const int t = token - first;  // the token's place in the step's portion of its sequence
+    float* before = c.past + static_cast<size_t>(slot_row) * max(taps - 1, 1) * channels + channel;
+    const bool paired = (((proj_stride | column | n) & 1) == 0);  // (the base of `proj` is aligned to a pair)
+    const T* src = proj + static_cast<size_t>(first) * proj_stride + column;
+
+    float2 y[2];
+    float sum_sq = 0.f;
+#pragma unroll
+    for (int i = 0; i < 2; ++i) {
+        const int d = 2 * lane + 128 * i;
+        y[i] = float2{0.f, 0.f};
+        if (d >= n) continue;
+        const bool two = d + 1 < n;
+        if (!c.taps) {
+            y[i] = load_pair(src + static_cast<size_t>(t) * proj_stride, d, n, paired);
+        } else {
+            const T* w = c.taps + static_cast<size_t>(channel + d) * taps;
+            float2 in[TAPS > 0 ? TAPS : kMaxConvTaps];
+#pragma unroll
+            for (int j = 0; j < (TAPS > 0 ? TAPS : kMaxConvTaps); ++j) {
+                if (TAPS == 0 && j >= taps) break;
+                const int from = t - (taps - 1) + j;
+                if (from >= 0) {
+                    in[j] = load_pair(src + static_cast<size_t>(from) * proj_stride, d, n, paired);
+                } else {
+                    const float* old = before + static_cast<size_t>(taps - 1 + from) * channels + d;
+                    in[j] = float2{old[0], two ? old[1] : 0.f};
+                }
+            }
+#pragma unroll
+            for (int j = 0; j < (TAPS > 0 ? TAPS : kMaxConvTaps); ++j) {
+                if (TAPS == 0 && j >= taps) break;
+                y[i].x = fmaf(to_float(w[j]), in[j].x, y[i].x);
+                if (two) y[i].y = fmaf(to_float(w[taps + j]), in[j].y, y[i].y);
+            }
+            if (c.single) {  // (t = 0: in[j] is what the state held at j, and the last is the token's own)
+#pragma unroll
+                for (int j = 1; j < (TAPS > 0 ? TAPS : kMaxConvTaps); ++j) {
+                    if (TAPS == 0 && j >= taps) break;
+                    float* now = before + static_cast<size_t>(j - 1) * channels + d;
+                    now[0] = in[j].x;
+                    if (two) now[1] = in[j].y;
+                }
+            }
+        }
+        sum_sq += y[i].x * y[i].x + y[i].y * y[i].y;
+    }
+    const size_t page = is_q ? 0 : static_cast<size_t>(block_table[static_cast<size_t>(slot_row) * table_width + (pos >> page_shift)]);
+    const int in_page = pos & ((1 << page_shift) - 1);
+    if (is_v) {
+        T* dst = v_pool + ((page * kv_heads + head) * DV << page_shift) + in_page;
+        const size_t at = (static_cast<size_t>(token) * kv_heads + head) * vdim;
+#pragma unroll
+        for (int i = 0; i < 2; ++i) {
+            const int d = 2 * lane + 128 * i;
+            if (d >= padded) continue;
+            float x[2] = {y[i].x, y[i].y};
+#pragma unroll
+            for (int e = 0; e < 2; ++e) {
+                if (d + e < n) {
+                    if (c.first_out) c.first_out[at + d + e] = from_float<T>(x[e]);
+                    if (c.first_in) x[e] = (1.0f - c.mix) * x[e] + c.mix * to_float(c.first_in[at + d + e]);
+                }
+                dst[static_cast<size_t>(d + e) << page_shift] = from_float<T>(x[e]);
+            }
+        }
+        return;
+    }
+    float factor = 1.f;
+    if (norm_mode != 0) factor = 1.0f / sqrtf(wave_sum(sum_sq) / static_cast<float>(dim) + eps);
+    const float* weight = norm_mode == 2 ? (is_q ? q_weight : k_weight) : nullptr;
+    float after = 1.f;  // the queries' factor of the position
+    if (is_q && temp_every > 0) after = 1.0f + temp_coef * logf(static_cast<float>((pos + 1) / temp_every) + 1.0f);
+#pragma unroll
+    for (int i = 0; i < 2; ++i) {
+        const int d = 2 * lane + 128 * i;
+        if (d >= n) continue;
+        y[i].x *= factor * (weight ? weight[d] : 1.f);
+        y[i].y *= factor * (weight && d + 1 < n ? weight[d + 1] : 1.f);
+        if (rot > 0 && !neighbours) {
+            staged[wave][d] = y[i].x;
+            if (d + 1 < n) staged[wave][d + 1] = y[i].y;
+        }
+    }
+    __builtin_amdgcn_wave_barrier();  // (a wave's LDS operations keep their order; the compiler is held to it too)
+    T* dst = is_q ? q_out + (static_cast<size_t>(token) * q_heads + head) * D
+                  : k_pool + (((page * kv_heads + head) << page_shift) + in_page) * D;
+    const int half = rot / 2;
+    const float* cos_row = rot > 0 ? cos_table + static_cast<size_t>(pos) * half : nullptr;
+    const float* sin_row = rot > 0 ? sin_table + static_cast<size_t>(pos) * half : nullptr;
+#pragma unroll
+    for (int i = 0; i < 2; ++i) {
+        const int d = 2 * lane + 128 * i;
+        if (d >= padded) continue;
+        float2 x = y[i];
+        if (d < rot && neighbours) {  // (rot is even: a pair turns or stays as one)
+            const float cs = cos_row[d >> 1], sn = sin_row[d >> 1];
+            x = float2{y[i].x * cs - y[i].y * sn, y[i].y * cs + y[i].x * sn};
+        } else if (rot > 0 && d < rot) {
+            float turned[2] = {x.x, x.y};
+#pragma unroll
+            for (int e = 0; e < 2; ++e) {
+                const int at = d + e;
+                const bool is_u = at < half;
+                const float mate = staged[wave][is_u ? at + half : at - half];
+                const int angle = is_u ? at : at - half;
+                turned[e] = is_u ? turned[e] * cos_row[angle] - mate * sin_row[angle] : turned[e] * cos_row[angle] + mate * sin_row[angle];
+            }
+            x = float2{turned[0], turned[1]};
+        }
+        x.x *= after;
+        x.y *= after;
+        store_pair(dst + d, x);
+    }
+}
+
 // ------------------------------------------------------------------------------------------------ generic
 // One workgroup (4 waves) per (query token, query head); each wave takes 64-key chunks in turn, one key per
 // lane for the scores, then one slice of the value head per lane; the four running (max, sum, accumulator)
@@ -219,7 +402,7 @@ scored_attention_generic_kernel(const T* __restrict__ q, const T* __restrict__ k
                                 const int* __restrict__ block_table, int table_width,
                                 const int* __restrict__ positions, const int* __restrict__ seq_of_token,
                                 const int* __restrict__ seq_slot, const T* __restrict__ gate, int gate_stride,
-                                T* __restrict__ out, int q_heads, int kv_heads, int D, int DV, int page_size,
+                                T* __restrict__ out, long out_stride, int q_heads, int kv_heads, int D, int DV, int page_size,
                                 int maps, ScoreShape shape) {
     extern __shared__ float lds[];
     float* q_s = lds;            // [D]
@@ -335,7 +518,7 @@ scored_attention_generic_kernel(const T* __restrict__ q, const T* __restrict__ k
         by = shape.factor / sqrtf(block_sum(sum, scratch) / static_cast<float>(shape.vdim) + shape.eps);
     }
     const T* gates = gate ? gate + static_cast<size_t>(token) * gate_stride : nullptr;
-    T* out_row = out + (static_cast<size_t>(token) * q_heads + head) * DV;
+    T* out_row = out + static_cast<size_t>(token) * out_stride + head * DV;
     for (int d = threadIdx.x; d < DV; d += blockDim.x) {
         float x = d < shape.vdim ? done_s[d] * by : 0.f;
         if (gates && d < shape.vdim)
@@ -371,7 +554,8 @@ struct ScoredArgs {
     const int* q_start_loc;
     const bf16_t* gate;       // [tokens, gate_stride], column = head; or null
     int gate_stride;
-    bf16_t* out;              // [tokens, q_heads, DV]
+    bf16_t* out;              // [tokens, q_heads, DV], rows out_stride numbers apart
+    long out_stride;
     int q_heads;
     int kv_heads;
     int page_shift;
@@ -405,7 +589,7 @@ __device__ __forceinline__ void write_head(const ScoredArgs& a, const float (&x)
     }
     const bf16_t* gates = a.gate ? a.gate + token * a.gate_stride : nullptr;
     if (gates && !a.shape.gate_wide) factor *= 1.0f / (1.0f + __expf(-to_float(gates[head])));
-    bf16_t* dst = a.out + (token * a.q_heads + head) * DV;
+    bf16_t* dst = a.out + token * a.out_stride + head * DV;
 #pragma unroll
     for (int i = 0; i < N; ++i) {
         const int d = lane + i * kWave;
@@ -839,6 +1023,51 @@ CIE_API int cie_heads_prepare(void* stream, int dtype, const void* proj, int pro
     return cie_after_launch();
 }
 
+// The preparation behind a convolution (see heads_conv_prepare_kernel).  norm_mode 0, 1 or 2; heads of up to 256 numbers.
+CIE_API int cie_heads_conv_prepare(void* stream, int dtype, const void* proj, int proj_stride, int q_off, int k_off,
+                                   int v_off, const void* taps, int n_taps, float* past, const int* q_start_loc, int single,
+                                   void* first_out, const void* first_in, float mix, const float* q_weight,
+                                   const float* k_weight, int norm_mode, float eps, float temp_coef, int temp_every,
+                                   const int* positions, const int* seq_of_token, const int* seq_slot,
+                                   const int* block_table, int table_width, void* q_out, void* k_pool, void* v_pool,
+                                   int tokens, int q_heads, int kv_heads, int dim, int vdim, int D, int DV, int page_size,
+                                   const float* cos_table, const float* sin_table, int rot, int neighbours) {
+    if (rot < 0 || rot % 2 || rot > dim || (rot > 0 && (!cos_table || !sin_table))) return CIE_BAD_ARGUMENT;
+    if (tokens < 0 || q_heads <= 0 || kv_heads <= 0 || dim <= 0 || vdim <= 0 || D < dim || DV < vdim || D > 256 || DV > 256 ||
+        D % 2 || DV % 2 || page_size <= 0 || (page_size & (page_size - 1)) || table_width <= 0 || norm_mode < 0 ||
+        norm_mode > 2 || (norm_mode == 2 && (!q_weight || !k_weight)) || (norm_mode != 0 && !(eps > 0.f)) || temp_every < 0 ||
+        q_off < 0 || k_off < 0 || v_off < 0 || proj_stride <= 0 || n_taps < 1 || n_taps > kMaxConvTaps || !q_start_loc ||
+        (!taps && n_taps != 1) || (n_taps > 1 && !past))
+        return CIE_BAD_ARGUMENT;
+    if (tokens == 0) return CIE_OK;
+    int page_shift = 0;
+    while ((1 << page_shift) < page_size) ++page_shift;
+    const long blocks = (static_cast<long>(tokens) * (q_heads + 2 * kv_heads) + 3) / 4;
+    if (blocks > 0x7fffffffL) return CIE_BAD_ARGUMENT;
+    hipStream_t s = static_cast<hipStream_t>(stream);
+#define CIE_CONV_HEADS(T, TAPS)                                                                                          \
+    heads_conv_prepare_kernel<T, TAPS><<<static_cast<unsigned>(blocks), 256, 0, s>>>(                                    \
+        static_cast<const T*>(proj), proj_stride, q_off, k_off, v_off,                                                   \
+        ConvHeads<T>{static_cast<const T*>(taps), n_taps, past, q_start_loc, single, static_cast<T*>(first_out),         \
+                     static_cast<const T*>(first_in), mix},                                                              \
+        q_weight, k_weight, norm_mode, eps, temp_coef, temp_every, positions, seq_of_token, seq_slot, block_table,       \
+        table_width, static_cast<T*>(q_out), static_cast<T*>(k_pool), static_cast<T*>(v_pool), tokens, q_heads, kv_heads, \
+        dim, vdim, D, DV, page_shift, cos_table, sin_table, rot, neighbours)
+#define CIE_CONV_HEADS_TYPE(T)                     \
+    do {                                           \
+        if (n_taps == 2) CIE_CONV_HEADS(T, 2);     \
+        else if (n_taps == 3) CIE_CONV_HEADS(T, 3); \
+        else if (n_taps == 4) CIE_CONV_HEADS(T, 4); \
+        else CIE_CONV_HEADS(T, 0);                 \
+    } while (0)
+    if (dtype == CIE_F32) CIE_CONV_HEADS_TYPE(float);
+    else if (dtype == CIE_BF16) CIE_CONV_HEADS_TYPE(bf16_t);
+    else return CIE_BAD_ARGUMENT;
+#undef CIE_CONV_HEADS_TYPE
+#undef CIE_CONV_HEADS
+    return cie_after_launch();
+}
+
 CIE_API int cie_scored_attention_generic(void* stream, int dtype, const void* q, const void* k_pool,
                                          const void* v_pool, const int* block_table, int table_width,
                                          const int* positions, const int* seq_of_token, const int* seq_slot,
@@ -846,10 +1075,10 @@ CIE_API int cie_scored_attention_generic(void* stream, int dtype, const void* q,
                                          int kv_heads, int D, int DV, int page_size, int window, float scale,
                                          float softcap, const float* slopes, const float* sinks, int chunk,
                                          int keep, int gate_wide, int real_vdim, int maps, float lambda, float factor,
-                                         float eps) {
+                                         float eps, long out_stride) {
     if (tokens < 0 || q_heads <= 0 || kv_heads <= 0 || q_heads % kv_heads || D <= 0 || D % 8 || DV <= 0 || DV % 8 ||
         DV > kWave * kMaxWideSlices || page_size <= 0 || table_width <= 0 || q_heads > 65535 || real_vdim <= 0 ||
-        real_vdim > DV || maps < 1 || maps > 2 || (maps == 2 && !(eps > 0.f)) ||
+        real_vdim > DV || maps < 1 || maps > 2 || (maps == 2 && !(eps > 0.f)) || out_stride < static_cast<long>(q_heads) * DV ||
         (gate && gate_stride < (gate_wide ? q_heads * real_vdim : q_heads)))
         return CIE_BAD_ARGUMENT;
     if (tokens == 0) return CIE_OK;
@@ -862,7 +1091,7 @@ CIE_API int cie_scored_attention_generic(void* stream, int dtype, const void* q,
 #define CIE_GENERIC(T, SLICES)                                                                                          \
     scored_attention_generic_kernel<T, SLICES><<<grid, 256, lds, s>>>(                                                  \
         static_cast<const T*>(q), static_cast<const T*>(k_pool), static_cast<const T*>(v_pool), block_table, table_width, \
-        positions, seq_of_token, seq_slot, static_cast<const T*>(gate), gate_stride, static_cast<T*>(out), q_heads, kv_heads, \
+        positions, seq_of_token, seq_slot, static_cast<const T*>(gate), gate_stride, static_cast<T*>(out), out_stride, q_heads, kv_heads, \
         D, DV, page_size, maps, shape)
     const bool wide = DV > kWave * kMaxSlices;
     if (dtype == CIE_F32 && !wide) CIE_GENERIC(float, kMaxSlices);
@@ -884,14 +1113,15 @@ CIE_API int cie_scored_attention_mfma(void* stream, const void* q, const void* k
                                       int page_size, int tokens_per_tile, int row_tiles, int window, float scale,
                                       float softcap, const float* slopes, const float* sinks, int n_splits,
                                       int keys_per_split, float* part_o, float* part_ml, int chunk, int keep,
-                                      int gate_wide, int real_vdim, int maps, float lambda, float factor, float eps) {
+                                      int gate_wide, int real_vdim, int maps, float lambda, float factor, float eps,
+                                      long out_stride) {
     if (chunk < 0 || (chunk > 0 && window > 0) || keep < 0 || (keep > 0 && window <= 0)) return CIE_BAD_ARGUMENT;
     if (n_tiles < 0 || q_heads <= 0 || kv_heads <= 0 || q_heads % kv_heads || page_size < 4 ||
         (page_size & (page_size - 1)) || table_width <= 0 || tokens_per_tile < 1 || kv_heads > 65535 ||
         (tile_seq == nullptr) != (tile_q0 == nullptr) || maps < 1 || maps > 2 || (maps == 2 && (!(eps > 0.f) || sinks)) ||
         real_vdim <= 0 || real_vdim > DV || (gate && gate_stride < (gate_wide ? q_heads * real_vdim : q_heads)))
         return CIE_BAD_ARGUMENT;
-    if (tokens_per_tile * (q_heads / kv_heads) * maps > 16 * row_tiles) return CIE_BAD_ARGUMENT;
+    if (tokens_per_tile * (q_heads / kv_heads) * maps > 16 * row_tiles || out_stride < static_cast<long>(q_heads) * DV) return CIE_BAD_ARGUMENT;
     if (n_splits < 1 || n_splits > 65535 ||
         (n_splits > 1 && (keys_per_split < 128 || keys_per_split % 128 || !part_o || !part_ml)))
         return CIE_BAD_ARGUMENT;
@@ -915,6 +1145,7 @@ CIE_API int cie_scored_attention_mfma(void* stream, const void* q, const void* k
     a.gate = static_cast<const bf16_t*>(gate);
     a.gate_stride = gate_stride;
     a.out = static_cast<bf16_t*>(out);
+    a.out_stride = out_stride;
     a.q_heads = q_heads;
     a.kv_heads = kv_heads;
     a.page_shift = 0;

@@ -6,7 +6,8 @@
 // Such a product is bound by streaming W once and by the number of kernel launches
 // (no kernel on this GPU finishes in under about 5 microseconds), so the epilogue
 // takes over the neighbour's work:
-//   BF16 / F32  C[m,n] = acc + bias[n]
+//   BF16 / F32  C[m,n] = acc + bias[n]; of BF16 the columns from `split` on may pass through the square of relu into a
+//               matrix of their own (a feed-forward's first product that shares its rows with another product)
 //   SILU        W stacks gate rows over up rows: C[m,n] = silu(acc_gate) * acc_up, bf16
 //   RESID       residual[m,n] += acc + bias[n] (float32, in place), and the partial sums of
 //               squares of the new residual row (one per 16 columns) are written, so that the
@@ -34,6 +35,7 @@
 // this GPU than the whole product.
 #include <type_traits>
 
+#include "activation_forms.h"
 #include "common.h"
 
 namespace {
@@ -84,6 +86,11 @@ struct FusedArgs {
     // product is multiplied by each row's 1/rms, whose sums of squares the lanes gather on the way.
     const float* fold_residual;  // [M, K] float32 or null
     const float* fold_weight;    // [K] float32
+    // BF16: columns n >= split are not stored in C (whose rows then have `split` numbers) but go, as max(v, 0)^2, to
+    // act_out[m * act_ld + n - split].  Without it split = N.
+    int split;
+    bf16_t* act_out;
+    long act_ld;
     RopeArgs rope;         // ROPE only
 };
 
@@ -129,8 +136,10 @@ __device__ __forceinline__ void store_tile(const FusedArgs& a, const floatx4& ac
                 unsafeAtomicAdd(a.residual + static_cast<size_t>(m) * a.N + n, v);
             else if (EPI == EPI_F32)
                 static_cast<float*>(a.c)[static_cast<size_t>(m) * a.N + n] = v;
+            else if (n < a.split)
+                static_cast<bf16_t*>(a.c)[static_cast<size_t>(m) * a.split + n] = from_float<bf16_t>(v);
             else
-                static_cast<bf16_t*>(a.c)[static_cast<size_t>(m) * a.N + n] = from_float<bf16_t>(v);
+                a.act_out[static_cast<size_t>(m) * a.act_ld + (n - a.split)] = from_float<bf16_t>(squared_relu(v));
         }
     }
 }
@@ -1027,11 +1036,14 @@ int launch_shared_rows(hipStream_t s, int waves, int k_parts, const FusedArgs& a
 // norm_weight [N] float32 and scaled_out [M, N] bf16 (both or neither; RESID only): the epilogue also writes
 // the new residual times the weight.  row_sumsq [M, sumsq_parts] and eps (SILU with one row tile only): the
 // rows of `a` lack the factor rsqrt(sum of the row's partial sums / K + eps), applied before the SiLU.
+// act_out (BF16 only): columns from `split` on go there, squared behind relu; `c` is [M, split].
 CIE_API int cie_gemm_fused(void* stream, const void* a, int lda, const void* w, const void* bias, void* c,
                            float* residual, float* sumsq, int M, int N, int K, int epilogue, int row_tiles,
                            int waves, int column_tiles, const float* norm_weight, void* scaled_out,
-                           const float* row_sumsq, int sumsq_parts, float eps) {
+                           const float* row_sumsq, int sumsq_parts, float eps, int split, void* act_out,
+                           long act_ld) {
     if (M <= 0 || N <= 0 || K <= 0 || K % 8 || !a || !w || lda < K || lda % 8) return CIE_BAD_ARGUMENT;
+    if (act_out && (epilogue != EPI_BF16 || split < 1 || split >= N || act_ld < N - split)) return CIE_BAD_ARGUMENT;
     if (row_tiles != 1 && row_tiles != 2 && row_tiles != 4) return CIE_BAD_ARGUMENT;
     if (waves != 1 && waves != 2 && waves != 4 && waves != 8) return CIE_BAD_ARGUMENT;
     if (epilogue == EPI_SILU && (N % 2 || bias)) return CIE_BAD_ARGUMENT;
@@ -1062,6 +1074,9 @@ CIE_API int cie_gemm_fused(void* stream, const void* a, int lda, const void* w, 
     f.eps = eps;
     f.fold_residual = nullptr;
     f.fold_weight = nullptr;
+    f.split = act_out ? split : N;
+    f.act_out = static_cast<bf16_t*>(act_out);
+    f.act_ld = act_ld;
     f.rope = RopeArgs{};
     hipStream_t s = static_cast<hipStream_t>(stream);
     switch (epilogue) {
@@ -1129,6 +1144,9 @@ int qkv_rope(void* stream, const void* a, int lda, const void* w, const void* bi
     f.eps = 0.f;
     f.fold_residual = nullptr;
     f.fold_weight = nullptr;
+    f.split = N;
+    f.act_out = nullptr;
+    f.act_ld = 0;
     f.rope = RopeArgs{cos_table, sin_table, positions, seq_of_token, seq_slot, block_table, table_width,
                       static_cast<bf16_t*>(k_pool), static_cast<bf16_t*>(v_pool), q_heads, kv_heads, head_dim,
                       page_size, rotate, write_kv};
@@ -1222,6 +1240,9 @@ CIE_API int cie_gemm_shared_rows(void* stream, const void* a, int lda, const voi
     f.eps = eps;
     f.fold_residual = nullptr;
     f.fold_weight = nullptr;
+    f.split = N;
+    f.act_out = nullptr;
+    f.act_ld = 0;
     f.rope = RopeArgs{};
     hipStream_t s = static_cast<hipStream_t>(stream);
     switch (epilogue) {

@@ -53,6 +53,8 @@ class StepBatch:
     # where token_feed[t] >= 0 (both int32 on the device)
     token_feed: Any = None
     token_pool: Any = None
+    # what one layer of a step hands to later ones (the model empties it at the step's start): tensors by name
+    carried: dict = field(default_factory=dict)
     _tiles: dict = field(default_factory=dict)
 
     @property

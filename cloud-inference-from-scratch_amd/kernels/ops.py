@@ -110,12 +110,12 @@ def _check_pools(k_pool: torch.Tensor, v_pool: torch.Tensor, dtype: torch.dtype,
 # ---------------------------------------------------------------------------
 def embed(table: torch.Tensor, ids: torch.Tensor, out: Optional[torch.Tensor] = None,
           feed: Optional[torch.Tensor] = None, pool: Optional[torch.Tensor] = None, scale: float = 1.0,
-          rows: Optional[torch.Tensor] = None) -> torch.Tensor:
+          rows: Optional[torch.Tensor] = None, ids_out: Optional[torch.Tensor] = None) -> torch.Tensor:
     """``out[t] = float32(table[ids[t]]) * scale``; ids int32 [T] (already checked against the vocabulary).
     With ``feed`` (int32 [T]) and ``pool`` (int32): row t takes ``pool[feed[t]]`` as its id where
     ``feed[t] >= 0`` (tokens another kernel left on the device; ``feed[t]`` must index ``pool``).
     ``rows`` ([T, hidden] in the table's dtype; a view whose rows lie apart is fine) also takes the same values, rounded
-    to that dtype."""
+    to that dtype.  ``ids_out`` (int32 [T]) takes every row's token as it was taken."""
     _gpu("table", table, dims=2)
     _gpu("ids", ids, torch.int32, 1)
     vocab, hidden = table.shape
@@ -132,11 +132,50 @@ def embed(table: torch.Tensor, ids: torch.Tensor, out: Optional[torch.Tensor] = 
         raise ValueError(f"out must be {(tokens, hidden)}, is {tuple(out.shape)}")
     if rows is not None:
         _row_view("rows", rows, (tokens, hidden), (table.dtype,))
+    if ids_out is not None:
+        _gpu("ids_out", ids_out, torch.int32, 1)
+        if ids_out.shape[0] != tokens:
+            raise ValueError(f"ids_out must be [{tokens}]")
     _run("cie_embed", load_library().cie_embed(_stream(), _i(_code(table.dtype)), _ptr(table), _ptr(ids), _ptr(feed),
                                                _ptr(pool if feed is not None else None), _ptr(out), _ptr(rows),
                                                _ld(rows) if rows is not None else 0, _i(tokens), _i(hidden), _i(vocab),
-                                               _f(scale)))
+                                               _f(scale), _ptr(ids_out)))
     return out
+
+
+def embed_normed(table: torch.Tensor, ids: torch.Tensor, weight: torch.Tensor, eps: float,
+                 feed: Optional[torch.Tensor] = None, pool: Optional[torch.Tensor] = None, scale: float = 1.0,
+                 next_weight: Optional[torch.Tensor] = None, ids_out: Optional[torch.Tensor] = None
+                 ) -> tuple[torch.Tensor, Optional[torch.Tensor]]:
+    """The embedding's rows (as :func:`embed` takes them) under an RMS norm, as a float32 stream [T, hidden], and, with
+    ``next_weight`` (float32 [hidden]), the RMS norm of that stream under it, in the table's dtype."""
+    _gpu("table", table, dims=2)
+    _gpu("ids", ids, torch.int32, 1)
+    vocab, hidden = table.shape
+    tokens = ids.shape[0]
+    if feed is not None:
+        _gpu("feed", feed, torch.int32, 1)
+        if pool is None or feed.shape[0] < tokens:
+            raise ValueError("feed needs a pool and one entry per token")
+        _gpu("pool", pool, torch.int32, 1)
+    for name, w in (("weight", weight), ("next_weight", next_weight)):
+        if w is not None:
+            _gpu(name, w, torch.float32, 1)
+            if w.shape[0] != hidden:
+                raise ValueError(f"{name} must be [{hidden}], is {tuple(w.shape)}")
+    if hidden > MAX_NORM_WIDTH or not eps > 0:
+        raise ValueError(f"rows of {hidden} numbers (at most {MAX_NORM_WIDTH}), eps {eps}")
+    if ids_out is not None:
+        _gpu("ids_out", ids_out, torch.int32, 1)
+        if ids_out.shape[0] != tokens:
+            raise ValueError(f"ids_out must be [{tokens}]")
+    out = torch.empty((tokens, hidden), dtype=torch.float32, device=table.device)
+    normed = torch.empty((tokens, hidden), dtype=table.dtype, device=table.device) if next_weight is not None else None
+    _run("cie_embed_normed", load_library().cie_embed_normed(
+        _stream(), _i(_code(table.dtype)), _ptr(table), _ptr(ids), _ptr(feed), _ptr(pool if feed is not None else None),
+        _ptr(weight), _ptr(out), _ptr(ids_out), _ptr(next_weight), _ptr(normed), _i(tokens), _i(hidden), _i(vocab), _f(scale),
+        _f(eps)))
+    return out, normed
 
 
 MAX_NORM_WIDTH = 16384  # a row of the norm kernels is held in 64 KB of LDS as float32
@@ -448,7 +487,8 @@ def gemm_fused(weight: torch.Tensor, epilogue: int, a: torch.Tensor, bias: Optio
                residual_out: Optional[torch.Tensor] = None, sumsq_out: Optional[torch.Tensor] = None,
                plan: Optional[tuple[int, int, int]] = None,
                norm_weight: Optional[torch.Tensor] = None, scaled_out: Optional[torch.Tensor] = None,
-               row_sumsq: Optional[torch.Tensor] = None, eps: float = 0.0) -> torch.Tensor:
+               row_sumsq: Optional[torch.Tensor] = None, eps: float = 0.0,
+               act_out: Optional[torch.Tensor] = None) -> torch.Tensor:
     """Few-row matrix product ``a @ weight.T`` (bf16 operands, float32 sums) fused
     with its neighbour.  ``epilogue``: ``EPI_BF16`` / ``EPI_F32`` return
     ``a W^T + bias``; ``EPI_SILU`` (weight = gate rows over up rows) returns
@@ -459,7 +499,9 @@ def gemm_fused(weight: torch.Tensor, epilogue: int, a: torch.Tensor, bias: Optio
     rows can ride along: with ``norm_weight`` (float32 [N]) and ``scaled_out`` (bf16
     [M, N]) the former also writes the new residual times the weight, and the latter,
     given these rows as ``a`` with ``row_sumsq`` (the former's result) and ``eps``,
-    multiplies its sums by each row's ``rsqrt(mean square + eps)`` before the SiLU."""
+    multiplies its sums by each row's ``rsqrt(mean square + eps)`` before the SiLU.
+    ``act_out`` (bf16 [M, n], rows may lie apart; ``EPI_BF16``): the last n columns go there, squared behind relu, and the
+    result that comes back holds the columns in front of them."""
     _gpu("weight", weight, torch.bfloat16, 2)
     n, k = weight.shape
     if not (a.is_cuda and a.dtype == torch.bfloat16 and a.dim() == 2 and a.stride(1) == 1):
@@ -487,8 +529,15 @@ def gemm_fused(weight: torch.Tensor, epilogue: int, a: torch.Tensor, bias: Optio
     ):
         raise ValueError(f"plan {(row_tiles, waves, column_tiles)} is not one the kernel has")
     residual = sumsq = None
+    split, act_ld = n, 0
+    if act_out is not None:
+        split = n - act_out.shape[1]
+        if epilogue != EPI_BF16 or not 0 < split < n:
+            raise ValueError("columns that pass through an activation are the last ones of a bf16 result, and not all of it")
+        _row_view("act_out", act_out, (m, n - split), (torch.bfloat16,))
+        act_ld = _ld(act_out)
     if epilogue == EPI_BF16:
-        out = torch.empty((m, n), dtype=torch.bfloat16, device=device)
+        out = torch.empty((m, split), dtype=torch.bfloat16, device=device)
     elif epilogue == EPI_F32:
         out = torch.empty((m, n), dtype=torch.float32, device=device)
     elif epilogue == EPI_SILU:
@@ -526,7 +575,7 @@ def gemm_fused(weight: torch.Tensor, epilogue: int, a: torch.Tensor, bias: Optio
     _run("cie_gemm_fused", load_library().cie_gemm_fused(
         _stream(), _ptr(a), _i(lda), _ptr(weight), _ptr(bias), _ptr(None if epilogue == EPI_RESID else out),
         _ptr(residual), _ptr(sumsq), _i(m), _i(n), _i(k), _i(epilogue), _i(row_tiles), _i(waves), _i(column_tiles),
-        _ptr(norm_weight), _ptr(scaled_out), _ptr(row_sumsq), _i(parts_in), _f(eps)))
+        _ptr(norm_weight), _ptr(scaled_out), _ptr(row_sumsq), _i(parts_in), _f(eps), _i(split), _ptr(act_out), act_ld))
     return out
 
 
@@ -1745,6 +1794,55 @@ def clamped_glu(gate_up: torch.Tensor, limit: float, alpha: float, offset: float
     return out
 
 
+def squared_relu(x: torch.Tensor, out: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """``max(x, 0)^2`` of a matrix [T, n] into ``out`` (the rows of either may lie apart; a new tensor if none is given)."""
+    _row_view("x", x, tuple(x.shape), tuple(_CODES))
+    if out is None:
+        out = torch.empty(tuple(x.shape), dtype=x.dtype, device=x.device)
+    _row_view("out", out, tuple(x.shape), (x.dtype,))
+    tokens, columns = x.shape
+    _run("cie_squared_relu", load_library().cie_squared_relu(_stream(), _i(_code(x.dtype)), _ptr(x), _ld(x), _ptr(out), _ld(out),
+                                                             _i(tokens), _i(columns)))
+    return out
+
+
+def gated_token_rows(z: torch.Tensor, table: torch.Tensor, column: int, ids: torch.Tensor) -> torch.Tensor:
+    """``gelu_tanh(z[t]) * table[ids[t], column : column + dim]`` for ``z`` float32 [T, dim], in the table's dtype."""
+    _gpu("z", z, torch.float32, 2)
+    _gpu("table", table, dims=2)
+    _gpu("ids", ids, torch.int32, 1)
+    tokens, dim = z.shape
+    vocab, width = table.shape
+    if column < 0 or column + dim > width or ids.shape[0] < tokens:
+        raise ValueError(f"columns {column} .. {column + dim} of a table of {width}, {ids.shape[0]} ids for {tokens} rows")
+    out = torch.empty((tokens, dim), dtype=table.dtype, device=z.device)
+    _run("cie_gated_token_rows", load_library().cie_gated_token_rows(
+        _stream(), _i(_code(table.dtype)), _ptr(z), _ptr(table), width, _i(column), _ptr(ids), _ptr(out), _i(tokens), _i(dim),
+        _i(vocab)))
+    return out
+
+
+def stream_rows(residual: torch.Tensor, branch: Optional[torch.Tensor], branch2: Optional[torch.Tensor],
+                out_dtype: torch.dtype, want_rows: bool = True) -> Optional[torch.Tensor]:
+    """``residual += branch + branch2`` (whichever are given; float32, in place), and the new stream in ``out_dtype``."""
+    _gpu("residual", residual, torch.float32, 2)
+    tokens, hidden = residual.shape
+    if branch is None:
+        branch, branch2 = branch2, None
+    for name, t in (("branch", branch), ("branch2", branch2)):
+        if t is not None:
+            _gpu(name, t, dims=2)
+            if not (t.shape == residual.shape and t.dtype in (torch.float32, out_dtype) and t.dtype == branch.dtype):
+                raise ValueError(f"{name} {tuple(t.shape)} {t.dtype} does not fit {tuple(residual.shape)} {out_dtype}")
+    rows = torch.empty((tokens, hidden), dtype=out_dtype, device=residual.device) if want_rows else None
+    if branch is None and rows is None:
+        return None
+    _run("cie_stream_rows", load_library().cie_stream_rows(
+        _stream(), _i(_code(branch.dtype if branch is not None else out_dtype)), _i(_code(out_dtype)), _ptr(residual),
+        _ptr(branch), _ptr(branch2), _ptr(rows), _i(tokens), _i(hidden)))
+    return rows
+
+
 def soft_cap_(x: torch.Tensor, cap: float) -> torch.Tensor:
     """``x <- cap * tanh(x / cap)`` in place on a float32 tensor."""
     _gpu("x", x, torch.float32)
@@ -1848,6 +1946,93 @@ def heads_prepare(proj: torch.Tensor, offsets: tuple[int, int, int], q_heads: in
     return q_out
 
 
+MAX_CONV_HEAD = 256        # numbers of a head that passes a convolution
+
+
+def heads_conv_prepare(proj: torch.Tensor, offsets: tuple[int, int, int], q_heads: int, kv_heads: int, dim: int, vdim: int,
+                       kernel_dim: int, kernel_vdim: int, taps_w: Optional[torch.Tensor], past: Optional[torch.Tensor],
+                       q_start_loc: torch.Tensor, sequences: int, single: bool, norm: Optional[str],
+                       q_weight: Optional[torch.Tensor], k_weight: Optional[torch.Tensor], eps: float,
+                       temperature: Optional[tuple[float, int]], positions: torch.Tensor, seq_of_token: torch.Tensor,
+                       seq_slot: torch.Tensor, block_table: torch.Tensor, k_pool: torch.Tensor, v_pool: torch.Tensor,
+                       rotary: Optional[tuple] = None, first_out: Optional[torch.Tensor] = None,
+                       first_in: Optional[torch.Tensor] = None, mix: float = 0.0) -> torch.Tensor:
+    """What :func:`heads_prepare` does (``norm``: ``None``, ``"unit"`` or ``"weight"``; one map a head; keys and values are
+    always written), for projections that first pass a causal convolution over each sequence's tokens, channel by
+    channel: ``taps_w`` [(q_heads + kv_heads) * dim + kv_heads * vdim, n] in ``proj``'s dtype, its last tap meeting the
+    token itself (``None``: no convolution).  ``past`` (float32 [slots, max(n - 1, 1), channels], oldest first) holds each
+    request's last inputs; they are moved on by the step's inputs.  ``single``: every sequence of the step brings one token.
+    The values may be mixed: ``first_out`` ([T, kv_heads * vdim]) takes them as convolved; with ``first_in`` (another
+    layer's) they become ``(1 - mix) * v + mix * first_in`` before they are cached."""
+    if not (proj.is_cuda and proj.dim() == 2 and proj.stride(1) == 1 and proj.dtype in _CODES):
+        raise ValueError("proj must be a float32 or bfloat16 GPU matrix with unit inner stride")
+    dtype, tokens = proj.dtype, proj.shape[0]
+    q_off, k_off, v_off = offsets
+    channels = (q_heads + kv_heads) * dim + kv_heads * vdim
+    if min(offsets) < 0 or proj.shape[1] < max(q_off + q_heads * dim, k_off + kv_heads * dim, v_off + kv_heads * vdim):
+        raise ValueError(f"proj {tuple(proj.shape)} does not hold heads at {offsets}")
+    if norm not in (None, "unit", "weight"):
+        raise ValueError(f"the norm over the heads must be None, 'unit' or 'weight', got {norm!r}")
+    if norm == "weight":
+        for name, w in (("q_weight", q_weight), ("k_weight", k_weight)):
+            if w is None:
+                raise ValueError(f"{name} is missing")
+            _gpu(name, w, torch.float32, 1)
+            if w.shape[0] != dim:
+                raise ValueError(f"{name} {tuple(w.shape)} does not fit heads of {dim}")
+    if not (dim <= kernel_dim <= MAX_CONV_HEAD and vdim <= kernel_vdim <= MAX_CONV_HEAD):
+        raise ValueError(f"heads of {dim} and {vdim} numbers in {kernel_dim} and {kernel_vdim}, at most {MAX_CONV_HEAD}")
+    page_size = _check_kv_pools(k_pool, v_pool, dtype, kv_heads, kernel_dim, kernel_vdim)
+    taps = 1
+    if taps_w is not None:
+        _gpu("taps_w", taps_w, dtype, 2)
+        taps = taps_w.shape[1]
+        if taps_w.shape[0] != channels or not 1 <= taps <= MAX_CONV_TAPS:
+            raise ValueError(f"taps {tuple(taps_w.shape)} for {channels} channels (up to {MAX_CONV_TAPS} taps)")
+    if taps > 1:
+        if past is None:
+            raise ValueError("a convolution of more than one tap needs the inputs of the tokens before the step")
+        _gpu("past", past, torch.float32, 3)
+        if tuple(past.shape[1:]) != (taps - 1, channels):
+            raise ValueError(f"past {tuple(past.shape)} must be [slots, {taps - 1}, {channels}]")
+        if offsets != (q_off, q_off + q_heads * dim, q_off + (q_heads + kv_heads) * dim):
+            raise ValueError("queries, keys and values of a convolution lie side by side")
+    _gpu("block_table", block_table, torch.int32, 2)
+    for name, meta, least in (("positions", positions, tokens), ("seq_of_token", seq_of_token, tokens),
+                              ("seq_slot", seq_slot, sequences), ("q_start_loc", q_start_loc, sequences + 1)):
+        _gpu(name, meta, torch.int32, 1)
+        if meta.shape[0] < least:
+            raise ValueError(f"{name} has {meta.shape[0]} entries, the step asks for {least}")
+    if single and sequences != tokens:
+        raise ValueError(f"{tokens} tokens of {sequences} sequences are not one each")
+    for name, t in (("first_out", first_out), ("first_in", first_in)):
+        if t is not None:
+            _gpu(name, t, dtype, 2)
+            if tuple(t.shape) != (tokens, kv_heads * vdim):
+                raise ValueError(f"{name} must be {(tokens, kv_heads * vdim)}, is {tuple(t.shape)}")
+    coef, every = temperature if temperature else (0.0, 0)
+    cos, sin, rot, neighbours = _check_rotary(rotary, dim)
+    q_out = torch.empty((tokens, q_heads * kernel_dim), dtype=dtype, device=proj.device)
+    _run("cie_heads_conv_prepare", load_library().cie_heads_conv_prepare(
+        _stream(), _i(_code(dtype)), _ptr(proj), _i(_ld(proj)), _i(q_off), _i(k_off), _i(v_off), _ptr(taps_w), _i(taps),
+        _ptr(past if taps > 1 else None), _ptr(q_start_loc), _i(1 if single else 0), _ptr(first_out), _ptr(first_in), _f(mix),
+        _ptr(q_weight), _ptr(k_weight), _i(NORM_MODES[norm]), _f(eps), _f(coef), _i(every), _ptr(positions), _ptr(seq_of_token),
+        _ptr(seq_slot), _ptr(block_table), _i(block_table.shape[1]), _ptr(q_out), _ptr(k_pool), _ptr(v_pool), _i(tokens),
+        _i(q_heads), _i(kv_heads), _i(dim), _i(vdim), _i(kernel_dim), _i(kernel_vdim), _i(page_size), _ptr(cos), _ptr(sin),
+        _i(rot), _i(1 if neighbours else 0)))
+    if taps > 1 and not single:
+        conv_keep(proj[:, q_off: q_off + channels], past, seq_slot, q_start_loc, sequences, taps)
+    return q_out
+
+
+def _attention_out(out: Optional[torch.Tensor], tokens: int, numbers: int, dtype: torch.dtype, device) -> torch.Tensor:
+    """Where attention writes its rows: a new matrix, or one of the caller's whose rows may lie apart."""
+    if out is None:
+        return torch.empty((tokens, numbers), dtype=dtype, device=device)
+    _row_view("out", out, (tokens, numbers), (dtype,))
+    return out
+
+
 def _check_score_shape(q_heads: int, slopes, sinks, softcap, window=None, chunk=None, keep_first=0) -> None:
     if chunk is not None and (chunk < 1 or window):
         raise ValueError(f"chunks hold at least one token and stand in a window's place, got chunk {chunk}, window {window}")
@@ -1890,7 +2075,8 @@ def scored_attention_generic(q: torch.Tensor, k_pool: torch.Tensor, v_pool: torc
                              softcap: Optional[float] = None, slopes: Optional[torch.Tensor] = None,
                              sinks: Optional[torch.Tensor] = None, gate: Optional[torch.Tensor] = None,
                              chunk: Optional[int] = None, keep_first: int = 0, gate_wide: bool = False,
-                             real_vdim: Optional[int] = None, differential: Optional[tuple] = None) -> torch.Tensor:
+                             real_vdim: Optional[int] = None, differential: Optional[tuple] = None,
+                             out: Optional[torch.Tensor] = None) -> torch.Tensor:
     """Attention of each token over its request's cached keys with shaped scores (see ``csrc/attention_scored.hip``;
     ``chunk``: a token sees the keys of its own chunk of that many positions, counted from position 0, up to itself;
     ``keep_first``: beside its window a token sees the first that many keys of its sequence):
@@ -1914,13 +2100,13 @@ def scored_attention_generic(q: torch.Tensor, k_pool: torch.Tensor, v_pool: torc
     _gpu("seq_slot", seq_slot, torch.int32, 1)
     _check_score_shape(q_heads, slopes, sinks, softcap, window, chunk, keep_first)
     gate_stride = _check_gate(gate, tokens, q_heads * real if gate_wide else q_heads, q.dtype)
-    out = torch.empty((tokens, q_heads * vdim), dtype=q.dtype, device=q.device)
+    out = _attention_out(out, tokens, q_heads * vdim, q.dtype, q.device)
     _run("cie_scored_attention_generic", load_library().cie_scored_attention_generic(
         _stream(), _i(_code(q.dtype)), _ptr(q), _ptr(k_pool), _ptr(v_pool), _ptr(block_table), _i(block_table.shape[1]),
         _ptr(positions), _ptr(seq_of_token), _ptr(seq_slot), _ptr(gate), _i(gate_stride), _ptr(out), _i(tokens),
         _i(q_heads), _i(kv_heads), _i(dim), _i(vdim), _i(page_size), _i(window or 0), _f(scale), _f(softcap or 0.0),
         _ptr(slopes), _ptr(sinks), _i(chunk or 0), _i(keep_first), _i(1 if gate_wide else 0), _i(real), _i(maps), _f(lam),
-        _f(factor), _f(eps)))
+        _f(factor), _f(eps), _ld(out)))
     return out
 
 
@@ -1933,7 +2119,7 @@ def scored_attention_mfma(q: torch.Tensor, k_pool: torch.Tensor, v_pool: torch.T
                           sinks: Optional[torch.Tensor] = None, gate: Optional[torch.Tensor] = None,
                           n_splits: int = 1, keys_per_split: int = 0, chunk: Optional[int] = None,
                           keep_first: int = 0, gate_wide: bool = False, real_vdim: Optional[int] = None,
-                          differential: Optional[tuple] = None) -> torch.Tensor:
+                          differential: Optional[tuple] = None, out: Optional[torch.Tensor] = None) -> torch.Tensor:
     """The same on the matrix cores (bfloat16, (dim, vdim) in ``SCORED_MFMA_DIMS`` or ``LATENT_MFMA_DIMS``, with two maps in
     ``DIFFERENTIAL_MFMA_DIMS``; pages of a power of two >= 4; two maps' rows fill ``row_tiles`` tiles together):
     tiles of ``tokens_per_tile`` consecutive tokens of one sequence (``tile_seq``, ``tile_q0`` int32 [n_tiles]; both
@@ -1971,7 +2157,7 @@ def scored_attention_mfma(q: torch.Tensor, k_pool: torch.Tensor, v_pool: torch.T
         raise ValueError(f"{n_tiles} tiles for {sequences} sequences")
     _check_score_shape(q_heads, slopes, sinks, softcap, window, chunk, keep_first)
     gate_stride = _check_gate(gate, tokens, q_heads * real if gate_wide else q_heads, q.dtype)
-    out = torch.empty((tokens, q_heads * vdim), dtype=q.dtype, device=q.device)
+    out = _attention_out(out, tokens, q_heads * vdim, q.dtype, q.device)
     part_o = part_ml = None
     if n_splits > 1:
         if keys_per_split < 128 or keys_per_split % 128:
@@ -1987,7 +2173,7 @@ def scored_attention_mfma(q: torch.Tensor, k_pool: torch.Tensor, v_pool: torch.T
         _i(gate_stride), _ptr(out), _i(q_heads), _i(kv_heads), _i(maps * dim), _i(vdim), _i(page_size), _i(tokens_per_tile),
         _i(row_tiles), _i(window or 0), _f(scale), _f(softcap or 0.0), _ptr(slopes), _ptr(sinks), _i(n_splits),
         _i(keys_per_split), _ptr(part_o), _ptr(part_ml), _i(chunk or 0), _i(keep_first), _i(1 if gate_wide else 0), _i(real),
-        _i(maps), _f(lam), _f(factor), _f(eps)))
+        _i(maps), _f(lam), _f(factor), _f(eps), _ld(out)))
     return out
 
 

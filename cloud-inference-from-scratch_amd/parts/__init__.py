@@ -1,5 +1,5 @@
 from . import (attention, block, delta_rule, entry, feed_forward, latent_attention, norm, parallel_mixers, position,  # noqa: F401
-               recurrent, routed_experts, scored_attention)  # (fill the registries)
+               recurrent, routed_experts, scored_attention, token_side)  # (fill the registries)
 from .base import (
     BLOCKS,
     FEED_FORWARDS,

@@ -21,6 +21,8 @@ Interfaces (``x`` is ``[tokens, hidden]`` in the engine's activation dtype,
                 unit of this call (``PagedView`` or ``StateView``), ``writes``
                 tells whether this call appends to it.
 ``FeedForward`` ``forward(x) -> y``
+``Side``        ``forward(residual, pending, batch, dtype, then=None) -> rows | None``: adds what is pending and then a
+                branch of its own to the stream in place; ``then``: a norm whose rows of the new stream come back.
 ``Entry``       ``joint(tokens) -> [tokens, 2 * hidden]`` and ``forward(joint, number) -> (residual, plus)``: remakes
                 the stream in front of a call of the run order from a row's two halves, the stream and the
                 embedding's rows; ``plus`` (float32) still joins the new stream.
@@ -44,6 +46,7 @@ MIXERS: dict[str, Callable[..., Any]] = {}
 FEED_FORWARDS: dict[str, Callable[..., Any]] = {}
 BLOCKS: dict[str, Callable[..., Any]] = {}
 ENTRIES: dict[str, Callable[..., Any]] = {}
+SIDES: dict[str, Callable[..., Any]] = {}
 
 _REGISTRIES = {
     "norm": NORMS,
@@ -52,11 +55,12 @@ _REGISTRIES = {
     "feed_forward": FEED_FORWARDS,
     "block": BLOCKS,
     "entry": ENTRIES,
+    "side": SIDES,
 }
 
 
 def register_part(role: str, kind: str, factory: Callable[..., Any]) -> None:
-    """``role`` is one of norm, position, mixer, feed_forward, block, entry."""
+    """``role`` is one of norm, position, mixer, feed_forward, block, entry, side."""
     _REGISTRIES[role][kind] = factory
 
 
@@ -79,6 +83,10 @@ class Part:
     # ``adds_to_residual``: ``forward`` takes ``residual=`` and may add its output there itself
     # (returning a ``RowSumsq`` or an ``Added``).
     adds_to_residual = False
+    # ``joins_products``: the part is one product in, something between, one product out.  Two such parts that read the
+    # same rows and whose results are added may share both products: ``product_in()`` and ``product_out()`` give the
+    # weights, and the part's own step between them takes the first product's rows and writes into a given matrix.
+    joins_products = False
 
     def expected_tensors(self, prefix: str) -> dict[str, TensorSpec]:
         return {}

@@ -14,6 +14,9 @@ cheaper form or rides along with the product behind it (``parts/linear.py``).
 ``SandwichNormBlock``: a norm in front of every sublayer and one on its output, which may then be scaled per channel:
 ``h += s1 * norm1_out(mixer(norm1(h))); h += s2 * norm2_out(feed_forward(norm2(h)))``.
 
+``ParallelBlock``: both sublayers read one norm of the stream, ``h += mixer(norm(h)) + feed_forward(norm(h))``, and a
+branch of the layer's own may follow.
+
 ``ParallelDepthBlock``: both branches read the same stream, and the next layer reads a weighted average of what
 the embedding and all layers so far left (below).
 """
@@ -29,7 +32,7 @@ from ..config.specs import LayerSpec
 from ..kernels import ops
 from ..weights.tensors import TensorSpec
 from .base import build_part, register_part
-from .linear import Added, RawRows, RowSumsq, StreamRows, WeightedPair
+from .linear import Added, RawRows, RowSumsq, StreamRows, WeightedPair, linear, linear_beside
 
 
 class PreNormBlock:
@@ -376,3 +379,107 @@ class SandwichNormBlock(PreNormBlock):
 
 
 register_part("block", "sandwich_norm", SandwichNormBlock)
+
+
+class ParallelBlock:
+    """``h += mixer(norm1(h)) + feed_forward(norm1(h))``: one norm, both sublayers read it.  Where both parts say
+    ``joins_products`` the layer runs two products in all: the mixer's first and the feed-forward's first as one (the
+    activation in its epilogue or right behind it), and, since the results are added, the mixer's last and the
+    feed-forward's last as one over their inputs side by side.  A ``side`` part (``LayerSpec.side``) adds a branch of its own
+    behind them.  What follows may have its first norm made by this block's last kernel (``follower``)."""
+
+    takes_follower = True
+
+    def __init__(self, spec: LayerSpec) -> None:
+        self.spec = spec
+        self.norm1 = build_part("norm", spec.norm1)
+        self.mixer = build_part("mixer", spec.mixer)
+        self.feed_forward = build_part("feed_forward", spec.feed_forward)
+        self.has_feed_forward = spec.feed_forward.kind != "none"
+        self.side = build_part("side", spec.side) if spec.side is not None else None
+        self.joined = self.has_feed_forward and self.mixer.joins_products and self.feed_forward.joins_products
+
+    def _parts(self):
+        parts = [("norm1", self.norm1), ("mixer", self.mixer)]
+        if self.has_feed_forward:
+            parts.append(("feed_forward", self.feed_forward))
+        if self.side is not None:
+            parts.append(("side", self.side))
+        return parts
+
+    def expected_tensors(self, prefix: str) -> dict[str, TensorSpec]:
+        out: dict[str, TensorSpec] = {}
+        for role, part in self._parts():
+            out.update(part.expected_tensors(f"{prefix}{self.spec.name_of(role)}."))
+        return out
+
+    def bind(self, tensors, prefix, dtype, device) -> None:
+        self.dtype = dtype
+        for role, part in self._parts():
+            part.bind(tensors, f"{prefix}{self.spec.name_of(role)}.", dtype, device)
+        if not self.joined:
+            return
+        first, up = self.mixer.product_in(), self.feed_forward.product_in()
+        last, down = self.mixer.product_out(), self.feed_forward.product_out()
+        # (the feed-forward's columns of the first result start at a multiple of 16 bytes; of the last product's input rows
+        # they are the first ones, whose number is a multiple of 8)
+        pad = first.new_zeros((-first.shape[0] % 8, first.shape[1]))
+        self.w_in = torch.cat([first, pad, up], dim=0).contiguous()
+        self.w_out = torch.cat([down, last], dim=1).contiguous()
+        self.inner = up.shape[0]
+        self.mixer.drop_products()
+        self.feed_forward.drop_products()
+
+    def cache_need(self):
+        return self.mixer.cache_need()
+
+    @property
+    def graph_safe(self) -> bool:
+        return all(getattr(part, "graph_safe", False) for _, part in self._parts())
+
+    def _between(self, rows: int, device) -> torch.Tensor:
+        """Rows for the last product's input: the feed-forward's, then the mixer's."""
+        k = self.w_out.shape[1]
+        return torch.empty((rows, -(-k // 8) * 8), dtype=self.dtype, device=device)[:, :k]
+
+    def warm_up(self, rows: int) -> None:
+        for _, part in self._parts():
+            warm = getattr(part, "warm_up", None)
+            if warm is not None:
+                warm(rows)
+        if self.joined:
+            between = self._between(rows, self.w_in.device).zero_()
+            linear_beside(torch.zeros((rows, self.w_in.shape[1]), dtype=self.dtype, device=self.w_in.device), self.w_in,
+                          between[:, : self.inner])
+            linear(between, self.w_out)
+
+    def forward(self, residual: torch.Tensor, pending, batch, view, writes: bool = True, plus: Optional[torch.Tensor] = None,
+                follower: Any = None, stream_rows: Optional[torch.Tensor] = None):
+        if stream_rows is not None:
+            raise ValueError("this arrangement does not leave the stream in the activation type: not built")
+        if isinstance(pending, NormedRows) and pending.owner is self and plus is None:
+            x = pending.first
+        elif plus is not None:
+            x = self.norm1.forward(residual, None if isinstance(pending, NormedRows) else pending, self.dtype, plus=plus)
+        else:
+            x = normalise(self.norm1, residual, None if isinstance(pending, NormedRows) else pending, self.dtype)
+        if self.joined:
+            between = self._between(x.shape[0], x.device)
+            proj = linear_beside(x, self.w_in, between[:, : self.inner])
+            self.mixer.mix(proj, batch, view, writes, out=between[:, self.inner:])
+            branch = linear(between, self.w_out, into=residual)
+        else:
+            branch = self.mixer.forward(x, batch, view, writes)
+            if self.has_feed_forward:
+                branch = WeightedPair(branch, self.feed_forward.forward(x))
+        if self.side is None:
+            return residual, branch
+        then = None
+        if isinstance(getattr(follower, "norm1", None), type(self.norm1)) and getattr(follower, "takes_follower", False) \
+                and hasattr(self.norm1, "joins_into") and self.norm1.joins_into(follower.norm1):
+            then = follower.norm1
+        rows = self.side.forward(residual, branch, batch, self.dtype, then)
+        return residual, None if then is None else NormedRows(rows, None, follower)
+
+
+register_part("block", "parallel", ParallelBlock)

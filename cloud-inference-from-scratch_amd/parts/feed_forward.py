@@ -90,6 +90,54 @@ class ClampedGatedMLP(Part):
         return linear(hidden, self.w_down)
 
 
+class DenseMLP(Part):
+    """``W_down act(W_up x)`` with ``act`` the square of relu (the one ``activation`` there is), no gate and no biases.  The
+    inner width is padded to a multiple of 8 with channels that stay zero."""
+
+    graph_safe = True
+    joins_products = True
+
+    def __init__(self, hidden_size: int, intermediate_size: int, activation: str = "squared_relu",
+                 names: tuple[str, str] = ("up", "down")) -> None:
+        if min(hidden_size, intermediate_size) < 1:
+            raise ValueError("sizes must be positive")
+        if activation != "squared_relu":
+            raise ValueError(f"this feed-forward runs squared_relu only, got {activation!r}")
+        self.hidden_size, self.intermediate_size = hidden_size, intermediate_size
+        self.width = -(-intermediate_size // 8) * 8
+        self.names = tuple(names)
+
+    def expected_tensors(self, prefix: str) -> dict[str, TensorSpec]:
+        up, down = self.names
+        return {prefix + up: TensorSpec((self.intermediate_size, self.hidden_size)),
+                prefix + down: TensorSpec((self.hidden_size, self.intermediate_size))}
+
+    def bind(self, tensors, prefix, dtype, device) -> None:
+        super().bind(tensors, prefix, dtype, device)
+        up, down = tensors[prefix + self.names[0]], tensors[prefix + self.names[1]]
+        more = self.width - self.intermediate_size
+        if more:
+            up = torch.cat([up, up.new_zeros((more, self.hidden_size))], dim=0)
+            down = torch.cat([down, down.new_zeros((self.hidden_size, more))], dim=1)
+        self.w_up, self.w_down = up.contiguous(), down.contiguous()
+
+    def product_in(self) -> torch.Tensor:
+        return self.w_up
+
+    def product_out(self) -> torch.Tensor:
+        return self.w_down
+
+    def drop_products(self) -> None:
+        self.w_up = self.w_down = None
+
+    def warm_up(self, rows: int) -> None:
+        if self.w_up is not None:
+            self.forward(torch.zeros((rows, self.hidden_size), dtype=self.w_down.dtype, device=self.w_down.device))
+
+    def forward(self, x, residual: Optional[torch.Tensor] = None):
+        return linear(ops.squared_relu(linear(x, self.w_up)), self.w_down)
+
+
 class NoFeedForward(Part):
     """A layer without a feed-forward: no tensors, and ``forward`` gives nothing to add."""
 
@@ -104,4 +152,5 @@ class NoFeedForward(Part):
 
 register_part("feed_forward", "gated_mlp", GatedMLP)
 register_part("feed_forward", "clamped_gated_mlp", ClampedGatedMLP)
+register_part("feed_forward", "dense_mlp", DenseMLP)
 register_part("feed_forward", "none", NoFeedForward)

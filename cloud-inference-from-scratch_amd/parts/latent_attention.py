@@ -117,6 +117,7 @@ class WindowedLatentAttention(Part):
     key.  ``q_rank=0`` reads the rank off the checkpoint."""
 
     graph_safe = True
+    joins_products = True
 
     def __init__(self, hidden_size: int, num_heads: int, head_dim: int, rot_dim: int, value_dim: int, kv_rank: int,
                  scale: float, eps: float, position: Optional[PartSpec] = None, q_rank: Optional[int] = None,
@@ -197,21 +198,34 @@ class WindowedLatentAttention(Part):
         self.sinks = tensors[prefix + "sink"].float().contiguous() if self.sink else None
 
     def warm_up(self, rows: int) -> None:
-        blank = lambda width: torch.zeros((rows, width), dtype=self.w_in.dtype, device=self.w_in.device)
-        linear(blank(self.hidden_size), self.w_in)
+        blank = lambda width: torch.zeros((rows, width), dtype=self.dtype, device=self.device)
         if self.w_uq is not None:
             linear(blank(self.q_latent), self.w_uq)
-        linear(blank(self.num_heads * self.value_dim), self.w_o)
+        if self.w_in is not None:
+            linear(blank(self.hidden_size), self.w_in)
+            linear(blank(self.num_heads * self.value_dim), self.w_o)
+
+    def product_in(self) -> torch.Tensor:
+        return self.w_in
+
+    def product_out(self) -> torch.Tensor:
+        return self.w_o
+
+    def drop_products(self) -> None:
+        self.w_in = self.w_o = None
 
     def forward(self, x: torch.Tensor, batch, view, writes: bool = True) -> torch.Tensor:
+        return linear(self.mix(linear(x, self.w_in), batch, view, writes), self.w_o)
+
+    def mix(self, proj: torch.Tensor, batch, view, writes: bool = True, out: Optional[torch.Tensor] = None) -> torch.Tensor:
+        """What lies between the layer's first product and its last; the heads' outputs go to ``out`` if it is given."""
         h, p, r, c = self.num_heads, self.head_dim, self.rot_dim, self.kv_rank
         rotary = None
         if self.position is not None and self.position.rotates:
             if batch.max_context > self.position.max_position:
                 raise ValueError(f"position {batch.max_context - 1} is beyond the rotary table of {self.position.max_position}")
-            cos, sin = self.position.tables(x.device, positions_bound(batch))
+            cos, sin = self.position.tables(proj.device, positions_bound(batch))
             rotary = (cos, sin, self.position.rotary_dim, getattr(self.position, "pairing", "halves") == "neighbours")
-        proj = linear(x, self.w_in)
         q_latent = ops.latent_down(proj, 0, self.q_latent, self.c_offset, self.dq_weight, self.dkv_weight, c, r, rotary,
                                    batch.positions, batch.seq_of_token, batch.seq_slot, view.block_table, view.k_pool,
                                    view.v_pool, self.eps, write_kv=writes)
@@ -221,7 +235,7 @@ class WindowedLatentAttention(Part):
         shape = dict(window=self.window, scale=self.scale, sinks=self.sinks)
         context = scored_attend(rows, batch, view, h, 1, self.entry_dim, self.latent_dim,
                                 ops.LATENT_MFMA_DIMS[self.mfma_dims] if self.mfma_dims else 0, shape)
-        return linear(ops.block_linear(context, self.w_unfold), self.w_o)
+        return ops.block_linear(context, self.w_unfold, out=out)
 
 
 register_part("mixer", "windowed_latent_attention", WindowedLatentAttention)

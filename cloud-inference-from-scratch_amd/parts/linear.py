@@ -196,6 +196,21 @@ class RawRows:
         return ops.add_rmsnorm(self.residual, None, self.norm.weight, self.norm.eps, self.dtype)
 
 
+def linear_beside(x: torch.Tensor, weight: torch.Tensor, act_out: torch.Tensor) -> torch.Tensor:
+    """One product for two readers of the same rows: ``x @ weight.T``, whose last columns (as many as ``act_out`` has) go
+    to ``act_out`` as the square of their relu (in the product's own epilogue where the hand-written form runs, in a
+    kernel behind it otherwise).  The columns in front of them come back (their rows may lie apart)."""
+    rows, k = x.shape
+    n = weight.shape[0]
+    split = n - act_out.shape[1]
+    if _fusable(rows, k, x.stride(0) if rows > 1 else k, weight) and (
+            rows <= FUSED_ROWS or (rows <= FUSED_SMALL_ROWS and n * k <= FUSED_SMALL_WEIGHT)):
+        return ops.gemm_fused(weight, ops.EPI_BF16, x, act_out=act_out)
+    out = linear(x, weight)
+    ops.squared_relu(out[:, split:], act_out)
+    return out[:, :split]
+
+
 _WIDENED: dict[int, tuple["weakref.ref", torch.Tensor]] = {}
 
 

@@ -15,7 +15,7 @@ from ..kernels import ops
 from ..weights.loader import torch_dtype
 from ..weights.tensors import TensorSpec
 from .base import BLOCKS, build_part
-from .block import normalise, whole_stream
+from .block import NormedRows, normalise, whole_stream
 from .linear import StreamRows, linear
 
 
@@ -33,6 +33,10 @@ def _expected(spec: ModelSpec, blocks: list[Any], final_norm: Any) -> dict[str, 
     out.update(final_norm.expected_tensors(spec.final_norm_name + "."))
     if not spec.tie_word_embeddings:
         out[spec.head_name] = TensorSpec((spec.vocab_size, spec.hidden_size))
+    if spec.embedding_norm is not None:
+        out.update(build_part("norm", spec.embedding_norm).expected_tensors(spec.embedding_norm_name + "."))
+    if spec.side_table_columns:
+        out[spec.side_table_name] = TensorSpec((spec.vocab_size, spec.side_table_columns))
     if spec.entry is not None:
         out.update(build_part("entry", spec.entry).expected_tensors(spec.entry_name + "."))
     for index, block in enumerate(blocks):
@@ -65,6 +69,11 @@ class DecoderModel:
                 raise ValueError(f"layer {call.layer} is run behind entry {call.entry}, and there are {self.entry.times}")
         if self.entry is not None and self.keeps_history:
             raise ValueError("an entry step remakes a stream that is averaged over the depth: not built")
+        self.embedding_norm = build_part("norm", spec.embedding_norm) if spec.embedding_norm is not None else None
+        if self.embedding_norm is not None and (self.entry is not None or self.keeps_history or self.keeps_embedding
+                                                or not hasattr(self.embedding_norm, "joins_into")):
+            raise ValueError("a norm on the embedding comes with a plain run order and is an RMS norm of one group")
+        self.side_table: torch.Tensor | None = None
         calls = [self.blocks[call.layer] for call in spec.order]
         # what runs behind each call, for blocks that make its first norm themselves; nothing where the stream is remade
         # or added to in between
@@ -133,6 +142,10 @@ class DecoderModel:
         self.folded_scale = hasattr(self.final_norm, "fold_scale")
         if self.folded_scale and self.spec.logit_scale != 1.0:
             self.final_norm.fold_scale(self.spec.logit_scale)
+        if self.embedding_norm is not None:
+            self.embedding_norm.bind(tensors, self.spec.embedding_norm_name + ".", self.dtype, device)
+        if self.spec.side_table_columns:
+            self.side_table = tensors[self.spec.side_table_name].contiguous()
         if self.entry is not None:
             self.entry.bind(tensors, self.spec.entry_name + ".", self.dtype, device)
         for index, block in enumerate(self.blocks):
@@ -175,10 +188,26 @@ class DecoderModel:
             # a first layer whose products read the stream itself: the embedding kernel also leaves it in their type
             rows = torch.empty((batch.token_ids.shape[0], self.embedding.shape[1]), dtype=self.embedding.dtype,
                                device=self.embedding.device)
-        residual = ops.embed(self.embedding, batch.token_ids, feed=batch.token_feed, pool=batch.token_pool,
-                             out=history[0] if history is not None else None, scale=self.spec.embedding_scale,
-                             rows=rows)
-        pending = StreamRows(rows) if rows is not None and joint is None else None
+        batch.carried.clear()
+        taken = None
+        if self.side_table is not None:
+            # (a row's token may come from the device's pool: whoever looks it up again takes it from here)
+            taken = batch.token_ids if batch.token_feed is None else torch.empty_like(batch.token_ids)
+            batch.carried.update(side_table=self.side_table, token_ids=taken)
+        given = dict(feed=batch.token_feed, pool=batch.token_pool, scale=self.spec.embedding_scale,
+                     ids_out=taken if batch.token_feed is not None else None)
+        if self.embedding_norm is not None:
+            then = None
+            if getattr(first, "takes_follower", False) and self.embedding_norm.joins_into(first.norm1):
+                then = first.norm1
+            residual, normed = ops.embed_normed(self.embedding, batch.token_ids, self.embedding_norm.weight_f32,
+                                                self.embedding_norm.eps,
+                                                next_weight=None if then is None else then.weight_f32, **given)
+            pending = None if then is None else NormedRows(normed, None, first)
+        else:
+            residual = ops.embed(self.embedding, batch.token_ids, out=history[0] if history is not None else None, rows=rows,
+                                 **given)
+            pending = StreamRows(rows) if rows is not None and joint is None else None
         embedded = residual.clone() if self.keeps_embedding else None
         left = False  # whether the stream lies in the joint rows already
         for index, call in enumerate(self.spec.order):

@@ -17,7 +17,10 @@ pairs for contexts beyond the ``original`` length the frequencies were made for:
 ``ramp_j = clamp((j - lo) / max(hi - lo, 0.001), 0, 1)``, pair j turns at
 ``inv_freq_j * (1 - ramp_j) + inv_freq_j / factor * ramp_j``, and cos and sin are both multiplied by
 ``0.1 ln(factor) + 1``.  ``scaling=(factor,)`` alone divides every frequency by the factor and leaves cos and sin as
-they are.  ``max_position=None`` is a model without a longest position: the tables then grow as
+they are.  ``bands=(factor, low, high, original)`` divides by wavelength: a pair that turns more than ``high`` times
+over the ``original`` length keeps its frequency, one that turns fewer than ``low`` times has it divided by the factor,
+and in between the frequency is the mean of the two, weighted by where its turns lie between ``low`` and ``high``.
+``max_position=None`` is a model without a longest position: the tables then grow as
 positions are asked for (``tables(device, upto)``), in powers of two.
 """
 
@@ -47,7 +50,7 @@ class RotaryHalf(Part):
     FIRST_ROWS = 4096     # the smallest table of a model without one
 
     def __init__(self, head_dim: int, theta: float, max_position: int | None, rotary_dim: int | None = None,
-                 scaling: tuple | None = None) -> None:
+                 scaling: tuple | None = None, bands: tuple | None = None) -> None:
         rotary_dim = head_dim if rotary_dim is None else rotary_dim
         if head_dim <= 0 or rotary_dim <= 0 or rotary_dim % 2 or rotary_dim > head_dim:
             raise ValueError(f"rotary_dim must be even, positive and at most the head size {head_dim}, got {rotary_dim}")
@@ -57,6 +60,11 @@ class RotaryHalf(Part):
             scaling = tuple(float(v) for v in scaling)
             if len(scaling) not in (1, 4) or not all(v > 0 for v in scaling) or (len(scaling) == 4 and theta == 1.0):
                 raise ValueError(f"scaling is (factor,) or (factor, original, fast, slow), all positive, got {scaling}")
+        if bands is not None:
+            bands = tuple(float(v) for v in bands)
+            if scaling is not None or len(bands) != 4 or not all(v > 0 for v in bands) or not bands[1] < bands[2]:
+                raise ValueError(f"bands are (factor, low, high, original), all positive, low < high, in scaling's place, got {bands}")
+        self.bands = bands
         self.head_dim = head_dim
         self.rotary_dim = rotary_dim
         self.theta = float(theta)
@@ -69,6 +77,11 @@ class RotaryHalf(Part):
         inv_freq = 1.0 / (
             self.theta ** (torch.arange(0, self.rotary_dim, 2, dtype=torch.float32) / self.rotary_dim)
         )
+        if self.bands is not None:
+            factor, low, high, original = self.bands
+            turns = original * inv_freq.double() / (2.0 * math.pi)
+            kept = ((turns - low) / (high - low)).clamp(0.0, 1.0)
+            return (kept * inv_freq.double() + (1.0 - kept) * inv_freq.double() / factor).float(), 1.0
         if self.scaling is None:
             return inv_freq, 1.0
         if len(self.scaling) == 1:
@@ -89,7 +102,7 @@ class RotaryHalf(Part):
         rows = self.max_position
         if self.grows:
             rows = max(self.FIRST_ROWS, 1 << max(0, (upto or 1) - 1).bit_length())
-        key = (self.rotary_dim, self.theta, self.scaling, self.grows, str(device))
+        key = (self.rotary_dim, self.theta, self.scaling, self.bands, self.grows, str(device))
         if not self.grows:
             key += (rows,)
         kept = _TABLES.get(key)

@@ -21,6 +21,11 @@ the position in other ways.  Every step is a parameter of the part and may be le
 * two maps a head (``differential = d``): queries and keys are projected as pairs of ``head_dim`` numbers, each map is a
   softmax of its own over the same values, and with ``lambda = exp(lq1 . lk1) - exp(lq2 . lk2) + d`` (learned vectors of
   ``head_dim`` numbers) a head's output is ``a1 - lambda a2``, divided by its root mean square, times ``1 - d``;
+* a causal convolution over the tokens of every channel of the projected queries, keys and values (``conv_taps``, in
+  front of the heads' norm), whose last inputs are a state of the request beside its pages;
+* values that are a mean of the layer's own and of those that an earlier layer of the same step made of the same token
+  (``value_mix``: ``"first"`` is that earlier layer, ``"mixed"`` one that mixes, by a learned weight; what is cached is the
+  mean);
 * key and value heads of different sizes;
 * no keys and values of its own (``own_kv=False``): the layer has no tensors for them and reads the cache unit that
   another layer of the same head sizes writes, with its own queries, mask and everything else.
@@ -40,7 +45,7 @@ from typing import Optional
 
 import torch
 
-from ..cache.manager import PagedKV
+from ..cache.manager import FixedState, PagedKV
 from ..config.specs import PartSpec
 from ..kernels import ops
 from ..weights.tensors import TensorSpec
@@ -65,7 +70,8 @@ class ScoredAttention(Part):
                  slope_base: Optional[float] = None, sink: bool = False, head_gate: bool = False,
                  chunk: Optional[int] = None, qkv_bias: bool = False, position: Optional[PartSpec] = None,
                  keep_first: int = 0, own_kv: bool = True, output_gate: bool = False,
-                 differential: Optional[float] = None) -> None:
+                 differential: Optional[float] = None, conv_taps: Optional[int] = None,
+                 value_mix: Optional[str] = None) -> None:
         for name, value in (("hidden_size", hidden_size), ("num_heads", num_heads), ("num_kv_heads", num_kv_heads),
                             ("head_dim", head_dim), ("value_dim", value_dim)):
             if isinstance(value, bool) or not isinstance(value, int) or value < 1:
@@ -107,6 +113,14 @@ class ScoredAttention(Part):
             raise ValueError("one gate: a number a head or a number for every number of it")
         if self.maps == 2 and (self.sink or qk_norm is not None or not self.own_kv):
             raise ValueError("two maps a head come with neither a sink nor a norm on the heads, and with keys of their own")
+        if conv_taps is not None and (isinstance(conv_taps, bool) or not isinstance(conv_taps, int)
+                                      or not 1 <= conv_taps <= ops.MAX_CONV_TAPS):
+            raise ValueError(f"a convolution of 1 to {ops.MAX_CONV_TAPS} taps, got {conv_taps!r}")
+        if value_mix not in (None, "first", "mixed"):
+            raise ValueError(f"value_mix is 'first' or 'mixed' or None, got {value_mix!r}")
+        self.conv_taps, self.value_mix = conv_taps, value_mix
+        if self.by_channel and (self.maps == 2 or qk_norm == "whole" or not self.own_kv):
+            raise ValueError("a convolution and mixed values come with one map a head, a norm of single heads and keys of their own")
         self.position = build_part("position", position) if position is not None else None
         if self.position is not None and self.position.rotates and self.position.rotary_dim > head_dim:
             raise ValueError(f"{self.position.rotary_dim} turning numbers in heads of {head_dim}")
@@ -121,12 +135,28 @@ class ScoredAttention(Part):
             self.most_row_tiles = 4
         self.kernel_dim, self.kernel_vdim = self.mfma_dims or (_round8(head_dim), _round8(value_dim))
 
-    def cache_need(self) -> PagedKV:
+    @property
+    def by_channel(self) -> bool:
+        """Whether the projections pass the kernel that convolves them and mixes values."""
+        return self.conv_taps is not None or self.value_mix is not None
+
+    @property
+    def joins_products(self) -> bool:
+        return not self.qkv_bias
+
+    @property
+    def channels(self) -> int:
+        return (self.num_heads + self.num_kv_heads) * self.head_dim + self.num_kv_heads * self.value_dim
+
+    def cache_need(self):
         # (a chunk's keys all lie inside a window of the chunk's length: pages behind it go back to the pool)
         width = self.maps * self.kernel_dim
-        return PagedKV(self.num_kv_heads, width, self.window if self.chunk is None else self.chunk,
-                       value_dim=self.kernel_vdim if self.kernel_vdim != width else None,
-                       keep_first=self.keep_first)
+        pages = PagedKV(self.num_kv_heads, width, self.window if self.chunk is None else self.chunk,
+                        value_dim=self.kernel_vdim if self.kernel_vdim != width else None,
+                        keep_first=self.keep_first)
+        if self.conv_taps is None or self.conv_taps == 1:
+            return pages
+        return (pages, FixedState((self.conv_taps - 1, self.channels)))
 
     def expected_tensors(self, prefix: str) -> dict[str, TensorSpec]:
         h, g, d, v, width = self.num_heads, self.num_kv_heads, self.head_dim, self.value_dim, self.hidden_size
@@ -145,6 +175,11 @@ class ScoredAttention(Part):
             out[prefix + "q.norm"] = TensorSpec((h * d if whole else d,), init="norm", keeps_float32=True)
             if self.own_kv:
                 out[prefix + "k.norm"] = TensorSpec((g * d if whole else d,), init="norm", keeps_float32=True)
+        if self.conv_taps is not None:
+            for name, rows in (("q", h * d), ("k", g * d), ("v", g * v)):
+                out[f"{prefix}{name}.conv"] = TensorSpec((rows, self.conv_taps))
+        if self.value_mix is not None:  # (the first of the layers has nothing to mix with: its weight is not read)
+            out[prefix + "vmix"] = TensorSpec((), keeps_float32=True, optional=self.value_mix == "first")
         if self.sink:
             out[prefix + "sink"] = TensorSpec((h,), keeps_float32=True)
         if self.head_gate or self.output_gate:
@@ -186,6 +221,11 @@ class ScoredAttention(Part):
             self.q_weight = tensors[prefix + "q.norm"].float().contiguous()
             if self.own_kv:
                 self.k_weight = tensors[prefix + "k.norm"].float().contiguous()
+        self.taps_w, self.mix_weight = None, 0.0
+        if self.conv_taps is not None:
+            self.taps_w = torch.cat([tensors[f"{prefix}{name}.conv"] for name in ("q", "k", "v")], dim=0).contiguous()
+        if self.value_mix == "mixed":
+            self.mix_weight = float(tensors[prefix + "vmix"].float().item())
         self.pair = None  # what joins the two maps of a head: lambda, the factor behind the norm, its eps
         if self.maps == 2:
             dot = lambda n: float((tensors[f"{prefix}lq{n}"].float() * tensors[f"{prefix}lk{n}"].float()).sum())
@@ -203,33 +243,69 @@ class ScoredAttention(Part):
         self.w_o = w_o.contiguous()
 
     def warm_up(self, rows: int) -> None:
+        if self.w_in is None:
+            return
         blank = lambda width: torch.zeros((rows, width), dtype=self.w_in.dtype, device=self.w_in.device)
         linear(blank(self.hidden_size), self.w_in, self.b_in)
         linear(blank(self.num_heads * self.kernel_vdim), self.w_o)
 
+    def product_in(self) -> torch.Tensor:
+        return self.w_in
+
+    def product_out(self) -> torch.Tensor:
+        return self.w_o
+
+    def drop_products(self) -> None:
+        self.w_in = self.w_o = None
+
     def forward(self, x: torch.Tensor, batch, view, writes: bool = True) -> torch.Tensor:
+        return linear(self.mix(linear(x, self.w_in, self.b_in), batch, view, writes), self.w_o)
+
+    def mix(self, proj: torch.Tensor, batch, view, writes: bool = True, out: Optional[torch.Tensor] = None) -> torch.Tensor:
+        """What lies between the layer's first product and its last; the heads' outputs go to ``out`` if it is given."""
         if writes and not self.own_kv:
             raise ValueError("a layer without keys and values of its own reads the cache unit that another layer writes")
-        proj = linear(x, self.w_in, self.b_in)
         rotary = None
         if self.position is not None and self.position.rotates:
             if batch.max_context > self.position.max_position:
                 raise ValueError(f"position {batch.max_context - 1} is beyond the rotary table of {self.position.max_position}")
-            cos, sin = self.position.tables(x.device, positions_bound(batch))
+            cos, sin = self.position.tables(proj.device, positions_bound(batch))
             rotary = (cos, sin, self.position.rotary_dim, getattr(self.position, "pairing", "halves") == "neighbours")
+        gate = proj[:, self.gate_offset:] if self.gate_offset is not None else None
+        if self.by_channel:
+            q, view = self._convolve(proj, batch, view, writes, rotary)
+            return self.attend(q, gate, batch, view, out)
         q = ops.heads_prepare(proj, self.offsets, self.num_heads, self.num_kv_heads, self.head_dim, self.value_dim,
                               self.kernel_dim, self.kernel_vdim, self.qk_norm, self.q_weight, self.k_weight, self.eps,
                               self.q_temperature, batch.positions, batch.seq_of_token, batch.seq_slot,
                               view.block_table, view.k_pool, view.v_pool, batch.tokens, write_kv=writes, rotary=rotary,
                               maps=self.maps)
-        gate = proj[:, self.gate_offset:] if self.gate_offset is not None else None
-        context = self.attend(q, gate, batch, view)
-        return linear(context, self.w_o)
+        return self.attend(q, gate, batch, view, out)
 
-    def attend(self, q: torch.Tensor, gate, batch, view) -> torch.Tensor:
+    def _convolve(self, proj: torch.Tensor, batch, view, writes: bool, rotary: Optional[tuple]):
+        if not writes:
+            raise ValueError("a layer whose projections are convolved moves its state on whenever it runs")
+        pages, past = (view[0], view[1].state) if isinstance(view, (tuple, list)) else (view, None)
+        first_out = first_in = None
+        if self.value_mix == "first":
+            first_out = torch.empty((batch.tokens, self.num_kv_heads * self.value_dim), dtype=proj.dtype, device=proj.device)
+            batch.carried["first_values"] = first_out
+        elif self.value_mix == "mixed":
+            first_in = batch.carried.get("first_values")
+            if first_in is None:
+                raise ValueError("a layer mixes its values with an earlier layer's, and none has left any")
+        q = ops.heads_conv_prepare(proj, self.offsets, self.num_heads, self.num_kv_heads, self.head_dim, self.value_dim,
+                                   self.kernel_dim, self.kernel_vdim, self.taps_w, past, batch.q_start_loc, batch.sequences,
+                                   batch.max_q_len <= 1, self.qk_norm, self.q_weight, self.k_weight, self.eps,
+                                   self.q_temperature, batch.positions, batch.seq_of_token, batch.seq_slot, pages.block_table,
+                                   pages.k_pool, pages.v_pool, rotary=rotary, first_out=first_out, first_in=first_in,
+                                   mix=self.mix_weight)
+        return q, pages
+
+    def attend(self, q: torch.Tensor, gate, batch, view, out: Optional[torch.Tensor] = None) -> torch.Tensor:
         shape = dict(window=self.window, scale=self.scale, softcap=self.softcap, slopes=self.slopes,
                      sinks=self.sinks, gate=gate, chunk=self.chunk, keep_first=self.keep_first, gate_wide=self.output_gate,
-                     real_vdim=self.value_dim, differential=self.pair)
+                     real_vdim=self.value_dim, differential=self.pair, out=out)
         return scored_attend(q, batch, view, self.num_heads, self.num_kv_heads, self.kernel_dim, self.kernel_vdim,
                              self.most_row_tiles if self.mfma_dims else 0, shape)
 
