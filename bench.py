@@ -5,7 +5,7 @@
     python bench.py [--gpus 1] [--steps K] [--warmup W] [--batch 8] [--context 4096]
                     [--shape 0.5b|3b|7b|14b|32b|72b] [--layers N] [--long-contexts 32768]
                     [--mixed-portions 16,64,248] [--other-shapes 7b,14b]
-    python bench.py --design polosun|givizen|nokipel|senuvik|nopunex [--design-shapes 3b,7b] [--design-layers 12]
+    python bench.py --design polosun|givizen|nokipel|senuvik|nopunex|nogapel [--design-shapes 3b,7b] [--design-layers 12]
 
 A "step" is one decode step of the whole engine (scheduler iteration: plan,
 step function, sampling, token hand-over).  Protocol after the reference's
@@ -55,7 +55,14 @@ delta rule, latent attention under a window and differential attention in
 chunks in turn, each with a dense feed-forward) beside the Polosun model of
 equal width, memory and latent sizes, feed-forward, vocabulary and layer count,
 the closest of the engine's models: a memory of outer products, latent
-attention, dense feed-forwards.
+attention, dense feed-forwards.  ``--design nogapel`` measures the Nogapel
+design (window attention behind short convolutions, twice, and latent attention
+over all earlier tokens in turn, each beside an ungated feed-forward and with a
+branch from a token table) beside the Nopunex model of equal width, head and
+latent sizes, vocabulary and layer count, the closest of the engine's models:
+latent attention with a sink and a query latent, short convolutions, dense
+feed-forwards (Nogapel's inner width is half as large again, so that its two
+matrices hold as many weights as Nopunex's three).
 """
 
 from __future__ import annotations
@@ -587,11 +594,66 @@ def nopunex_costs(config, batch: int, context: float, tokens: int, elem: int) ->
     return moved, 2.0 * tokens * (weights - head) + 2.0 * head + other
 
 
+NOGAPEL_SIDE = 256
+
+
+def nogapel_raw(shape: dict, layers: int) -> dict:
+    """A Nogapel configuration with the width and vocabulary of a Qwen2.5 shape and layers of realistic proportions: two
+    layers of window attention (the shape's heads, windows of 1,024 tokens, convolutions of 4 taps, frequencies divided by
+    wavelength, mixed values) to one of latent attention (Nopunex's heads of 128 + 32, its latents of 96 and of a quarter of
+    the width, over all earlier tokens), each beside a feed-forward whose two matrices hold as many weights as the shape's
+    three, and with 256 columns of the token table."""
+    width = shape["hidden_size"]
+    heads, kv_heads = shape["num_attention_heads"], shape["num_key_value_heads"]
+    dim = width // heads
+    mlp = {"kind": "dense", "ff": shape["intermediate_size"] * 3 // 2}
+    attention = {"type": "attention", "mlp": mlp,
+                 "mixer": {"heads": heads, "kv_heads": kv_heads, "dim": dim, "vdim": dim, "conv": 4, "scale": dim ** -0.5,
+                           "v_mix": True, "mask": {"size": NOPUNEX_REACH},
+                           "rot": {"base": 500000.0, "dims": dim,
+                                   "scaling": {"factor": 8.0, "low": 1.0, "high": 4.0, "original": 8192}}}}
+    latent = {"type": "latent_attention", "mlp": mlp,
+              "mixer": {"heads": width // 128, "dim": 128, "rot_dim": 32, "vdim": 128, "q_rank": width // 4, "kv_rank": 96,
+                        "scale": 160 ** -0.5, "rot": {"base": 1000000.0, "dims": 32}}}
+    return {"architecture": "Nogapel", "vocab": shape["vocab_size"], "width": width, "norm": {"eps": 1e-6},
+            "token_side": {"dim": NOGAPEL_SIDE}, "layers": [latent if i % 3 == 2 else attention for i in range(layers)]}
+
+
+def nogapel_costs(config, batch: int, context: float, tokens: int, elem: int) -> tuple[float, float]:
+    """(bytes one decode step has to move, flops of a prefill of ``tokens`` tokens) for a Nogapel configuration: every
+    weight once (the two tables are only looked up), each request's keys and values inside the window or its latents;
+    products at two flops per weight and token, attention over the keys each token sees, for a latent in the latent's own
+    space."""
+    from cie_amd.parts.model import expected_tensors
+
+    expected = expected_tensors(config.model_spec())
+    weights = sum(int(__import__("math").prod(spec.shape)) for name, spec in expected.items()
+                  if name not in ("embed", "side.embed") and not spec.optional)
+    head = config.vocab_size * config.hidden_size
+    moved, other = float(weights * elem), 0.0
+    for layer in config.raw["layers"]:
+        m = layer["mixer"]
+        size = m["mask"]["size"] if m.get("mask") else None
+        reach = tokens if size is None else min(tokens, size)
+        pairs = reach * (reach + 1) / 2 + (tokens - reach) * reach
+        seen = context if size is None else min(context, size)
+        if layer["type"] == "latent_attention":
+            entry = m["kv_rank"] + m["rot_dim"]
+            moved += batch * seen * (entry + m["kv_rank"]) * elem
+            other += 2.0 * pairs * m["heads"] * (entry + m["kv_rank"])
+        else:
+            moved += batch * seen * m["kv_heads"] * (m["dim"] + m["vdim"]) * elem
+            moved += batch * 2 * (m["conv"] - 1) * ((m["heads"] + m["kv_heads"]) * m["dim"] + m["kv_heads"] * m["vdim"]) * 4
+            other += 2.0 * pairs * m["heads"] * (m["dim"] + m["vdim"])
+    return moved, 2.0 * tokens * (weights - head) + 2.0 * head + other
+
+
 def compare_designs(args) -> int:
-    """``--design polosun``, ``givizen``, ``nokipel``, ``senuvik`` or ``nopunex``: see the module's text."""
+    """``--design polosun``, ``givizen``, ``nokipel``, ``senuvik``, ``nopunex`` or ``nogapel``: see the module's text."""
     import torch
 
-    from cie_amd.config import GivizenConfig, NokipelConfig, NopunexConfig, PolosunConfig, Qwen2Config, SenuvikConfig
+    from cie_amd.config import (GivizenConfig, NogapelConfig, NokipelConfig, NopunexConfig, PolosunConfig, Qwen2Config,
+                                SenuvikConfig)
     from cie_amd.workloads import SHAPES
 
     elem = 2 if args.dtype == "bf16" else 4
@@ -608,6 +670,9 @@ def compare_designs(args) -> int:
         elif args.design == "nopunex":
             designs = {"nopunex": NopunexConfig.from_hf_config(nopunex_raw(shape, layers)),
                        "polosun": PolosunConfig.from_hf_config(polosun_raw(shape, layers))}
+        elif args.design == "nogapel":
+            designs = {"nogapel": NogapelConfig.from_hf_config(nogapel_raw(shape, layers)),
+                       "nopunex": NopunexConfig.from_hf_config(nopunex_raw(shape, layers))}
         else:
             designs = {
                 args.design: (PolosunConfig.from_hf_config(polosun_raw(shape, layers)) if args.design == "polosun"
@@ -627,6 +692,8 @@ def compare_designs(args) -> int:
                     return senuvik_costs(config, batch, context, args.prefill_tokens, elem)
                 if design == "nopunex":
                     return nopunex_costs(config, batch, context, args.prefill_tokens, elem)
+                if design == "nogapel":
+                    return nogapel_costs(config, batch, context, args.prefill_tokens, elem)
                 return (decode_bytes(config, layers, batch, context, elem), prefill_flops(config, layers, args.prefill_tokens))
 
             record = {}
@@ -662,8 +729,12 @@ def compare_designs(args) -> int:
     nopunex_layers = (f"gated delta rule, latent attention (window {NOPUNEX_REACH}), differential attention (chunks of "
                       f"{NOPUNEX_REACH}) in turn, each with a dense feed-forward, in one pass behind a joining product; beside "
                       f"it Polosun: retention, latent_attention, rglru in turn, each with a dense feed-forward")
+    nogapel_layers = (f"window attention behind convolutions (window {NOPUNEX_REACH}) twice, latent attention over all tokens, in "
+                      f"turn, each beside an ungated feed-forward of one and a half times the width and with {NOGAPEL_SIDE} columns "
+                      f"of a token table")
     beside = ("the Givizen model of equal width, head and expert sizes" if args.design == "nokipel"
               else "the Nokipel model of equal width, head and expert sizes" if args.design == "senuvik"
+              else "the Nopunex model of equal width, head and latent sizes, feed-forward weights" if args.design == "nogapel"
               else "the Polosun model of equal width, memory and latent sizes, feed-forward" if args.design == "nopunex"
               else "the Qwen2.5 decoder of equal width, feed-forward")
     print(json.dumps({
@@ -674,6 +745,8 @@ def compare_designs(args) -> int:
                    "design_layers": ("retention, latent_attention, rglru in turn, each with a dense feed-forward"
                                      if args.design == "polosun" else givizen_layers if args.design == "givizen" else
                                      nopunex_layers if args.design == "nopunex" else
+                                     nogapel_layers + "; beside it Nopunex: " + nopunex_layers.split("; beside")[0]
+                                     if args.design == "nogapel" else
                                      senuvik_layers + "; beside it Nokipel: " + nokipel_layers if args.design == "senuvik" else
                                      nokipel_layers + "; beside it Givizen: " + givizen_layers)},
         "shapes": out,
@@ -702,9 +775,9 @@ def main(argv=None) -> int:
                              "(default 16,64,248; '' for none, as with --no-points)")
     parser.add_argument("--other-shapes", default="7b,14b",
                         help="further shapes whose decode at the main batch and context and whose prefill go into the points ('' for none)")
-    parser.add_argument("--design", default=None, choices=["polosun", "givizen", "nokipel", "senuvik", "nopunex"],
+    parser.add_argument("--design", default=None, choices=["polosun", "givizen", "nokipel", "senuvik", "nopunex", "nogapel"],
                         help="instead of the default record: this design beside the Qwen2.5 decoder of equal size "
-                             "(nokipel: beside the Givizen model of equal size; senuvik: beside the Nokipel model; nopunex: beside the Polosun model)")
+                             "(nokipel: beside the Givizen model of equal size; senuvik: beside the Nokipel model; nopunex: beside the Polosun model; nogapel: beside the Nopunex model)")
     parser.add_argument("--design-shapes", default="3b,7b", help="the Qwen2.5 shapes whose sizes the comparison takes")
     parser.add_argument("--design-layers", type=int, default=12, help="layers of both models in the comparison")
     args = parser.parse_args(argv)
