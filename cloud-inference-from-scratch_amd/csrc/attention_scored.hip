@@ -199,9 +199,12 @@ __device__ __forceinline__ float2 load_pair(const bf16_t* p, int d, int n, bool 
 __device__ __forceinline__ void store_pair(float* p, float2 v) { *reinterpret_cast<float2*>(p) = v; }
 __device__ __forceinline__ void store_pair(bf16_t* p, float2 v) { *reinterpret_cast<uint32_t*>(p) = pack_bf16(v.x, v.y); }
 
-// One wave per (token, head slot) as above; a lane holds neighbours 2l, 2l + 1 (and those 128 further on).  TAPS: the
-// convolution's taps where the kernel knows them (their loads then travel together), 0: c.n of them.
-template <typename T, int TAPS>
+// One wave per (run of RUN tokens of the step, head slot); slots as above.  A lane holds neighbours 2l, 2l + 1 of the head
+// (CHUNKS = 2: and those 128 further on) for all of the run's tokens: a projected row is read once for all taps, the taps and
+// what a token's place leads to (sequence, slot, page) once a run, and eight values of a channel are stored together where
+// they lie side by side in the transposed pool.  TAPS: the convolution's taps where the kernel knows them, 0 (runs of one
+// token only): c.n of them.
+template <typename T, int TAPS, int RUN, int CHUNKS>
 __global__ void __launch_bounds__(256)
 heads_conv_prepare_kernel(const T* __restrict__ proj, int proj_stride, int q_off, int k_off, int v_off, ConvHeads<T> c,
                           const float* __restrict__ q_weight, const float* __restrict__ k_weight, int norm_mode, float eps,
@@ -211,14 +214,18 @@ heads_conv_prepare_kernel(const T* __restrict__ proj, int proj_stride, int q_off
                           T* __restrict__ k_pool, T* __restrict__ v_pool, int tokens, int q_heads, int kv_heads, int dim,
                           int vdim, int D, int DV, int page_shift, const float* __restrict__ cos_table,
                           const float* __restrict__ sin_table, int rot, int neighbours) {
-    __shared__ float staged[4][256];  // a head of each wave, for partners that another lane holds
+    static_assert(TAPS > 0 || RUN == 1, "runs of several tokens know their taps");
+    constexpr int kTaps = TAPS > 0 ? TAPS : kMaxConvTaps;
+    constexpr int kRows = RUN + kTaps - 1;
+    __shared__ float staged[4][128 * CHUNKS];  // a head of each wave, for partners that another lane holds
     const int lane = threadIdx.x % kWave;
     const int wave = threadIdx.x / kWave;
     const int slots = q_heads + 2 * kv_heads;
     const long unit = static_cast<long>(blockIdx.x) * 4 + wave;
-    if (unit >= static_cast<long>(tokens) * slots) return;
-    const int token = static_cast<int>(unit / slots);
-    const int slot = static_cast<int>(unit - static_cast<long>(token) * slots);
+    if (unit >= static_cast<long>((tokens + RUN - 1) / RUN) * slots) return;
+    const int token0 = static_cast<int>(unit / slots) * RUN;
+    const int slot = static_cast<int>(unit - static_cast<long>(token0 / RUN) * slots);
+    const int count = min(RUN, tokens - token0);
     const bool is_q = slot < q_heads, is_v = slot >= q_heads + kv_heads;
     const int head = is_q ? slot : is_v ? slot - q_heads - kv_heads : slot - q_heads;
     const int n = is_v ? vdim : dim;
@@ -226,124 +233,177 @@ heads_conv_prepare_kernel(const T* __restrict__ proj, int proj_stride, int q_off
     const int column = (is_q ? q_off : is_v ? v_off : k_off) + head * n;
     const int channels = (q_heads + kv_heads) * dim + kv_heads * vdim;
     const int channel = is_v ? (q_heads + kv_heads) * dim + head * vdim : (is_q ? 0 : q_heads * dim) + head * dim;
-    const int pos = positions[token];
-    const int seq = seq_of_token[token];
-    const int slot_row = seq_slot[seq];
     const int taps = TAPS > 0 ? TAPS : c.n;
-    const int first = c.q_start_loc[seq];
-    const int t = token - first;  // the token's place in the step's portion of its sequence
-    float* before = c.past + static_cast<size_t>(slot_row) * max(taps - 1, 1) * channels + channel;
     const bool paired = (((proj_stride | column | n) & 1) == 0);  // (the base of `proj` is aligned to a pair)
-    const T* src = proj + static_cast<size_t>(first) * proj_stride + column;
+    // lane i knows the place of the run's token i
+    const int mine = token0 + min(lane, count - 1);
+    const int my_pos = positions[mine];
+    const int my_seq = seq_of_token[mine];
+    const int my_slot = seq_slot[my_seq];
+    const int my_first = c.q_start_loc[my_seq];
+    const int my_page = is_q ? 0 : block_table[static_cast<size_t>(my_slot) * table_width + (my_pos >> page_shift)];
+    auto of = [&](int value, int tt) { return __builtin_amdgcn_readlane(value, tt); };
 
-    float2 y[2];
-    float sum_sq = 0.f;
+    float2 y[RUN][CHUNKS];
+    float sum_sq[RUN];
 #pragma unroll
-    for (int i = 0; i < 2; ++i) {
+    for (int tt = 0; tt < RUN; ++tt) sum_sq[tt] = 0.f;
+#pragma unroll
+    for (int i = 0; i < CHUNKS; ++i) {
         const int d = 2 * lane + 128 * i;
-        y[i] = float2{0.f, 0.f};
+#pragma unroll
+        for (int tt = 0; tt < RUN; ++tt) y[tt][i] = float2{0.f, 0.f};
         if (d >= n) continue;
         const bool two = d + 1 < n;
-        if (!c.taps) {
-            y[i] = load_pair(src + static_cast<size_t>(t) * proj_stride, d, n, paired);
-        } else {
-            const T* w = c.taps + static_cast<size_t>(channel + d) * taps;
-            float2 in[TAPS > 0 ? TAPS : kMaxConvTaps];
+        float2 u[kRows];  // the projected rows token0 - (taps - 1) and on (a place in front of the step's first row: not used)
+        float2 w[kTaps];
 #pragma unroll
-            for (int j = 0; j < (TAPS > 0 ? TAPS : kMaxConvTaps); ++j) {
-                if (TAPS == 0 && j >= taps) break;
-                const int from = t - (taps - 1) + j;
-                if (from >= 0) {
-                    in[j] = load_pair(src + static_cast<size_t>(from) * proj_stride, d, n, paired);
-                } else {
-                    const float* old = before + static_cast<size_t>(taps - 1 + from) * channels + d;
-                    in[j] = float2{old[0], two ? old[1] : 0.f};
-                }
-            }
-#pragma unroll
-            for (int j = 0; j < (TAPS > 0 ? TAPS : kMaxConvTaps); ++j) {
-                if (TAPS == 0 && j >= taps) break;
-                y[i].x = fmaf(to_float(w[j]), in[j].x, y[i].x);
-                if (two) y[i].y = fmaf(to_float(w[taps + j]), in[j].y, y[i].y);
-            }
-            if (c.single) {  // (t = 0: in[j] is what the state held at j, and the last is the token's own)
-#pragma unroll
-                for (int j = 1; j < (TAPS > 0 ? TAPS : kMaxConvTaps); ++j) {
-                    if (TAPS == 0 && j >= taps) break;
-                    float* now = before + static_cast<size_t>(j - 1) * channels + d;
-                    now[0] = in[j].x;
-                    if (two) now[1] = in[j].y;
-                }
-            }
+        for (int r = 0; r < kRows; ++r) {
+            if (TAPS == 0 && r >= taps) break;
+            const int row = min(max(token0 - (taps - 1) + r, 0), tokens - 1);
+            u[r] = load_pair(proj + static_cast<size_t>(row) * proj_stride + column, d, n, paired);
         }
-        sum_sq += y[i].x * y[i].x + y[i].y * y[i].y;
-    }
-    const size_t page = is_q ? 0 : static_cast<size_t>(block_table[static_cast<size_t>(slot_row) * table_width + (pos >> page_shift)]);
-    const int in_page = pos & ((1 << page_shift) - 1);
-    if (is_v) {
-        T* dst = v_pool + ((page * kv_heads + head) * DV << page_shift) + in_page;
-        const size_t at = (static_cast<size_t>(token) * kv_heads + head) * vdim;
 #pragma unroll
-        for (int i = 0; i < 2; ++i) {
+        for (int j = 0; j < kTaps; ++j) {
+            if (TAPS == 0 && j >= taps) break;
+            const T* at = c.taps + static_cast<size_t>(channel + d) * taps + j;
+            w[j] = c.taps ? float2{to_float(at[0]), two ? to_float(at[taps]) : 0.f} : float2{1.f, 1.f};
+        }
+#pragma unroll
+        for (int tt = 0; tt < RUN; ++tt) {
+            if (tt >= count) break;
+            const int t = token0 + tt - of(my_first, tt);  // the token's place in the step's portion of its sequence
+            float* before = c.past + static_cast<size_t>(of(my_slot, tt)) * max(taps - 1, 1) * channels + channel + d;
+#pragma unroll
+            for (int j = 0; j < kTaps; ++j) {
+                if (TAPS == 0 && j >= taps) break;
+                float2 in = u[tt + j];
+                if (t - (taps - 1) + j < 0) {  // (in front of the portion: what earlier steps left)
+                    const float* old = before + static_cast<size_t>(t + j) * channels;
+                    in = float2{old[0], two ? old[1] : 0.f};
+                    if (RUN == 1) u[j] = in;
+                }
+                y[tt][i].x = fmaf(w[j].x, in.x, y[tt][i].x);
+                y[tt][i].y = fmaf(w[j].y, in.y, y[tt][i].y);
+            }
+            if (RUN == 1 && c.single) {  // (t = 0: u[j] is what the state held at j, and the last is the token's own)
+#pragma unroll
+                for (int j = 1; j < kTaps; ++j) {
+                    if (TAPS == 0 && j >= taps) break;
+                    float* now = before + static_cast<size_t>(j - 1) * channels;
+                    now[0] = u[j].x;
+                    if (two) now[1] = u[j].y;
+                }
+            }
+            sum_sq[tt] += y[tt][i].x * y[tt][i].x + y[tt][i].y * y[tt][i].y;
+        }
+    }
+    const int page_mask = (1 << page_shift) - 1;
+    if (is_v) {
+        // a run of one sequence that lies in one page from a place that is a multiple of eight on
+        const bool together = RUN == 8 && sizeof(T) == 2 && count == RUN && of(my_seq, 0) == of(my_seq, RUN - 1) &&
+                              page_shift >= 3 && (of(my_pos, 0) & 7) == 0;
+#pragma unroll
+        for (int i = 0; i < CHUNKS; ++i) {
             const int d = 2 * lane + 128 * i;
             if (d >= padded) continue;
-            float x[2] = {y[i].x, y[i].y};
 #pragma unroll
-            for (int e = 0; e < 2; ++e) {
-                if (d + e < n) {
-                    if (c.first_out) c.first_out[at + d + e] = from_float<T>(x[e]);
-                    if (c.first_in) x[e] = (1.0f - c.mix) * x[e] + c.mix * to_float(c.first_in[at + d + e]);
+            for (int tt = 0; tt < RUN; ++tt) {
+                if (tt >= count) break;
+                const size_t at = (static_cast<size_t>(token0 + tt) * kv_heads + head) * vdim + d;
+                if (c.first_out) {
+                    if (d < n) c.first_out[at] = from_float<T>(y[tt][i].x);
+                    if (d + 1 < n) c.first_out[at + 1] = from_float<T>(y[tt][i].y);
                 }
-                dst[static_cast<size_t>(d + e) << page_shift] = from_float<T>(x[e]);
+                if (c.first_in) {
+                    if (d < n) y[tt][i].x = (1.0f - c.mix) * y[tt][i].x + c.mix * to_float(c.first_in[at]);
+                    if (d + 1 < n) y[tt][i].y = (1.0f - c.mix) * y[tt][i].y + c.mix * to_float(c.first_in[at + 1]);
+                }
+            }
+            if constexpr (RUN == 8 && sizeof(T) == 2) {
+                if (together) {
+                    T* dst = v_pool + (((static_cast<size_t>(of(my_page, 0)) * kv_heads + head) * DV + d) << page_shift) + (of(my_pos, 0) & page_mask);
+                    *reinterpret_cast<uint4*>(dst) = uint4{pack_bf16(y[0][i].x, y[1 % RUN][i].x), pack_bf16(y[2 % RUN][i].x, y[3 % RUN][i].x),
+                                                           pack_bf16(y[4 % RUN][i].x, y[5 % RUN][i].x), pack_bf16(y[6 % RUN][i].x, y[7 % RUN][i].x)};
+                    *reinterpret_cast<uint4*>(dst + (static_cast<size_t>(1) << page_shift)) =
+                        uint4{pack_bf16(y[0][i].y, y[1 % RUN][i].y), pack_bf16(y[2 % RUN][i].y, y[3 % RUN][i].y),
+                              pack_bf16(y[4 % RUN][i].y, y[5 % RUN][i].y), pack_bf16(y[6 % RUN][i].y, y[7 % RUN][i].y)};
+                    continue;
+                }
+            }
+#pragma unroll
+            for (int tt = 0; tt < RUN; ++tt) {
+                if (tt >= count) break;
+                T* dst = v_pool + (((static_cast<size_t>(of(my_page, tt)) * kv_heads + head) * DV + d) << page_shift) + (of(my_pos, tt) & page_mask);
+                dst[0] = from_float<T>(y[tt][i].x);
+                dst[static_cast<size_t>(1) << page_shift] = from_float<T>(y[tt][i].y);
             }
         }
         return;
     }
-    float factor = 1.f;
-    if (norm_mode != 0) factor = 1.0f / sqrtf(wave_sum(sum_sq) / static_cast<float>(dim) + eps);
     const float* weight = norm_mode == 2 ? (is_q ? q_weight : k_weight) : nullptr;
-    float after = 1.f;  // the queries' factor of the position
-    if (is_q && temp_every > 0) after = 1.0f + temp_coef * logf(static_cast<float>((pos + 1) / temp_every) + 1.0f);
+    float2 scale[CHUNKS];
 #pragma unroll
-    for (int i = 0; i < 2; ++i) {
+    for (int i = 0; i < CHUNKS; ++i) {
         const int d = 2 * lane + 128 * i;
-        if (d >= n) continue;
-        y[i].x *= factor * (weight ? weight[d] : 1.f);
-        y[i].y *= factor * (weight && d + 1 < n ? weight[d + 1] : 1.f);
-        if (rot > 0 && !neighbours) {
-            staged[wave][d] = y[i].x;
-            if (d + 1 < n) staged[wave][d + 1] = y[i].y;
-        }
+        scale[i] = float2{weight && d < n ? weight[d] : 1.f, weight && d + 1 < n ? weight[d + 1] : 1.f};
     }
-    __builtin_amdgcn_wave_barrier();  // (a wave's LDS operations keep their order; the compiler is held to it too)
-    T* dst = is_q ? q_out + (static_cast<size_t>(token) * q_heads + head) * D
-                  : k_pool + (((page * kv_heads + head) << page_shift) + in_page) * D;
     const int half = rot / 2;
-    const float* cos_row = rot > 0 ? cos_table + static_cast<size_t>(pos) * half : nullptr;
-    const float* sin_row = rot > 0 ? sin_table + static_cast<size_t>(pos) * half : nullptr;
+    if (norm_mode != 0) {  // (the tokens' sums side by side: their steps across the lanes do not wait for one another)
 #pragma unroll
-    for (int i = 0; i < 2; ++i) {
-        const int d = 2 * lane + 128 * i;
-        if (d >= padded) continue;
-        float2 x = y[i];
-        if (d < rot && neighbours) {  // (rot is even: a pair turns or stays as one)
-            const float cs = cos_row[d >> 1], sn = sin_row[d >> 1];
-            x = float2{y[i].x * cs - y[i].y * sn, y[i].y * cs + y[i].x * sn};
-        } else if (rot > 0 && d < rot) {
-            float turned[2] = {x.x, x.y};
+        for (int offset = kWave / 2; offset > 0; offset >>= 1)
 #pragma unroll
-            for (int e = 0; e < 2; ++e) {
-                const int at = d + e;
-                const bool is_u = at < half;
-                const float mate = staged[wave][is_u ? at + half : at - half];
-                const int angle = is_u ? at : at - half;
-                turned[e] = is_u ? turned[e] * cos_row[angle] - mate * sin_row[angle] : turned[e] * cos_row[angle] + mate * sin_row[angle];
+            for (int tt = 0; tt < RUN; ++tt) sum_sq[tt] += __shfl_xor(sum_sq[tt], offset, kWave);
+    }
+#pragma unroll
+    for (int tt = 0; tt < RUN; ++tt) {
+        if (tt >= count) break;
+        const int token = token0 + tt;
+        const int pos = of(my_pos, tt);
+        float factor = 1.f;
+        if (norm_mode != 0) factor = 1.0f / sqrtf(sum_sq[tt] / static_cast<float>(dim) + eps);
+        float after = 1.f;  // the queries' factor of the position
+        if (is_q && temp_every > 0) after = 1.0f + temp_coef * logf(static_cast<float>((pos + 1) / temp_every) + 1.0f);
+#pragma unroll
+        for (int i = 0; i < CHUNKS; ++i) {
+            const int d = 2 * lane + 128 * i;
+            y[tt][i].x *= factor * scale[i].x;
+            y[tt][i].y *= factor * scale[i].y;
+            if (rot > 0 && !neighbours) {
+                if (d < n) staged[wave][d] = y[tt][i].x;
+                if (d + 1 < n) staged[wave][d + 1] = y[tt][i].y;
             }
-            x = float2{turned[0], turned[1]};
         }
-        x.x *= after;
-        x.y *= after;
-        store_pair(dst + d, x);
+        __builtin_amdgcn_wave_barrier();  // (a wave's LDS operations keep their order; the compiler is held to it too)
+        T* dst = is_q ? q_out + (static_cast<size_t>(token) * q_heads + head) * D
+                      : k_pool + (((static_cast<size_t>(of(my_page, tt)) * kv_heads + head) << page_shift) + (pos & page_mask)) * D;
+        const float* cos_row = rot > 0 ? cos_table + static_cast<size_t>(pos) * half : nullptr;
+        const float* sin_row = rot > 0 ? sin_table + static_cast<size_t>(pos) * half : nullptr;
+#pragma unroll
+        for (int i = 0; i < CHUNKS; ++i) {
+            const int d = 2 * lane + 128 * i;
+            if (d >= padded) continue;
+            float2 x = y[tt][i];
+            if (d < rot && neighbours) {  // (rot is even: a pair turns or stays as one)
+                const float cs = cos_row[d >> 1], sn = sin_row[d >> 1];
+                x = float2{y[tt][i].x * cs - y[tt][i].y * sn, y[tt][i].y * cs + y[tt][i].x * sn};
+            } else if (d < rot) {
+                float turned[2] = {x.x, x.y};
+#pragma unroll
+                for (int e = 0; e < 2; ++e) {
+                    const int at = d + e;
+                    const bool is_u = at < half;
+                    const float mate = staged[wave][is_u ? at + half : at - half];
+                    const int angle = is_u ? at : at - half;
+                    turned[e] = is_u ? turned[e] * cos_row[angle] - mate * sin_row[angle] : turned[e] * cos_row[angle] + mate * sin_row[angle];
+                }
+                x = float2{turned[0], turned[1]};
+            }
+            x.x *= after;
+            x.y *= after;
+            store_pair(dst + d, x);
+        }
+        __builtin_amdgcn_wave_barrier();
     }
 }
 
@@ -901,6 +961,7 @@ scored_attention_mfma_kernel(ScoredArgs a) {
 // s (and s + 64, ...), so the common reference and every share's factor are known after one round of loads; the shares'
 // sums are then fetched without waiting on one another.
 constexpr int kMergeShares = 64;  // shares whose factors one pass keeps in a lane each
+constexpr int kMergeAhead = 8;    // shares whose sums are on their way at once
 
 template <int DV, int MAPS>
 __global__ void __launch_bounds__(256) scored_attention_merge_kernel(ScoredArgs a, int rows_per_tile) {
@@ -946,12 +1007,21 @@ __global__ void __launch_bounds__(256) scored_attention_merge_kernel(ScoredArgs 
                 den += ml[1] * mine;
             }
             const int count = min(kMergeShares, a.n_splits - base);
-            for (int sp = 0; sp < count; ++sp) {
-                const float f = __shfl(mine, sp, kWave);
-                const float* po = a.part_o + ((unit0 + base + sp) * rows_per_tile + at) * DV;
+            for (int sp0 = 0; sp0 < count; sp0 += kMergeAhead) {  // (the loads of that many shares travel together)
+                float v[kMergeAhead][N];
 #pragma unroll
-                for (int i = 0; i < N; ++i)
-                    if (lane + i * kWave < DV) acc[i] = fmaf(f == 0.f ? 0.f : po[lane + i * kWave], f, acc[i]);
+                for (int s = 0; s < kMergeAhead; ++s) {
+                    const float* po = a.part_o + ((unit0 + base + min(sp0 + s, count - 1)) * rows_per_tile + at) * DV;
+#pragma unroll
+                    for (int i = 0; i < N; ++i) v[s][i] = lane + i * kWave < DV ? po[lane + i * kWave] : 0.f;
+                }
+#pragma unroll
+                for (int s = 0; s < kMergeAhead; ++s) {
+                    // (0 past the last share, and for a share without keys, whose sums nobody wrote)
+                    const float f = sp0 + s < count ? __shfl(mine, sp0 + s, kWave) : 0.f;
+#pragma unroll
+                    for (int i = 0; i < N; ++i) acc[i] = fmaf(f == 0.f ? 0.f : v[s][i], f, acc[i]);
+                }
             }
         }
         const float inverse = 1.0f / (wave_sum(den) + sink_term);
@@ -1023,7 +1093,8 @@ CIE_API int cie_heads_prepare(void* stream, int dtype, const void* proj, int pro
     return cie_after_launch();
 }
 
-// The preparation behind a convolution (see heads_conv_prepare_kernel).  norm_mode 0, 1 or 2; heads of up to 256 numbers.
+// The preparation behind a convolution (see heads_conv_prepare_kernel).  norm_mode 0, 1 or 2; heads of up to 256 numbers;
+// `run` 1, or 8 (2 to 4 taps): tokens that a wave takes.
 CIE_API int cie_heads_conv_prepare(void* stream, int dtype, const void* proj, int proj_stride, int q_off, int k_off,
                                    int v_off, const void* taps, int n_taps, float* past, const int* q_start_loc, int single,
                                    void* first_out, const void* first_in, float mix, const float* q_weight,
@@ -1031,7 +1102,7 @@ CIE_API int cie_heads_conv_prepare(void* stream, int dtype, const void* proj, in
                                    const int* positions, const int* seq_of_token, const int* seq_slot,
                                    const int* block_table, int table_width, void* q_out, void* k_pool, void* v_pool,
                                    int tokens, int q_heads, int kv_heads, int dim, int vdim, int D, int DV, int page_size,
-                                   const float* cos_table, const float* sin_table, int rot, int neighbours) {
+                                   const float* cos_table, const float* sin_table, int rot, int neighbours, int run) {
     if (rot < 0 || rot % 2 || rot > dim || (rot > 0 && (!cos_table || !sin_table))) return CIE_BAD_ARGUMENT;
     if (tokens < 0 || q_heads <= 0 || kv_heads <= 0 || dim <= 0 || vdim <= 0 || D < dim || DV < vdim || D > 256 || DV > 256 ||
         D % 2 || DV % 2 || page_size <= 0 || (page_size & (page_size - 1)) || table_width <= 0 || norm_mode < 0 ||
@@ -1042,27 +1113,39 @@ CIE_API int cie_heads_conv_prepare(void* stream, int dtype, const void* proj, in
     if (tokens == 0) return CIE_OK;
     int page_shift = 0;
     while ((1 << page_shift) < page_size) ++page_shift;
-    const long blocks = (static_cast<long>(tokens) * (q_heads + 2 * kv_heads) + 3) / 4;
+    if (single && run != 1) return CIE_BAD_ARGUMENT;
+    if (run != 1 && (run != 8 || n_taps < 2 || n_taps > 4)) return CIE_BAD_ARGUMENT;
+    const long blocks = (static_cast<long>((tokens + run - 1) / run) * (q_heads + 2 * kv_heads) + 3) / 4;
     if (blocks > 0x7fffffffL) return CIE_BAD_ARGUMENT;
+    const int chunks = (D > 128 || DV > 128) ? 2 : 1;
     hipStream_t s = static_cast<hipStream_t>(stream);
-#define CIE_CONV_HEADS(T, TAPS)                                                                                          \
-    heads_conv_prepare_kernel<T, TAPS><<<static_cast<unsigned>(blocks), 256, 0, s>>>(                                    \
+#define CIE_CONV_HEADS(T, TAPS, RUN, CHUNKS)                                                                             \
+    heads_conv_prepare_kernel<T, TAPS, RUN, CHUNKS><<<static_cast<unsigned>(blocks), 256, 0, s>>>(                       \
         static_cast<const T*>(proj), proj_stride, q_off, k_off, v_off,                                                   \
         ConvHeads<T>{static_cast<const T*>(taps), n_taps, past, q_start_loc, single, static_cast<T*>(first_out),         \
                      static_cast<const T*>(first_in), mix},                                                              \
         q_weight, k_weight, norm_mode, eps, temp_coef, temp_every, positions, seq_of_token, seq_slot, block_table,       \
         table_width, static_cast<T*>(q_out), static_cast<T*>(k_pool), static_cast<T*>(v_pool), tokens, q_heads, kv_heads, \
         dim, vdim, D, DV, page_shift, cos_table, sin_table, rot, neighbours)
-#define CIE_CONV_HEADS_TYPE(T)                     \
-    do {                                           \
-        if (n_taps == 2) CIE_CONV_HEADS(T, 2);     \
-        else if (n_taps == 3) CIE_CONV_HEADS(T, 3); \
-        else if (n_taps == 4) CIE_CONV_HEADS(T, 4); \
-        else CIE_CONV_HEADS(T, 0);                 \
+#define CIE_CONV_HEADS_CHUNKS(T, TAPS, RUN)                \
+    do {                                                   \
+        if (chunks == 1) CIE_CONV_HEADS(T, TAPS, RUN, 1);  \
+        else CIE_CONV_HEADS(T, TAPS, RUN, 2);              \
+    } while (0)
+#define CIE_CONV_HEADS_TYPE(T)                                     \
+    do {                                                           \
+        if (n_taps == 2 && run == 1) CIE_CONV_HEADS_CHUNKS(T, 2, 1);      \
+        else if (n_taps == 3 && run == 1) CIE_CONV_HEADS_CHUNKS(T, 3, 1); \
+        else if (n_taps == 4 && run == 1) CIE_CONV_HEADS_CHUNKS(T, 4, 1); \
+        else if (n_taps == 2 && run == 8) CIE_CONV_HEADS_CHUNKS(T, 2, 8); \
+        else if (n_taps == 3 && run == 8) CIE_CONV_HEADS_CHUNKS(T, 3, 8); \
+        else if (n_taps == 4 && run == 8) CIE_CONV_HEADS_CHUNKS(T, 4, 8); \
+        else CIE_CONV_HEADS_CHUNKS(T, 0, 1);                              \
     } while (0)
     if (dtype == CIE_F32) CIE_CONV_HEADS_TYPE(float);
     else if (dtype == CIE_BF16) CIE_CONV_HEADS_TYPE(bf16_t);
     else return CIE_BAD_ARGUMENT;
+#undef CIE_CONV_HEADS_CHUNKS
 #undef CIE_CONV_HEADS_TYPE
 #undef CIE_CONV_HEADS
     return cie_after_launch();

@@ -1822,6 +1822,92 @@ def gated_token_rows(z: torch.Tensor, table: torch.Tensor, column: int, ids: tor
     return out
 
 
+def _token_table(table: torch.Tensor, column: int, dim: int, ids: torch.Tensor, tokens: int, dtype: torch.dtype) -> None:
+    _gpu("table", table, dtype, 2)
+    _gpu("ids", ids, torch.int32, 1)
+    if column < 0 or column + dim > table.shape[1] or ids.shape[0] < tokens:
+        raise ValueError(f"columns {column} .. {column + dim} of a table of {table.shape[1]}, {ids.shape[0]} ids for {tokens} rows")
+
+
+def weight_pieces(weight: torch.Tensor) -> torch.Tensor:
+    """A weight [N, K] as the kernels of the token table's branch read it: pieces of 16 rows and 32 columns (zeros past either
+    end), each as the 64 lanes of a matrix product hold it, [ceil(N / 16), ceil(K / 32), 64, 8]."""
+    n, k = weight.shape
+    wide = weight.new_zeros((-(-n // 16) * 16, -(-k // 32) * 32))
+    wide[:n, :k] = weight
+    return (wide.reshape(wide.shape[0] // 16, 16, wide.shape[1] // 32, 4, 8).permute(0, 2, 3, 1, 4)
+            .reshape(wide.shape[0] // 16, wide.shape[1] // 32, 64, 8).contiguous())
+
+
+def _check_pieces(name: str, pieces: torch.Tensor, n: int, k: int) -> None:
+    _gpu(name, pieces, torch.bfloat16, 4)
+    if tuple(pieces.shape) != (-(-n // 16), -(-k // 32), 64, 8) or pieces.data_ptr() % 16:
+        raise ValueError(f"{name} {tuple(pieces.shape)} are not the pieces of a [{n}, {k}] weight")
+
+
+def token_gate(stream: torch.Tensor, gate: torch.Tensor, dim: int, table: torch.Tensor, column: int,
+               ids: torch.Tensor) -> torch.Tensor:
+    """``gelu_tanh(stream @ W_gate.T) * table[ids, column : column + dim]`` in one kernel for few rows: ``stream`` float32
+    [T, hidden] (rounded to bf16 on its way into the product), ``gate`` the pieces (:func:`weight_pieces`) of the bf16 weight
+    [dim, hidden], hidden a multiple of 8."""
+    _gpu("stream", stream, torch.float32, 2)
+    tokens, hidden = stream.shape
+    _check_pieces("gate", gate, dim, hidden)
+    if hidden % 8 or stream.data_ptr() % 16:
+        raise ValueError(f"rows of {hidden} numbers: a multiple of 8")
+    _token_table(table, column, dim, ids, tokens, torch.bfloat16)
+    out = torch.empty((tokens, dim), dtype=torch.bfloat16, device=stream.device)
+    _run("cie_token_gate", load_library().cie_token_gate(
+        _stream(), _ptr(stream), _ptr(gate), _ptr(table), table.shape[1], _i(column), _ptr(ids), _ptr(out), _i(tokens), _i(hidden),
+        _i(dim), _i(table.shape[0])))
+    return out
+
+
+def plan_token_side(hidden: int, dim: int) -> int:
+    """Shares of the width that :func:`token_side` cuts its first product into; 0: sizes that it does not take."""
+    if hidden % 8 or not 8 <= hidden <= 4096 or dim < 1:
+        return 0
+    tiles, shares = -(-dim // 16), 1
+    while tiles * shares * 2 <= 16:
+        shares *= 2
+    bytes_ = 16 * (-(-hidden // 32) * 32 + 8) * 2 + shares * 16 * tiles * 16 * 4 + 16 * (-(-dim // 32) * 32 + 8) * 2
+    return shares if bytes_ <= 160 * 1024 else 0
+
+
+def token_side(stream: torch.Tensor, branch: Optional[torch.Tensor], gate: torch.Tensor, proj: torch.Tensor, dim: int,
+               table: torch.Tensor, column: int, ids: torch.Tensor, weight: torch.Tensor, eps: float,
+               next_weight: Optional[torch.Tensor] = None) -> Optional[torch.Tensor]:
+    """``x = stream + branch``; ``g = gelu_tanh(x @ W_gate.T) * table[ids, column : column + dim]``; ``y = g @ W_proj.T``;
+    ``stream <- x + y / sqrt(mean(y^2) + eps) * weight``, in one kernel for many rows (sizes that :func:`plan_token_side`
+    takes): ``stream`` float32 [T, hidden] in place, ``branch`` bf16 or ``None``, ``gate`` and ``proj`` the pieces
+    (:func:`weight_pieces`) of the bf16 weights [dim, hidden] and [hidden, dim].  With ``next_weight`` (float32 [hidden]) the
+    RMS norm of the new stream under it comes back in bf16."""
+    _gpu("stream", stream, torch.float32, 2)
+    tokens, hidden = stream.shape
+    shares = plan_token_side(hidden, dim)
+    if not shares or not eps > 0:
+        raise ValueError(f"rows of {hidden} with {dim} columns of the table (eps {eps}) are not what this kernel takes")
+    _check_pieces("gate", gate, dim, hidden)
+    _check_pieces("proj", proj, hidden, dim)
+    if stream.data_ptr() % 16:
+        raise ValueError("operands must be 16-byte aligned")
+    if branch is not None:
+        _gpu("branch", branch, torch.bfloat16, 2)
+        if branch.shape != stream.shape or branch.data_ptr() % 16:
+            raise ValueError(f"branch {tuple(branch.shape)} vs stream {tuple(stream.shape)}")
+    for name, w in (("weight", weight), ("next_weight", next_weight)):
+        if w is not None:
+            _gpu(name, w, torch.float32, 1)
+            if w.shape[0] != hidden or w.data_ptr() % 16:
+                raise ValueError(f"{name} must be [{hidden}], is {tuple(w.shape)}")
+    _token_table(table, column, dim, ids, tokens, torch.bfloat16)
+    normed = torch.empty((tokens, hidden), dtype=torch.bfloat16, device=stream.device) if next_weight is not None else None
+    _run("cie_token_side", load_library().cie_token_side(
+        _stream(), _ptr(stream), _ptr(branch), _ptr(gate), _ptr(proj), _ptr(table), table.shape[1], _i(column), _ptr(ids),
+        _ptr(weight), _ptr(next_weight), _ptr(normed), _i(tokens), _i(hidden), _i(dim), _i(table.shape[0]), _f(eps), _i(shares)))
+    return normed
+
+
 def stream_rows(residual: torch.Tensor, branch: Optional[torch.Tensor], branch2: Optional[torch.Tensor],
                 out_dtype: torch.dtype, want_rows: bool = True) -> Optional[torch.Tensor]:
     """``residual += branch + branch2`` (whichever are given; float32, in place), and the new stream in ``out_dtype``."""
@@ -1947,6 +2033,8 @@ def heads_prepare(proj: torch.Tensor, offsets: tuple[int, int, int], q_heads: in
 
 
 MAX_CONV_HEAD = 256        # numbers of a head that passes a convolution
+CONV_HEADS_RUN = 8         # tokens that a wave of that kernel takes ...
+CONV_HEADS_RUN_FROM = 512  # ... in steps of at least this many
 
 
 def heads_conv_prepare(proj: torch.Tensor, offsets: tuple[int, int, int], q_heads: int, kv_heads: int, dim: int, vdim: int,
@@ -1956,14 +2044,15 @@ def heads_conv_prepare(proj: torch.Tensor, offsets: tuple[int, int, int], q_head
                        temperature: Optional[tuple[float, int]], positions: torch.Tensor, seq_of_token: torch.Tensor,
                        seq_slot: torch.Tensor, block_table: torch.Tensor, k_pool: torch.Tensor, v_pool: torch.Tensor,
                        rotary: Optional[tuple] = None, first_out: Optional[torch.Tensor] = None,
-                       first_in: Optional[torch.Tensor] = None, mix: float = 0.0) -> torch.Tensor:
+                       first_in: Optional[torch.Tensor] = None, mix: float = 0.0, run: Optional[int] = None) -> torch.Tensor:
     """What :func:`heads_prepare` does (``norm``: ``None``, ``"unit"`` or ``"weight"``; one map a head; keys and values are
     always written), for projections that first pass a causal convolution over each sequence's tokens, channel by
     channel: ``taps_w`` [(q_heads + kv_heads) * dim + kv_heads * vdim, n] in ``proj``'s dtype, its last tap meeting the
     token itself (``None``: no convolution).  ``past`` (float32 [slots, max(n - 1, 1), channels], oldest first) holds each
     request's last inputs; they are moved on by the step's inputs.  ``single``: every sequence of the step brings one token.
     The values may be mixed: ``first_out`` ([T, kv_heads * vdim]) takes them as convolved; with ``first_in`` (another
-    layer's) they become ``(1 - mix) * v + mix * first_in`` before they are cached."""
+    layer's) they become ``(1 - mix) * v + mix * first_in`` before they are cached.  ``run``: tokens that a wave of the kernel
+    takes, 1 or 8."""
     if not (proj.is_cuda and proj.dim() == 2 and proj.stride(1) == 1 and proj.dtype in _CODES):
         raise ValueError("proj must be a float32 or bfloat16 GPU matrix with unit inner stride")
     dtype, tokens = proj.dtype, proj.shape[0]
@@ -2012,6 +2101,8 @@ def heads_conv_prepare(proj: torch.Tensor, offsets: tuple[int, int, int], q_head
                 raise ValueError(f"{name} must be {(tokens, kv_heads * vdim)}, is {tuple(t.shape)}")
     coef, every = temperature if temperature else (0.0, 0)
     cos, sin, rot, neighbours = _check_rotary(rotary, dim)
+    if run is None:
+        run = CONV_HEADS_RUN if not single and 2 <= taps <= 4 and tokens >= CONV_HEADS_RUN_FROM else 1
     q_out = torch.empty((tokens, q_heads * kernel_dim), dtype=dtype, device=proj.device)
     _run("cie_heads_conv_prepare", load_library().cie_heads_conv_prepare(
         _stream(), _i(_code(dtype)), _ptr(proj), _i(_ld(proj)), _i(q_off), _i(k_off), _i(v_off), _ptr(taps_w), _i(taps),
@@ -2019,7 +2110,7 @@ def heads_conv_prepare(proj: torch.Tensor, offsets: tuple[int, int, int], q_head
         _ptr(q_weight), _ptr(k_weight), _i(NORM_MODES[norm]), _f(eps), _f(coef), _i(every), _ptr(positions), _ptr(seq_of_token),
         _ptr(seq_slot), _ptr(block_table), _i(block_table.shape[1]), _ptr(q_out), _ptr(k_pool), _ptr(v_pool), _i(tokens),
         _i(q_heads), _i(kv_heads), _i(dim), _i(vdim), _i(kernel_dim), _i(kernel_vdim), _i(page_size), _ptr(cos), _ptr(sin),
-        _i(rot), _i(1 if neighbours else 0)))
+        _i(rot), _i(1 if neighbours else 0), _i(run)))
     if taps > 1 and not single:
         conv_keep(proj[:, q_off: q_off + channels], past, seq_slot, q_start_loc, sequences, taps)
     return q_out

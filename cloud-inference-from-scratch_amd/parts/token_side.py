@@ -4,7 +4,9 @@
 table, ``y = W_proj (gelu_tanh(W_gate x) * e)``, and y joins the stream under an RMS norm of its own with a weight:
 ``x += y / sqrt(mean(y^2) + eps) * w``.  Layer i's part are the columns ``i * dim .. (i + 1) * dim - 1``.  The table is the
 model's (``ModelSpec.side_table_columns``); the step's batch carries it together with the tokens as the embedding took
-them.  The stream, the norm and the gate are float32; the two products run in the engine's type.
+them.  The stream, the norm and the gate are float32; the two products run in the engine's type.  In bfloat16 few rows take a
+kernel for everything up to ``gelu_tanh(W_gate x) * e``, many rows one kernel for all of it, the add of the layer's other
+branches and the next layer's norm included (``csrc/token_side.hip``).
 """
 
 from __future__ import annotations
@@ -17,6 +19,13 @@ from ..kernels import ops
 from ..weights.tensors import TensorSpec
 from .base import Part, register_part
 from .linear import Added, RowSumsq, WeightedPair, linear
+
+# Rows from which one kernel does all of it, a workgroup to sixteen rows, and up to which the gate's product, the gate and
+# the lookup are one kernel (all of the branch for a table part of 256, us, one kernel / few rows / in parts: width 2,048 at
+# 16 rows 33 / 18 / 19, at 64 35 / 19 / 34, at 256 35 / 26 / 29, at 512 35 / 34 / 34, at 2,048 41 / 72 / 51; width 3,584 at 512
+# rows 60 / 51 / 45, at 1,024 60 / 75 / 54, at 2,048 62 / 117 / 71)
+WHOLE_FROM_ROWS = 512
+FEW_ROWS = 511
 
 
 class TokenSide(Part):
@@ -41,6 +50,12 @@ class TokenSide(Part):
         gate, proj, norm = self.names
         self.w_gate, self.w_proj = tensors[prefix + gate].contiguous(), tensors[prefix + proj].contiguous()
         self.weight = tensors[prefix + norm].float().contiguous()
+        # the weights once more, as the kernels of this branch alone read them
+        self.gate_pieces = self.proj_pieces = None
+        if dtype == torch.bfloat16 and self.hidden_size % 8 == 0:
+            self.gate_pieces = ops.weight_pieces(self.w_gate)
+            if ops.plan_token_side(self.hidden_size, self.dim):
+                self.proj_pieces = ops.weight_pieces(self.w_proj)
 
     def warm_up(self, rows: int) -> None:
         blank = lambda width: torch.zeros((rows, width), dtype=self.dtype, device=self.device)
@@ -59,9 +74,18 @@ class TokenSide(Part):
             first = pending.combined()
         elif pending is not None and not isinstance(pending, (Added, RowSumsq)):
             first = pending
-        rows = ops.stream_rows(residual, first, second, dtype, want_rows=dtype != torch.float32)
-        z = linear(residual if rows is None else rows, self.w_gate, out_dtype=torch.float32)
-        y = linear(ops.gated_token_rows(z, table, self.column, ids), self.w_proj)
+        tokens = residual.shape[0]
+        if self.proj_pieces is not None and tokens >= WHOLE_FROM_ROWS and second is None:
+            return ops.token_side(residual, first, self.gate_pieces, self.proj_pieces, self.dim, table, self.column, ids, self.weight, self.eps,
+                                  next_weight=None if then is None else then.weight_f32)
+        few = self.gate_pieces is not None and tokens <= FEW_ROWS
+        rows = ops.stream_rows(residual, first, second, dtype, want_rows=dtype != torch.float32 and not few)
+        if few:
+            gated = ops.token_gate(residual, self.gate_pieces, self.dim, table, self.column, ids)
+        else:
+            z = linear(residual if rows is None else rows, self.w_gate, out_dtype=torch.float32)
+            gated = ops.gated_token_rows(z, table, self.column, ids)
+        y = linear(gated, self.w_proj)
         made = ops.branch_norm_add(residual, y, self.weight, self.eps, dtype, want_rows=False,
                                    next_weight=None if then is None else then.weight_f32)
         return None if then is None else made[1]

@@ -100,7 +100,7 @@ def test_the_token_table_at_other_widths(width, side):
     kernel takes at a time, for few rows and for many."""
     raw = gu.single(attention(2, 1, 16, 16, 3, 0.4, 13, ff=40), latent(2, 8, 4, 8, 16, 24, 0.4), width=width, side=side)
     weights = gu.make_weights(raw, seed=width)
-    requests = {"a": random_tokens(150, raw["vocab"], 1), "b": random_tokens(33, raw["vocab"], 2), "c": [7]}
+    requests = {"a": random_tokens(530, raw["vocab"], 1), "b": random_tokens(33, raw["vocab"], 2), "c": [7]}
     plain = plain_all(raw, weights, requests)
     for dtype in ("float32", "bfloat16"):
         run_and_compare(raw, weights, requests, replay_util.whole(requests), dtype, plain)
@@ -518,7 +518,7 @@ TOL = {torch.float32: dict(atol=2e-5, rtol=2e-5), torch.bfloat16: dict(atol=4e-2
 @pytest.mark.parametrize("pairing", ["neighbours", "halves"])
 @pytest.mark.parametrize("shape", [(2, 1, 16, 24, 3), (3, 3, 9, 5, 2), (4, 2, 128, 64, 4), (2, 1, 136, 256, 1), (1, 1, 40, 8, 7),
                                    (2, 2, 200, 33, 16), (2, 1, 24, 16, None)])
-def test_heads_behind_a_convolution(shape, pairing, dtype):
+def test_heads_behind_a_convolution(shape, pairing, dtype, run=None):
     """Convolution, norm, rotation, cache write and the values' mean, for portions of unequal length behind inputs that
     earlier steps left, in slots that are not in order; then single tokens."""
     from cie_amd.kernels import ops
@@ -536,7 +536,8 @@ def test_heads_behind_a_convolution(shape, pairing, dtype):
     taps_w = None if taps is None else (torch.randn(channels, taps, generator=g) * 0.7).to(dtype)
     keep = max((taps or 1) - 1, 1)
     mix = 0.3
-    for lengths, starts, slots in (([5, 1, 40, 2], [9, 0, 16, 70], [2, 0, 3, 1]), ([1, 1, 1], [31, 0, 64], [1, 3, 0])):
+    for lengths, starts, slots in (([5, 1, 40, 2], [9, 0, 16, 70], [2, 0, 3, 1]), ([1, 1, 1], [31, 0, 64], [1, 3, 0]),
+                                   ([33, 24], [8, 0], [3, 0])):
         tokens, single = sum(lengths), max(lengths) == 1
         table = torch.randperm(4 * pages, generator=g).reshape(4, pages).int()
         proj = torch.randn(tokens, channels + 8, generator=g).to(dtype)
@@ -551,7 +552,8 @@ def test_heads_behind_a_convolution(shape, pairing, dtype):
         q = ops.heads_conv_prepare(proj.cuda(), offsets, heads, kv, dim, vdim, D, DV, None if taps_w is None else taps_w.cuda(),
                                    past, q_start_loc, len(lengths), single, "weight", q_weight.cuda(), k_weight.cuda(), 1e-4, None,
                                    _ints(positions), seq_of_token, _ints(slots), table.cuda(), k_pool, v_pool,
-                                   rotary=(cos, sin, rot, pairing == "neighbours"), first_out=first_out, first_in=first_in.cuda(), mix=mix)
+                                   rotary=(cos, sin, rot, pairing == "neighbours"), first_out=first_out, first_in=first_in.cuda(), mix=mix,
+                                   run=None if single else run)
         at = 0
         written = 0
         for length, start, slot in zip(lengths, starts, slots):
@@ -588,6 +590,14 @@ def test_heads_behind_a_convolution(shape, pairing, dtype):
         untouched = [s for s in range(5) if s not in slots]
         assert torch.equal(past[untouched].cpu(), past0[untouched])
         assert int((k_pool[:, 0, :, 0] != 7.0).sum()) <= written and int((v_pool[:, 0, 0] != 7.0).sum()) <= written
+
+
+@pytest.mark.parametrize("dtype", [torch.float32, torch.bfloat16])
+@pytest.mark.parametrize("pairing", ["neighbours", "halves"])
+@pytest.mark.parametrize("shape", [(2, 1, 16, 24, 3), (3, 3, 9, 5, 2), (4, 2, 128, 64, 4), (2, 1, 136, 256, 3)])
+def test_heads_behind_a_convolution_in_runs_of_eight_tokens(shape, pairing, dtype):
+    """The form for many tokens, whose waves take eight tokens each: runs that cross sequences, pages and the last token."""
+    test_heads_behind_a_convolution(shape, pairing, dtype, run=8)
 
 
 @pytest.mark.parametrize("dtype", [torch.float32, torch.bfloat16])
@@ -662,3 +672,43 @@ def test_a_product_for_two_readers(rows, sizes):
         assert tuple(got.shape) == (rows, split) and torch.allclose(got.double().cpu(), want[:, :split], **TOL[dtype])
         assert torch.allclose(out[:, 8: 8 + inner].double().cpu(), pg.squared_relu(want[:, split:]), **TOL[dtype])
         assert float((out[:, :8] - 5.0).abs().sum()) == 0.0 and float((out[:, 8 + inner:] - 5.0).abs().sum()) == 0.0
+
+
+@pytest.mark.parametrize("sizes", [(64, 8), (192, 16), (256, 40), (264, 136), (2048, 256), (520, 520), (3584, 256), (1000, 24), (40, 9)])
+def test_the_token_tables_branch_in_one_kernel_and_in_parts(sizes):
+    """The kernel for few rows and the one for many against the equations, at widths and table parts on both sides of their
+    tiles, with and without a branch still to be added and a norm behind."""
+    from cie_amd.kernels import ops
+
+    hidden, dim = sizes
+    g = torch.Generator().manual_seed(hidden + dim)
+    table = torch.randn(20, 3 * dim, generator=g).to(torch.bfloat16)
+    gate = (torch.randn(dim, hidden, generator=g) * 1.5 / hidden ** 0.5).to(torch.bfloat16)
+    proj = (torch.randn(hidden, dim, generator=g) / dim ** 0.5).to(torch.bfloat16)
+    weight, after = torch.rand(hidden, generator=g) + 0.5, torch.rand(hidden, generator=g) + 0.5
+    assert ops.plan_token_side(hidden, dim) >= 1
+    gate_pieces, proj_pieces = ops.weight_pieces(gate.cuda()), ops.weight_pieces(proj.cuda())
+    for tokens, with_branch, with_norm in ((1, True, True), (37, False, True), (300, True, True), (64, True, False)):
+        x = torch.randn(tokens, hidden, generator=g) * 2
+        branch = torch.randn(tokens, hidden, generator=g).to(torch.bfloat16)
+        ids = torch.randint(0, 20, (tokens,), generator=g).int()
+        total = x.double() + (branch.double() if with_branch else 0.0)
+        stream = x.clone().cuda()
+        got = ops.token_side(stream, branch.cuda() if with_branch else None, gate_pieces, proj_pieces, dim, table.cuda(), dim, ids.cuda(),
+                             weight.cuda(), 1e-3, next_weight=after.cuda() if with_norm else None)
+        e = table.double()[ids.long(), dim: 2 * dim]
+        # (rounded where the kernel rounds: the norm brings out what rounding leaves of a row that nearly cancels)
+        rough = lambda t: t.to(torch.bfloat16).double()
+        y = rough(rough(pg.gelu_tanh(rough(total.float()) @ gate.double().t()) * e) @ proj.double().t())
+        want = total + pg.rms_norm(y, weight.double(), 1e-3)
+        assert torch.allclose(stream.double().cpu(), want, atol=4e-2, rtol=1e-2), float((stream.double().cpu() - want).abs().max())
+        if dim > 32:
+            exact = total + pg.token_side(total, e, gate.double(), proj.double(), weight.double(), 1e-3)
+            assert float((stream.double().cpu() - exact).pow(2).mean().sqrt()) < 2e-2
+        assert (got is None) == (not with_norm)
+        if with_norm:
+            assert torch.allclose(got.double().cpu(), pg.rms_norm(want, after.double(), 1e-3), atol=5e-2, rtol=2e-2)
+        few = ops.token_gate(x.cuda(), gate_pieces, dim, table.cuda(), dim, ids.cuda())
+        rounded = x.to(torch.bfloat16).double()
+        assert torch.allclose(few.double().cpu(), pg.gelu_tanh(rounded @ gate.double().t()) * e, atol=2e-2, rtol=1e-2)
+    assert ops.plan_token_side(50, 8) == ops.plan_token_side(8192, 256) == 0
