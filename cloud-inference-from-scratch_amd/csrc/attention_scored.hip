@@ -165,7 +165,7 @@ heads_prepare_kernel(const T* __restrict__ proj, int proj_stride, int q_off, int
 }
 
 // The same preparation for heads whose projections first pass a causal convolution over the tokens, channel by channel:
-//   y_t = sum_j taps[c, j] u_(t - n + 1 + j)   (the last tap meets the token itself),
+//   y_t = sum_j taps[j, c] u_(t - n + 1 + j)   (the last tap meets the token itself),
 // with the inputs of the tokens before the step in `past` [slots, max(n - 1, 1), channels] (float32, oldest first; the
 // channels are those of the queries, the keys and the values in that order), and for values that are mixed with those
 // that an earlier layer of the same step made of the same tokens:
@@ -173,7 +173,7 @@ heads_prepare_kernel(const T* __restrict__ proj, int proj_stride, int q_off, int
 // A layer that is the first of those leaves its convolved values in `first_out`.
 template <typename T>
 struct ConvHeads {
-    const T* taps;         // [channels, n]; null: the projection as it is (n = 1)
+    const T* taps;         // [n, channels]; null: the projection as it is (n = 1)
     int n;
     float* past;
     const int* q_start_loc;
@@ -235,6 +235,7 @@ heads_conv_prepare_kernel(const T* __restrict__ proj, int proj_stride, int q_off
     const int channel = is_v ? (q_heads + kv_heads) * dim + head * vdim : (is_q ? 0 : q_heads * dim) + head * dim;
     const int taps = TAPS > 0 ? TAPS : c.n;
     const bool paired = (((proj_stride | column | n) & 1) == 0);  // (the base of `proj` is aligned to a pair)
+    const bool paired_channels = (((channels | channel | n) & 1) == 0);
     // lane i knows the place of the run's token i
     const int mine = token0 + min(lane, count - 1);
     const int my_pos = positions[mine];
@@ -243,6 +244,22 @@ heads_conv_prepare_kernel(const T* __restrict__ proj, int proj_stride, int q_off
     const int my_first = c.q_start_loc[my_seq];
     const int my_page = is_q ? 0 : block_table[static_cast<size_t>(my_slot) * table_width + (my_pos >> page_shift)];
     auto of = [&](int value, int tt) { return __builtin_amdgcn_readlane(value, tt); };
+
+    // what the steps behind the convolution need from memory is asked for in front of it: single tokens wait for one round
+    // of loads instead of three
+    const float* weight = norm_mode == 2 && !is_v ? (is_q ? q_weight : k_weight) : nullptr;
+    const int half = rot / 2;
+    float2 scale[CHUNKS], turn[CHUNKS];  // (`turn`: runs of one token only)
+#pragma unroll
+    for (int i = 0; i < CHUNKS; ++i) {
+        const int d = 2 * lane + 128 * i;
+        scale[i] = float2{weight && d < n ? weight[d] : 1.f, weight && d + 1 < n ? weight[d + 1] : 1.f};
+        turn[i] = float2{1.f, 0.f};
+        if (RUN == 1 && neighbours && !is_v && d < rot) {
+            const size_t at = static_cast<size_t>(of(my_pos, 0)) * half + (d >> 1);
+            turn[i] = float2{cos_table[at], sin_table[at]};
+        }
+    }
 
     float2 y[RUN][CHUNKS];
     float sum_sq[RUN];
@@ -266,21 +283,19 @@ heads_conv_prepare_kernel(const T* __restrict__ proj, int proj_stride, int q_off
 #pragma unroll
         for (int j = 0; j < kTaps; ++j) {
             if (TAPS == 0 && j >= taps) break;
-            const T* at = c.taps + static_cast<size_t>(channel + d) * taps + j;
-            w[j] = c.taps ? float2{to_float(at[0]), two ? to_float(at[taps]) : 0.f} : float2{1.f, 1.f};
+            w[j] = c.taps ? load_pair(c.taps + static_cast<size_t>(j) * channels + channel, d, n, paired_channels) : float2{1.f, 1.f};
         }
 #pragma unroll
         for (int tt = 0; tt < RUN; ++tt) {
             if (tt >= count) break;
             const int t = token0 + tt - of(my_first, tt);  // the token's place in the step's portion of its sequence
-            float* before = c.past + static_cast<size_t>(of(my_slot, tt)) * max(taps - 1, 1) * channels + channel + d;
+            float* before = c.past + static_cast<size_t>(of(my_slot, tt)) * max(taps - 1, 1) * channels + channel;
 #pragma unroll
             for (int j = 0; j < kTaps; ++j) {
                 if (TAPS == 0 && j >= taps) break;
                 float2 in = u[tt + j];
                 if (t - (taps - 1) + j < 0) {  // (in front of the portion: what earlier steps left)
-                    const float* old = before + static_cast<size_t>(t + j) * channels;
-                    in = float2{old[0], two ? old[1] : 0.f};
+                    in = load_pair(before + static_cast<size_t>(t + j) * channels, d, n, paired_channels);
                     if (RUN == 1) u[j] = in;
                 }
                 y[tt][i].x = fmaf(w[j].x, in.x, y[tt][i].x);
@@ -290,9 +305,13 @@ heads_conv_prepare_kernel(const T* __restrict__ proj, int proj_stride, int q_off
 #pragma unroll
                 for (int j = 1; j < kTaps; ++j) {
                     if (TAPS == 0 && j >= taps) break;
-                    float* now = before + static_cast<size_t>(j - 1) * channels;
-                    now[0] = u[j].x;
-                    if (two) now[1] = u[j].y;
+                    float* now = before + static_cast<size_t>(j - 1) * channels + d;
+                    if (paired_channels) {
+                        store_pair(now, u[j]);
+                    } else {
+                        now[0] = u[j].x;
+                        if (two) now[1] = u[j].y;
+                    }
                 }
             }
             sum_sq[tt] += y[tt][i].x * y[tt][i].x + y[tt][i].y * y[tt][i].y;
@@ -341,14 +360,6 @@ heads_conv_prepare_kernel(const T* __restrict__ proj, int proj_stride, int q_off
         }
         return;
     }
-    const float* weight = norm_mode == 2 ? (is_q ? q_weight : k_weight) : nullptr;
-    float2 scale[CHUNKS];
-#pragma unroll
-    for (int i = 0; i < CHUNKS; ++i) {
-        const int d = 2 * lane + 128 * i;
-        scale[i] = float2{weight && d < n ? weight[d] : 1.f, weight && d + 1 < n ? weight[d + 1] : 1.f};
-    }
-    const int half = rot / 2;
     if (norm_mode != 0) {  // (the tokens' sums side by side: their steps across the lanes do not wait for one another)
 #pragma unroll
         for (int offset = kWave / 2; offset > 0; offset >>= 1)
@@ -385,7 +396,7 @@ heads_conv_prepare_kernel(const T* __restrict__ proj, int proj_stride, int q_off
             if (d >= padded) continue;
             float2 x = y[tt][i];
             if (d < rot && neighbours) {  // (rot is even: a pair turns or stays as one)
-                const float cs = cos_row[d >> 1], sn = sin_row[d >> 1];
+                const float cs = RUN == 1 ? turn[i].x : cos_row[d >> 1], sn = RUN == 1 ? turn[i].y : sin_row[d >> 1];
                 x = float2{y[tt][i].x * cs - y[tt][i].y * sn, y[tt][i].y * cs + y[tt][i].x * sn};
             } else if (d < rot) {
                 float turned[2] = {x.x, x.y};

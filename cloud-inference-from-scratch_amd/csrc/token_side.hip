@@ -212,20 +212,27 @@ __global__ void __launch_bounds__(64 * kSideWaves) token_side_kernel(SideArgs a)
     __syncthreads();
 
     // z = rows * gate^T: a wave takes one tile of 16 columns over one share of the width (several, for a wide table part)
+    // (The workgroups of an XCD go through the same weights at the same time: each begins at a place of its own, so that most
+    // pieces have been brought into the XCD's L2 by another one when they are asked for.)
     const int column_tiles = at.dim16 / 16, slices = at.hidden32 / 32;
+    const int first_slice = static_cast<int>((blockIdx.x / 8) * 8 % slices);
     for (int item = wave; item < column_tiles * a.k_shares; item += kSideWaves) {
         const int tile = item % column_tiles, share = item / column_tiles;
         floatx4 acc = {0.f, 0.f, 0.f, 0.f};
         constexpr int U = 8;
         for (int s0 = share; s0 < slices; s0 += U * a.k_shares) {
             uint4 w[U];
-#pragma unroll
-            for (int u = 0; u < U; ++u) w[u] = *piece(a.gate, tile, slices, min(s0 + u * a.k_shares, slices - 1), lane);
+            int slice[U];
 #pragma unroll
             for (int u = 0; u < U; ++u) {
-                const int slice = s0 + u * a.k_shares;
-                const uint4 x = *reinterpret_cast<const uint4*>(rows_s + r * row_stride + min(slice, slices - 1) * 32 + g * 8);
-                acc = mfma16(slice < slices ? x : uint4{0u, 0u, 0u, 0u}, w[u], acc);
+                slice[u] = min(s0 + u * a.k_shares, slices - 1) + first_slice;
+                if (slice[u] >= slices) slice[u] -= slices;
+                w[u] = *piece(a.gate, tile, slices, slice[u], lane);
+            }
+#pragma unroll
+            for (int u = 0; u < U; ++u) {
+                const uint4 x = *reinterpret_cast<const uint4*>(rows_s + r * row_stride + slice[u] * 32 + g * 8);
+                acc = mfma16(s0 + u * a.k_shares < slices ? x : uint4{0u, 0u, 0u, 0u}, w[u], acc);
             }
         }
 #pragma unroll
@@ -247,7 +254,7 @@ __global__ void __launch_bounds__(64 * kSideWaves) token_side_kernel(SideArgs a)
         floatx4 y[kTiles];
 #pragma unroll
         for (int t = 0; t < kTiles; ++t) y[t] = floatx4{0.f, 0.f, 0.f, 0.f};
-        for (int s = 0; s < y_slices; ++s) {
+        for (int s0 = 0, s = static_cast<int>((blockIdx.x / 8) % y_slices); s0 < y_slices; ++s0, s = s + 1 < y_slices ? s + 1 : 0) {
             uint4 w[kTiles];
 #pragma unroll
             for (int t = 0; t < kTiles; ++t) w[t] = *piece(a.proj, min(t0 + t, y_tiles - 1), y_slices, s, lane);

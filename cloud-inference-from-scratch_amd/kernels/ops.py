@@ -2034,7 +2034,7 @@ def heads_prepare(proj: torch.Tensor, offsets: tuple[int, int, int], q_heads: in
 
 MAX_CONV_HEAD = 256        # numbers of a head that passes a convolution
 CONV_HEADS_RUN = 8         # tokens that a wave of that kernel takes ...
-CONV_HEADS_RUN_FROM = 512  # ... in steps of at least this many
+CONV_HEADS_RUN_FROM = 768  # ... in steps of at least this many
 
 
 def heads_conv_prepare(proj: torch.Tensor, offsets: tuple[int, int, int], q_heads: int, kv_heads: int, dim: int, vdim: int,
@@ -2047,7 +2047,7 @@ def heads_conv_prepare(proj: torch.Tensor, offsets: tuple[int, int, int], q_head
                        first_in: Optional[torch.Tensor] = None, mix: float = 0.0, run: Optional[int] = None) -> torch.Tensor:
     """What :func:`heads_prepare` does (``norm``: ``None``, ``"unit"`` or ``"weight"``; one map a head; keys and values are
     always written), for projections that first pass a causal convolution over each sequence's tokens, channel by
-    channel: ``taps_w`` [(q_heads + kv_heads) * dim + kv_heads * vdim, n] in ``proj``'s dtype, its last tap meeting the
+    channel: ``taps_w`` [n, (q_heads + kv_heads) * dim + kv_heads * vdim] in ``proj``'s dtype, its last tap meeting the
     token itself (``None``: no convolution).  ``past`` (float32 [slots, max(n - 1, 1), channels], oldest first) holds each
     request's last inputs; they are moved on by the step's inputs.  ``single``: every sequence of the step brings one token.
     The values may be mixed: ``first_out`` ([T, kv_heads * vdim]) takes them as convolved; with ``first_in`` (another
@@ -2075,8 +2075,8 @@ def heads_conv_prepare(proj: torch.Tensor, offsets: tuple[int, int, int], q_head
     taps = 1
     if taps_w is not None:
         _gpu("taps_w", taps_w, dtype, 2)
-        taps = taps_w.shape[1]
-        if taps_w.shape[0] != channels or not 1 <= taps <= MAX_CONV_TAPS:
+        taps = taps_w.shape[0]
+        if taps_w.shape[1] != channels or not 1 <= taps <= MAX_CONV_TAPS:
             raise ValueError(f"taps {tuple(taps_w.shape)} for {channels} channels (up to {MAX_CONV_TAPS} taps)")
     if taps > 1:
         if past is None:

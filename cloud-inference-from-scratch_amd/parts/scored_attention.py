@@ -223,7 +223,7 @@ class ScoredAttention(Part):
                 self.k_weight = tensors[prefix + "k.norm"].float().contiguous()
         self.taps_w, self.mix_weight = None, 0.0
         if self.conv_taps is not None:
-            self.taps_w = torch.cat([tensors[f"{prefix}{name}.conv"] for name in ("q", "k", "v")], dim=0).contiguous()
+            self.taps_w = torch.cat([tensors[f"{prefix}{name}.conv"] for name in ("q", "k", "v")], dim=0).t().contiguous()
         if self.value_mix == "mixed":
             self.mix_weight = float(tensors[prefix + "vmix"].float().item())
         self.pair = None  # what joins the two maps of a head: lambda, the factor behind the norm, its eps

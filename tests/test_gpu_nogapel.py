@@ -100,7 +100,7 @@ def test_the_token_table_at_other_widths(width, side):
     kernel takes at a time, for few rows and for many."""
     raw = gu.single(attention(2, 1, 16, 16, 3, 0.4, 13, ff=40), latent(2, 8, 4, 8, 16, 24, 0.4), width=width, side=side)
     weights = gu.make_weights(raw, seed=width)
-    requests = {"a": random_tokens(530, raw["vocab"], 1), "b": random_tokens(33, raw["vocab"], 2), "c": [7]}
+    requests = {"a": random_tokens(800, raw["vocab"], 1), "b": random_tokens(33, raw["vocab"], 2), "c": [7]}
     plain = plain_all(raw, weights, requests)
     for dtype in ("float32", "bfloat16"):
         run_and_compare(raw, weights, requests, replay_util.whole(requests), dtype, plain)
@@ -549,7 +549,7 @@ def test_heads_behind_a_convolution(shape, pairing, dtype, run=None):
         q_start_loc, seq_of_token = _meta(lengths)
         positions = [s + t for s, n in zip(starts, lengths) for t in range(n)]
         offsets = (0, heads * dim, (heads + kv) * dim)
-        q = ops.heads_conv_prepare(proj.cuda(), offsets, heads, kv, dim, vdim, D, DV, None if taps_w is None else taps_w.cuda(),
+        q = ops.heads_conv_prepare(proj.cuda(), offsets, heads, kv, dim, vdim, D, DV, None if taps_w is None else taps_w.t().contiguous().cuda(),
                                    past, q_start_loc, len(lengths), single, "weight", q_weight.cuda(), k_weight.cuda(), 1e-4, None,
                                    _ints(positions), seq_of_token, _ints(slots), table.cuda(), k_pool, v_pool,
                                    rotary=(cos, sin, rot, pairing == "neighbours"), first_out=first_out, first_in=first_in.cuda(), mix=mix,
