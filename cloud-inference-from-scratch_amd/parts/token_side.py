@@ -66,6 +66,9 @@ class TokenSide(Part):
                 then: Any = None) -> Optional[torch.Tensor]:
         """``residual`` (float32, in place) takes what is pending and then this part's own branch; ``then``: an RMS norm of
         one group under which the new stream's rows come back."""
+        if then is not None and then.eps != self.eps:  # (the kernels have one eps for both norms)
+            self.forward(residual, pending, batch, dtype)
+            return then.forward(residual, None, dtype)
         table, ids = batch.carried["side_table"], batch.carried["token_ids"]
         first = second = None
         if isinstance(pending, WeightedPair) and pending.scales == (1.0, 1.0):
@@ -76,8 +79,8 @@ class TokenSide(Part):
             first = pending
         tokens = residual.shape[0]
         if self.proj_pieces is not None and tokens >= WHOLE_FROM_ROWS and second is None:
-            return ops.token_side(residual, first, self.gate_pieces, self.proj_pieces, self.dim, table, self.column, ids, self.weight, self.eps,
-                                  next_weight=None if then is None else then.weight_f32)
+            return ops.token_side(residual, first, self.gate_pieces, self.proj_pieces, self.dim, table, self.column, ids,
+                                  self.weight, self.eps, next_weight=None if then is None else then.weight_f32)
         few = self.gate_pieces is not None and tokens <= FEW_ROWS
         rows = ops.stream_rows(residual, first, second, dtype, want_rows=dtype != torch.float32 and not few)
         if few:
